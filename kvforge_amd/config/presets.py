@@ -319,6 +319,64 @@ PRESETS["ludelix-1b"] = ludelix_stack(vocab=128256, width=2048, groups=4, heads=
                                       shared_ff=2048)
 
 
+def balalorn(vocab: int, width: int, layers: list, eps: float = 1e-5,
+             max_positions: int | None = None) -> dict[str, Any]:
+    """A Balalorn config.json.  ``layers``: one ``(type, mixer, mlp)`` per layer.  For ``"mamba2"`` the mixer
+    holds ``heads vdim state groups norm_groups conv``; for ``"delta"`` ``heads kv_heads dim vdim conv``; for
+    ``"latent_attention"`` ``heads dim rot_dim vdim kv_rank scale`` and optionally ``base`` and ``kv_from``.
+    ``mlp``: ``None``, an ``int`` (a dense feed-forward of that width) or ``(ff, experts, top)``."""
+    out = []
+    for kind, m, mlp in layers:
+        mixer = dict(m)
+        if kind == "latent_attention":
+            base = mixer.pop("base", 10000.0)
+            mixer["rot"] = {"base": float(base), "dims": m["rot_dim"]} if m["rot_dim"] else None
+        if isinstance(mlp, int):
+            ff: dict[str, Any] | None = {"ff": mlp, "kind": "dense"}
+        else:
+            ff = ({"expert": {"ff": mlp[0]}, "kind": "moe", "router": {"experts": mlp[1], "top": mlp[2]}}
+                  if mlp else None)
+        out.append({"mixer": mixer, "mlp": ff, "type": kind})
+    cfg: dict[str, Any] = {"architecture": "Balalorn", "layers": out, "norm": {"eps": eps}, "vocab": vocab,
+                           "width": width}
+    if max_positions is not None:
+        cfg["max_positions"] = max_positions
+    return cfg
+
+
+def balalorn_stack(vocab: int, width: int, groups: int, heads: int, latent_dim: int, rot_dim: int, kv_rank: int,
+                   mem_heads: int, mem_kv_heads: int, mem_dim: int, mem_vdim: int, ssm_heads: int, ssm_vdim: int,
+                   state: int, ssm_groups: int, ff: int, moe_ff: int, experts: int, top: int,
+                   max_positions: int = 131072) -> dict[str, Any]:
+    """``groups`` times (delta with a dense feed-forward, latent attention with experts, mamba2 with
+    experts, latent attention over the same latents with a dense feed-forward)."""
+    delta = dict(heads=mem_heads, kv_heads=mem_kv_heads, dim=mem_dim, vdim=mem_vdim, conv=4)
+    ssm = dict(heads=ssm_heads, vdim=ssm_vdim, state=state, groups=ssm_groups, norm_groups=ssm_groups, conv=4)
+    lat = dict(heads=heads, dim=latent_dim, rot_dim=rot_dim, vdim=latent_dim, kv_rank=kv_rank,
+               scale=float(latent_dim + rot_dim) ** -0.5, base=1000000.0)
+    moe = (moe_ff, experts, top)
+    layers: list = []
+    for g in range(groups):
+        layers += [("delta", delta, ff), ("latent_attention", lat, moe), ("mamba2", ssm, moe),
+                   ("latent_attention", dict(lat, kv_from=4 * g + 1), ff)]
+    return balalorn(vocab, width, layers, max_positions=max_positions)
+
+
+PRESETS["balalorn-tiny"] = balalorn(
+    vocab=304, width=96,
+    layers=[("mamba2", dict(heads=4, vdim=24, state=16, groups=2, norm_groups=3, conv=3), (32, 6, 2)),
+            ("latent_attention", dict(heads=3, dim=16, rot_dim=8, vdim=24, kv_rank=40, scale=0.2), 160),
+            ("delta", dict(heads=4, kv_heads=2, dim=24, vdim=16, conv=4), None),
+            ("latent_attention", dict(heads=2, dim=24, rot_dim=8, vdim=16, kv_rank=40, scale=0.25, kv_from=1),
+             (32, 4, 1))],
+    max_positions=1024)
+# layers of the width of llama-1b: what this design's kernels are measured at
+PRESETS["balalorn-1b"] = balalorn_stack(
+    vocab=128256, width=2048, groups=4, heads=32, latent_dim=64, rot_dim=32, kv_rank=192, mem_heads=16, mem_kv_heads=8,
+    mem_dim=128, mem_vdim=128, ssm_heads=64, ssm_vdim=64, state=128, ssm_groups=8, ff=8192, moe_ff=1024, experts=32,
+    top=4)
+
+
 def preset_dict(name: str) -> dict[str, Any]:
     try:
         return dict(PRESETS[name])

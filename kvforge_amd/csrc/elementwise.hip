@@ -1151,6 +1151,7 @@ KVF_EXPORT int kvf_token_side_bf16(TOKEN_SIDE_DECL) {
 //   settle_cast: x[m] += bias + owed[m] (either may be null); copy[m] = x[m] in T (copy may be null)
 //   side_gate:   g[m, j] = gelu_tanh(a[m, j]) * side[token[m], col0 + j]
 //   rms_add:     x[m] += y[m] * rsqrt(mean(y[m]^2) + eps) * w
+//   rms_add_cast: the same, and out[m] = x[m] (the new x, rounded to out's type)
 //   rms_add_norm: the same, and out[m] = x[m] * rsqrt(mean(x[m]^2) + eps2) * w2 of the new x
 template <typename T, typename D>
 __global__ void settle_cast_kernel(float* __restrict__ x, const float* __restrict__ bias,
@@ -1231,6 +1232,89 @@ KVF_EXPORT int kvf_rms_add(float* x, const float* y, const float* w, float eps, 
   if (m <= 0) return 0;
   hipLaunchKernelGGL(rms_add_kernel, dim3(m), dim3(256), 0, s, x, y, w, eps, h);
   return kvf_last_error();
+}
+
+// A sublayer's rows join the stream through their norm, and the next sublayer reads the stream itself:
+// one pass over the row for the sum and its copy in the sublayers' type.  Q > 0: rows of a multiple of
+// four and at most 1024 Q elements, which a thread then holds in registers, four neighbours a load.
+template <typename T, int Q>
+__global__ __launch_bounds__(256) void rms_add_cast_kernel(float* __restrict__ x, const float* __restrict__ y,
+                                                           const float* __restrict__ w, float eps,
+                                                           T* __restrict__ out, int h) {
+  __shared__ float scratch[16];
+  const int m = blockIdx.x;
+  float* xr = x + static_cast<size_t>(m) * h;
+  const float* yr = y + static_cast<size_t>(m) * h;
+  T* o = out + static_cast<size_t>(m) * h;
+  if (Q > 0) {
+    constexpr int N = Q > 0 ? Q : 1;
+    float4 yv[N], xv[N], wv[N];
+    float ss = 0.f;
+#pragma unroll
+    for (int k = 0; k < N; ++k) {
+      const int i = 4 * (k * 256 + threadIdx.x);
+      yv[k] = xv[k] = wv[k] = make_float4(0.f, 0.f, 0.f, 0.f);
+      if (i < h) {
+        yv[k] = *reinterpret_cast<const float4*>(yr + i);
+        xv[k] = *reinterpret_cast<const float4*>(xr + i);
+        wv[k] = *reinterpret_cast<const float4*>(w + i);
+      }
+    }
+#pragma unroll
+    for (int k = 0; k < N; ++k)
+      ss = fmaf(yv[k].x, yv[k].x, fmaf(yv[k].y, yv[k].y, fmaf(yv[k].z, yv[k].z, fmaf(yv[k].w, yv[k].w, ss))));
+    const float r = rsqrtf(block_sum(ss, scratch) / static_cast<float>(h) + eps);
+#pragma unroll
+    for (int k = 0; k < N; ++k) {
+      const int i = 4 * (k * 256 + threadIdx.x);
+      if (i >= h) continue;
+      float4 v;
+      v.x = fmaf(yv[k].x * r, wv[k].x, xv[k].x);
+      v.y = fmaf(yv[k].y * r, wv[k].y, xv[k].y);
+      v.z = fmaf(yv[k].z * r, wv[k].z, xv[k].z);
+      v.w = fmaf(yv[k].w * r, wv[k].w, xv[k].w);
+      *reinterpret_cast<float4*>(xr + i) = v;
+      if (sizeof(T) == 4) {
+        *reinterpret_cast<float4*>(o + i) = v;
+      } else {
+        uint2 p;
+        p.x = static_cast<uint32_t>(f32_to_bf16(v.x)) | (static_cast<uint32_t>(f32_to_bf16(v.y)) << 16);
+        p.y = static_cast<uint32_t>(f32_to_bf16(v.z)) | (static_cast<uint32_t>(f32_to_bf16(v.w)) << 16);
+        *reinterpret_cast<uint2*>(o + i) = p;
+      }
+    }
+    return;
+  }
+  float ss = 0.f;
+  for (int i = threadIdx.x; i < h; i += blockDim.x) ss = fmaf(yr[i], yr[i], ss);
+  const float r = rsqrtf(block_sum(ss, scratch) / static_cast<float>(h) + eps);
+  for (int i = threadIdx.x; i < h; i += blockDim.x) {
+    const float v = fmaf(yr[i] * r, w[i], xr[i]);
+    xr[i] = v;
+    Elem<T>::store(o + i, v);
+  }
+}
+template <typename T>
+static int rms_add_cast_launch(float* x, const float* y, const float* w, float eps, void* out, int m, int h,
+                               hipStream_t s) {
+  const bool vec = h % 4 == 0 && reinterpret_cast<uintptr_t>(x) % 16 == 0 && reinterpret_cast<uintptr_t>(y) % 16 == 0 &&
+                   reinterpret_cast<uintptr_t>(w) % 16 == 0 && reinterpret_cast<uintptr_t>(out) % 16 == 0;
+  T* o = static_cast<T*>(out);
+  if (vec && h <= 1024)
+    hipLaunchKernelGGL((rms_add_cast_kernel<T, 1>), dim3(m), dim3(256), 0, s, x, y, w, eps, o, h);
+  else if (vec && h <= 4096)
+    hipLaunchKernelGGL((rms_add_cast_kernel<T, 4>), dim3(m), dim3(256), 0, s, x, y, w, eps, o, h);
+  else
+    hipLaunchKernelGGL((rms_add_cast_kernel<T, 0>), dim3(m), dim3(256), 0, s, x, y, w, eps, o, h);
+  return kvf_last_error();
+}
+// dtype of out: 0 = fp32, 1 = bf16
+KVF_EXPORT int kvf_rms_add_cast(int dtype, float* x, const float* y, const float* w, float eps, void* out, int m, int h,
+                                hipStream_t s) {
+  if (m <= 0) return 0;
+  if (dtype == 0) return rms_add_cast_launch<float>(x, y, w, eps, out, m, h, s);
+  if (dtype == 1) return rms_add_cast_launch<bf16_t>(x, y, w, eps, out, m, h, s);
+  return static_cast<int>(hipErrorInvalidValue);
 }
 
 // A sublayer's rows join the stream through their norm, and the next sublayer's input is the norm

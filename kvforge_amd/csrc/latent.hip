@@ -10,12 +10,14 @@
 //   latent_split : a projected row [q heads (dim | rot) ... | c_raw (rank) | k_r (rot)] becomes
 //                  the attention kernels' row [H q heads | k | v] of heads of d elements:
 //                  q head h = [q_r_h | (left for head_product) | 0], k = [k_r | norm(c) | 0],
-//                  v = [0 | norm(c) | 0]; the norm in fp32 with one rounding.
+//                  v = [0 | norm(c) | 0]; the norm in fp32 with one rounding.  Without a norm
+//                  weight the row holds the q heads alone (attention over another layer's keys).
 //   head_product : out[n, h, :] = W[h] in[n, h, :] for per-head matrices W [H, O, I].  bf16 rows and
 //                  weights whose heads start on 16 bytes go to the matrix cores (a workgroup
 //                  per 64 rows x 64 outputs of a head, a wave per 16 outputs, operands straight
 //                  from memory, fp32 sums); everything else is fp32 multiply and add on the
-//                  vector ALUs, tiles of 32 rows x 64 outputs through LDS.
+//                  vector ALUs, tiles of 32 rows x 64 outputs through LDS.  With `gate` (rows of
+//                  one number per head) what is stored is the product times sigmoid(gate[n, h]).
 #include "common.h"
 
 namespace {
@@ -30,12 +32,15 @@ __global__ __launch_bounds__(256) void latent_split_kernel(const T* __restrict__
   const T* in = proj + static_cast<size_t>(n) * ld_in;
   T* out = qkv + static_cast<size_t>(n) * ld_out;
   const T* down = in + H * (dim + rot);
-  float ss = 0.f;
-  for (int i = tid; i < rank; i += blockDim.x) {
-    const float v = Elem<T>::load(down + i);
-    ss = fmaf(v, v, ss);
+  float r = 0.f;
+  if (w != nullptr) {   // the same for the whole grid
+    float ss = 0.f;
+    for (int i = tid; i < rank; i += blockDim.x) {
+      const float v = Elem<T>::load(down + i);
+      ss = fmaf(v, v, ss);
+    }
+    r = 1.f / sqrtf(block_sum(ss, scratch) / static_cast<float>(rank) + eps);
   }
-  const float r = 1.f / sqrtf(block_sum(ss, scratch) / static_cast<float>(rank) + eps);
   // q heads: the rotated part to the front, zeros behind what head_product fills
   for (int i = tid; i < H * d; i += blockDim.x) {
     const int h = i / d, e = i - h * d;
@@ -44,6 +49,7 @@ __global__ __launch_bounds__(256) void latent_split_kernel(const T* __restrict__
     else if (e >= rot + rank || dim == 0)   // (heads without a plain part: nothing fills the middle)
       Elem<T>::store(out + i, 0.f);
   }
+  if (w == nullptr) return;
   T* k = out + H * d;
   T* v = k + d;
   for (int e = tid; e < d; e += blockDim.x) {
@@ -61,6 +67,10 @@ __global__ __launch_bounds__(256) void latent_split_kernel(const T* __restrict__
   }
 }
 
+template <typename T> __device__ __forceinline__ float gate_of(const T* gate, int ld_gate, int n, int h) {
+  return gate ? 1.f / (1.f + expf(-Elem<T>::load(gate + static_cast<size_t>(n) * ld_gate + h))) : 1.f;
+}
+
 constexpr int HP_M = 32, HP_N = 64, HP_K = 32;
 
 // grid (row tiles, output tiles, heads); 256 threads, thread (ty, tx) owns rows ty, ty + 16 and
@@ -68,7 +78,8 @@ constexpr int HP_M = 32, HP_N = 64, HP_K = 32;
 template <typename T, typename TW>
 __global__ __launch_bounds__(256) void head_product_kernel(const T* __restrict__ in, int ld_in, int in_head,
                                                            const TW* __restrict__ W, T* __restrict__ out,
-                                                           int ld_out, int out_head, int N, int O, int I) {
+                                                           int ld_out, int out_head, int N, int O, int I,
+                                                           const T* __restrict__ gate, int ld_gate) {
   __shared__ float As[HP_M][HP_K + 1];
   __shared__ float Bs[HP_N][HP_K + 1];
   const int n0 = blockIdx.x * HP_M, o0 = blockIdx.y * HP_N, h = blockIdx.z;
@@ -103,9 +114,10 @@ __global__ __launch_bounds__(256) void head_product_kernel(const T* __restrict__
     const int n = n0 + ty + 16 * i;
     if (n >= N) continue;
     T* o = out + static_cast<size_t>(n) * ld_out + static_cast<size_t>(h) * out_head;
+    const float g = gate_of(gate, ld_gate, n, h);
 #pragma unroll
     for (int j = 0; j < 4; ++j)
-      if (o0 + tx + 16 * j < O) Elem<T>::store(o + o0 + tx + 16 * j, acc[i][j]);
+      if (o0 + tx + 16 * j < O) Elem<T>::store(o + o0 + tx + 16 * j, acc[i][j] * g);
   }
 }
 
@@ -137,7 +149,8 @@ __device__ __forceinline__ void store4(bf16_t* o, const f32x4& a, int left, bool
 __global__ __launch_bounds__(256) void head_product_mfma_kernel(const bf16_t* __restrict__ in, int ld_in,
                                                                 int in_head, const bf16_t* __restrict__ W,
                                                                 bf16_t* __restrict__ out, int ld_out, int out_head,
-                                                                int N, int O, int I, bool wide) {
+                                                                int N, int O, int I, bool wide,
+                                                                const bf16_t* __restrict__ gate, int ld_gate) {
   const int n0 = blockIdx.x * 64, h = blockIdx.z;
   const int lane = threadIdx.x % KVF_WAVE, wave = threadIdx.x / KVF_WAVE;
   const int j = lane % 16, c = lane / 16;
@@ -176,7 +189,7 @@ __global__ __launch_bounds__(256) void head_product_mfma_kernel(const bf16_t* __
     const int n = n0 + 16 * r + j;
     if (r >= subs || n >= N) continue;
     bf16_t* o = out + static_cast<size_t>(n) * ld_out + static_cast<size_t>(h) * out_head + o0 + 4 * c;
-    store4(o, acc[r], O - (o0 + 4 * c), wide);
+    store4(o, acc[r] * gate_of(gate, ld_gate, n, h), O - (o0 + 4 * c), wide);
   }
 }
 
@@ -188,7 +201,8 @@ template <int KS>
 __global__ __launch_bounds__(256) void head_product_mfma_rows_kernel(const bf16_t* __restrict__ in, int ld_in,
                                                                      int in_head, const bf16_t* __restrict__ W,
                                                                      bf16_t* __restrict__ out, int ld_out,
-                                                                     int out_head, int N, int O, int I, bool wide) {
+                                                                     int out_head, int N, int O, int I, bool wide,
+                                                                     const bf16_t* __restrict__ gate, int ld_gate) {
   const int n0 = blockIdx.x * 64, h = blockIdx.y;
   const int lane = threadIdx.x % KVF_WAVE, wave = threadIdx.x / KVF_WAVE;
   const int j = lane % 16, c = lane / 16;
@@ -206,6 +220,9 @@ __global__ __launch_bounds__(256) void head_product_mfma_rows_kernel(const bf16_
       if (x && 32 * s + 8 * c + 8 <= I) xf[s][r] = *reinterpret_cast<const uint4*>(x + 32 * s);
     }
   }
+  float gv[4];
+#pragma unroll
+  for (int r = 0; r < 4; ++r) gv[r] = (r < subs && n0 + 16 * r + j < N) ? gate_of(gate, ld_gate, n0 + 16 * r + j, h) : 1.f;
   const int groups = (O + 15) / 16;
   for (int g = wave; g < groups; g += 4) {
     const int o0 = 16 * g;
@@ -231,27 +248,28 @@ __global__ __launch_bounds__(256) void head_product_mfma_rows_kernel(const bf16_
       const int n = n0 + 16 * r + j;
       if (r >= subs || n >= N) continue;
       bf16_t* o = out + static_cast<size_t>(n) * ld_out + static_cast<size_t>(h) * out_head + o0 + 4 * c;
-      store4(o, acc[r], O - (o0 + 4 * c), wide);
+      store4(o, acc[r] * gv[r], O - (o0 + 4 * c), wide);
     }
   }
 }
 
 template <typename T, typename TW>
 int head_product_launch(const void* in, int ld_in, int in_head, const void* W, void* out, int ld_out,
-                        int out_head, int N, int H, int O, int I, hipStream_t s) {
+                        int out_head, int N, int H, int O, int I, const void* gate, int ld_gate, hipStream_t s) {
   const dim3 grid((N + HP_M - 1) / HP_M, (O + HP_N - 1) / HP_N, H);
   hipLaunchKernelGGL((head_product_kernel<T, TW>), grid, dim3(256), 0, s, static_cast<const T*>(in), ld_in, in_head,
-                     static_cast<const TW*>(W), static_cast<T*>(out), ld_out, out_head, N, O, I);
+                     static_cast<const TW*>(W), static_cast<T*>(out), ld_out, out_head, N, O, I,
+                     static_cast<const T*>(gate), ld_gate);
   return kvf_last_error();
 }
 }  // namespace
 
-// dtype: 0 = fp32, 1 = bf16 (rows in and out).  d >= rot + rank.
+// dtype: 0 = fp32, 1 = bf16 (rows in and out).  d >= rot + rank.  w null: q heads alone.
 KVF_EXPORT int kvf_latent_split(int dtype, const void* proj, int ld_in, void* qkv, int ld_out, const float* w,
                                 float eps, int n, int H, int dim, int rot, int rank, int d, hipStream_t s) {
   if (n <= 0) return 0;
-  if (H <= 0 || dim < 0 || rot < 0 || rank <= 0 || d < rot + rank || ld_in < H * (dim + rot) + rank + rot ||
-      ld_out < (H + 2) * d || !w)
+  if (H <= 0 || dim < 0 || rot < 0 || rank <= 0 || d < rot + rank || ld_in < H * (dim + rot) + (w ? rank + rot : 0) ||
+      ld_out < (H + (w ? 2 : 0)) * d)
     return static_cast<int>(hipErrorInvalidValue);
   if (dtype == 0)
     hipLaunchKernelGGL(latent_split_kernel<float>, dim3(n), dim3(256), 0, s, static_cast<const float*>(proj), ld_in,
@@ -268,43 +286,44 @@ KVF_EXPORT int kvf_latent_split(int dtype, const void* proj, int ld_in, void* qk
 // and wtype of W: 0 = fp32, 1 = bf16.
 KVF_EXPORT int kvf_head_product(int dtype, int wtype, const void* in, int ld_in, int in_head, const void* W,
                                 void* out, int ld_out, int out_head, int N, int H, int O, int I,
-                                hipStream_t s) {
+                                const void* gate, int ld_gate, hipStream_t s) {
   if (N <= 0) return 0;
-  if (H <= 0 || O <= 0 || I <= 0 || H > 65535 || (O + HP_N - 1) / HP_N > 65535)
+  if (H <= 0 || O <= 0 || I <= 0 || H > 65535 || (O + HP_N - 1) / HP_N > 65535 || (gate && N > 1 && ld_gate < H))
     return static_cast<int>(hipErrorInvalidValue);
   if (dtype == 1 && wtype == 1 && I % 8 == 0 && in_head % 8 == 0 && ld_in % 8 == 0 &&
       reinterpret_cast<uintptr_t>(in) % 16 == 0 && reinterpret_cast<uintptr_t>(W) % 16 == 0) {
     const bf16_t* x = static_cast<const bf16_t*>(in);
     const bf16_t* w = static_cast<const bf16_t*>(W);
     bf16_t* y = static_cast<bf16_t*>(out);
+    const bf16_t* gt = static_cast<const bf16_t*>(gate);
     const dim3 rows((N + 63) / 64, H);
     const bool wide = ld_out % 4 == 0 && out_head % 4 == 0 && reinterpret_cast<uintptr_t>(out) % 8 == 0;
     if (N < 256 || I > 256) {   // few rows: more workgroups, each with one tile of outputs
       const dim3 grid((N + 63) / 64, (O + 63) / 64, H);
       hipLaunchKernelGGL(head_product_mfma_kernel, grid, dim3(256), 0, s, x, ld_in, in_head, w, y, ld_out, out_head, N,
-                         O, I, wide);
+                         O, I, wide, gt, ld_gate);
     } else if (I <= 64) {
       hipLaunchKernelGGL(head_product_mfma_rows_kernel<2>, rows, dim3(256), 0, s, x, ld_in, in_head, w, y, ld_out,
-                         out_head, N, O, I, wide);
+                         out_head, N, O, I, wide, gt, ld_gate);
     } else if (I <= 128) {
       hipLaunchKernelGGL(head_product_mfma_rows_kernel<4>, rows, dim3(256), 0, s, x, ld_in, in_head, w, y, ld_out,
-                         out_head, N, O, I, wide);
+                         out_head, N, O, I, wide, gt, ld_gate);
     } else if (I <= 192) {
       hipLaunchKernelGGL(head_product_mfma_rows_kernel<6>, rows, dim3(256), 0, s, x, ld_in, in_head, w, y, ld_out,
-                         out_head, N, O, I, wide);
+                         out_head, N, O, I, wide, gt, ld_gate);
     } else {
       hipLaunchKernelGGL(head_product_mfma_rows_kernel<8>, rows, dim3(256), 0, s, x, ld_in, in_head, w, y, ld_out,
-                         out_head, N, O, I, wide);
+                         out_head, N, O, I, wide, gt, ld_gate);
     }
     return kvf_last_error();
   }
   if (dtype == 0 && wtype == 0)
-    return head_product_launch<float, float>(in, ld_in, in_head, W, out, ld_out, out_head, N, H, O, I, s);
+    return head_product_launch<float, float>(in, ld_in, in_head, W, out, ld_out, out_head, N, H, O, I, gate, ld_gate, s);
   if (dtype == 1 && wtype == 1)
-    return head_product_launch<bf16_t, bf16_t>(in, ld_in, in_head, W, out, ld_out, out_head, N, H, O, I, s);
+    return head_product_launch<bf16_t, bf16_t>(in, ld_in, in_head, W, out, ld_out, out_head, N, H, O, I, gate, ld_gate, s);
   if (dtype == 1 && wtype == 0)
-    return head_product_launch<bf16_t, float>(in, ld_in, in_head, W, out, ld_out, out_head, N, H, O, I, s);
+    return head_product_launch<bf16_t, float>(in, ld_in, in_head, W, out, ld_out, out_head, N, H, O, I, gate, ld_gate, s);
   if (dtype == 0 && wtype == 1)
-    return head_product_launch<float, bf16_t>(in, ld_in, in_head, W, out, ld_out, out_head, N, H, O, I, s);
+    return head_product_launch<float, bf16_t>(in, ld_in, in_head, W, out, ld_out, out_head, N, H, O, I, gate, ld_gate, s);
   return static_cast<int>(hipErrorInvalidValue);
 }

@@ -6,13 +6,14 @@ namespace {
 constexpr int MAX_PER_LANE = 8;   // router outputs per lane: up to 512 of them
 constexpr int MAX_TOP = 16;
 
-// A wave per token.  s = softmax(z) over all R router outputs; the `top` outputs with the
-// largest s + correction are chosen (the lowest index among equals), and weighted by their s
-// alone, divided by the sum of the chosen s (+ 1e-20).  sel [N, top], wgt [N, top].
+// A wave per token.  s = softmax(z) over all R router outputs, or (`sigmoid`) s = sigmoid(z) of each by
+// itself; the `top` outputs with the largest s + correction (null: none) are chosen (the lowest index
+// among equals), and weighted by their s alone, divided (`renorm`) by the sum of the chosen s
+// (+ 1e-20).  sel [N, top], wgt [N, top].
 __global__ __launch_bounds__(KVF_WAVE) void moe_topk_kernel(const float* __restrict__ z, int z_stride,
                                                             const float* __restrict__ correction,
                                                             int* __restrict__ sel, float* __restrict__ wgt,
-                                                            int R, int top) {
+                                                            int R, int top, int sigmoid, int renorm) {
   const int n = blockIdx.x, lane = threadIdx.x;
   const float* zr = z + static_cast<size_t>(n) * z_stride;
   float s[MAX_PER_LANE], c[MAX_PER_LANE];
@@ -23,20 +24,26 @@ __global__ __launch_bounds__(KVF_WAVE) void moe_topk_kernel(const float* __restr
     s[j] = e < R ? zr[e] : -INFINITY;
     mx = fmaxf(mx, s[j]);
   }
-  mx = wave_max(mx);
-  float sum = 0.f;
+  if (sigmoid) {
 #pragma unroll
-  for (int j = 0; j < MAX_PER_LANE; ++j) {
-    const int e = lane + KVF_WAVE * j;
-    s[j] = e < R ? expf(s[j] - mx) : 0.f;
-    sum += s[j];
+    for (int j = 0; j < MAX_PER_LANE; ++j) s[j] = 1.f / (1.f + expf(-s[j]));
+  } else {
+    mx = wave_max(mx);
+    float sum = 0.f;
+#pragma unroll
+    for (int j = 0; j < MAX_PER_LANE; ++j) {
+      const int e = lane + KVF_WAVE * j;
+      s[j] = e < R ? expf(s[j] - mx) : 0.f;
+      sum += s[j];
+    }
+    sum = wave_sum(sum);
+#pragma unroll
+    for (int j = 0; j < MAX_PER_LANE; ++j) s[j] = s[j] / sum;
   }
-  sum = wave_sum(sum);
 #pragma unroll
   for (int j = 0; j < MAX_PER_LANE; ++j) {
     const int e = lane + KVF_WAVE * j;
-    s[j] = s[j] / sum;
-    c[j] = e < R ? s[j] + correction[e] : -INFINITY;
+    c[j] = e < R ? s[j] + (correction ? correction[e] : 0.f) : -INFINITY;
   }
   float picked_s = 0.f, total = 0.f;   // lane k keeps the k-th choice
   int picked_e = -1;
@@ -73,7 +80,7 @@ __global__ __launch_bounds__(KVF_WAVE) void moe_topk_kernel(const float* __restr
   }
   if (lane < top) {
     sel[static_cast<size_t>(n) * top + lane] = picked_e;
-    wgt[static_cast<size_t>(n) * top + lane] = picked_s / (total + 1e-20f);
+    wgt[static_cast<size_t>(n) * top + lane] = renorm ? picked_s / (total + 1e-20f) : picked_s;
   }
 }
 
@@ -82,11 +89,12 @@ __device__ __forceinline__ float silu(float g) { return g / (1.f + expf(-g)); }
 // Every expert's gate/up pair for every token is there (one product over all experts, columns
 // 2 (e ff + j) and 2 (e ff + j) + 1): act[n, e ff + j] = weight(n, e) * silu(gate) * up where the
 // token chose expert e, and an exact zero elsewhere, so that one product with the experts' down
-// matrices side by side along K is the weighted sum over the chosen experts.
+// matrices side by side along K is the weighted sum over the chosen experts.  `weigh_input`: the weight
+// belongs to the expert's input, act = silu(w gate) * (w up) (gate and up are linear in it).
 template <typename T>
 __global__ void moe_dense_act_kernel(const T* __restrict__ gu, const int* __restrict__ sel,
                                      const float* __restrict__ wgt, T* __restrict__ act, int E, int ff,
-                                     int top, long total) {
+                                     int top, int weigh_input, long total) {
   const long i = static_cast<long>(blockIdx.x) * blockDim.x + threadIdx.x;
   if (i >= total) return;
   const long cols = static_cast<long>(E) * ff;
@@ -102,7 +110,7 @@ __global__ void moe_dense_act_kernel(const T* __restrict__ gu, const int* __rest
   float y = 0.f;
   if (chosen) {
     const float g = Elem<T>::load(gu + 2 * i), u = Elem<T>::load(gu + 2 * i + 1);
-    y = w * (silu(g) * u);
+    y = weigh_input ? silu(w * g) * (w * u) : w * (silu(g) * u);
   }
   Elem<T>::store(act + i, y);
 }
@@ -184,14 +192,15 @@ __global__ __launch_bounds__(1024) void moe_plan_kernel(const int* __restrict__ 
 // moe_up: act[place, :] = silu(gate) * up for the tile's rows with their expert's matrices; the
 // weight holds every expert's gate and up rows interleaved (gate_j, up_j neighbours), so a lane's
 // four columns are two whole pairs.  Grid (column blocks, tiles); a wave takes GW groups of 16
-// weight rows.
+// weight rows.  in_wgt (or null): the choice's weight belongs to the expert's input; gate and up are
+// linear in it, so it is multiplied into both sums ahead of the activation.
 template <int RT, int GW>
 __global__ __launch_bounds__(256) void moe_up_kernel(const bf16_t* __restrict__ x, int ldx, int K,
                                                      const uint4* __restrict__ wt, int S,
                                                      const int* __restrict__ order,
                                                      const int* __restrict__ tiles,
                                                      const int* __restrict__ num_tiles, int top, int ff,
-                                                     bf16_t* __restrict__ act) {
+                                                     const float* __restrict__ in_wgt, bf16_t* __restrict__ act) {
   const int tile = blockIdx.y;
   if (tile >= *num_tiles) return;
   const int e = tiles[3 * tile], row0 = tiles[3 * tile + 1], rows = tiles[3 * tile + 2];
@@ -249,11 +258,12 @@ __global__ __launch_bounds__(256) void moe_up_kernel(const bf16_t* __restrict__ 
   for (int r = 0; r < RT; ++r) {
     if (16 * r + j >= rows) continue;
     bf16_t* out = act + static_cast<size_t>(row0 + 16 * r + j) * ff;
+    const float w = in_wgt ? in_wgt[order[row0 + 16 * r + j]] : 1.f;
 #pragma unroll
     for (int g = 0; g < GW; ++g) {
       if (g_first + g >= groups) continue;
       const int col = (g_first + g) * 8 + 2 * c;
-      const float y0 = silu(acc[r][g][0]) * acc[r][g][1], y1 = silu(acc[r][g][2]) * acc[r][g][3];
+      const float y0 = silu(w * acc[r][g][0]) * (w * acc[r][g][1]), y1 = silu(w * acc[r][g][2]) * (w * acc[r][g][3]);
       *reinterpret_cast<uint32_t*>(out + col) =
           static_cast<uint32_t>(f32_to_bf16(y0)) | (static_cast<uint32_t>(f32_to_bf16(y1)) << 16);
     }
@@ -339,7 +349,8 @@ __global__ __launch_bounds__(256) void moe_down_kernel(const bf16_t* __restrict_
 // x[n, :] += sum over the token's choices, in their order, of weight * (the expert's row of y, or
 // the token's own input h for a choice that names no expert): fp32 sums into the fp32 stream.
 // A thread takes eight neighbouring elements (hidden is a multiple of 8 here): per choice one
-// 16-byte load, the choice itself being the same for the whole workgroup.
+// 16-byte load, the choice itself being the same for the whole workgroup.  wgt null: weights of one
+// (they went into the experts' inputs).  `fresh`: x is written, not added to.
 __device__ __forceinline__ void load8_any(const bf16_t* p, float (&v)[8]) { load8(p, v); }
 __device__ __forceinline__ void load8_any(const float* p, float (&v)[8]) { load8(p, v); }
 
@@ -348,7 +359,7 @@ __global__ __launch_bounds__(256) void moe_combine_kernel(float* __restrict__ x,
                                                           const T* __restrict__ h, const int* __restrict__ sel,
                                                           const float* __restrict__ wgt,
                                                           const int* __restrict__ where, int hidden, int top,
-                                                          int E) {
+                                                          int E, int fresh) {
   const int n = blockIdx.x;
   float* xr = x + static_cast<size_t>(n) * hidden;
   const T* hr = h + static_cast<size_t>(n) * hidden;
@@ -356,7 +367,7 @@ __global__ __launch_bounds__(256) void moe_combine_kernel(float* __restrict__ x,
     float sum[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
     for (int k = 0; k < top; ++k) {
       const int p = n * top + k, e = sel[p];
-      const float w = wgt[p];
+      const float w = wgt ? wgt[p] : 1.f;
       float v[8];
       if (e >= E) load8_any(hr + i, v);
       else if (e >= 0) load8(y + static_cast<size_t>(where[p]) * hidden + i, v);
@@ -364,7 +375,11 @@ __global__ __launch_bounds__(256) void moe_combine_kernel(float* __restrict__ x,
 #pragma unroll
       for (int u = 0; u < 8; ++u) sum[u] = fmaf(w, v[u], sum[u]);
     }
-    float4 a = *reinterpret_cast<const float4*>(xr + i), b = *reinterpret_cast<const float4*>(xr + i + 4);
+    float4 a = make_float4(0.f, 0.f, 0.f, 0.f), b = a;
+    if (!fresh) {
+      a = *reinterpret_cast<const float4*>(xr + i);
+      b = *reinterpret_cast<const float4*>(xr + i + 4);
+    }
     a.x += sum[0]; a.y += sum[1]; a.z += sum[2]; a.w += sum[3];
     b.x += sum[4]; b.y += sum[5]; b.z += sum[6]; b.w += sum[7];
     *reinterpret_cast<float4*>(xr + i) = a;
@@ -387,11 +402,12 @@ __global__ void moe_table_kernel(const int* __restrict__ tokens, const int* __re
 }  // namespace
 
 KVF_EXPORT int kvf_moe_topk(const float* z, int z_stride, const float* correction, int* sel, float* wgt,
-                            int n, int R, int top, hipStream_t s) {
+                            int n, int R, int top, int sigmoid, int renorm, hipStream_t s) {
   if (n <= 0) return 0;
   if (R <= 0 || R > MAX_PER_LANE * KVF_WAVE || top <= 0 || top > MAX_TOP || top > R)
     return static_cast<int>(hipErrorInvalidValue);
-  hipLaunchKernelGGL(moe_topk_kernel, dim3(n), dim3(KVF_WAVE), 0, s, z, z_stride, correction, sel, wgt, R, top);
+  hipLaunchKernelGGL(moe_topk_kernel, dim3(n), dim3(KVF_WAVE), 0, s, z, z_stride, correction, sel, wgt, R, top,
+                     sigmoid, renorm);
   return kvf_last_error();
 }
 
@@ -405,16 +421,16 @@ KVF_EXPORT int kvf_moe_table(const int* tokens, const int* table, int* sel, floa
 }
 
 KVF_EXPORT int kvf_moe_dense_act(int dtype, const void* gu, const int* sel, const float* wgt, void* act,
-                                 int n, int E, int ff, int top, hipStream_t s) {
+                                 int n, int E, int ff, int top, int weigh_input, hipStream_t s) {
   const long total = static_cast<long>(n) * E * ff;
   if (total <= 0) return 0;
   const dim3 grid(static_cast<unsigned>((total + 255) / 256));
   if (dtype == 0)
     hipLaunchKernelGGL(moe_dense_act_kernel<float>, grid, dim3(256), 0, s, static_cast<const float*>(gu), sel,
-                       wgt, static_cast<float*>(act), E, ff, top, total);
+                       wgt, static_cast<float*>(act), E, ff, top, weigh_input, total);
   else if (dtype == 1)
     hipLaunchKernelGGL(moe_dense_act_kernel<bf16_t>, grid, dim3(256), 0, s, static_cast<const bf16_t*>(gu), sel,
-                       wgt, static_cast<bf16_t*>(act), E, ff, top, total);
+                       wgt, static_cast<bf16_t*>(act), E, ff, top, weigh_input, total);
   else
     return static_cast<int>(hipErrorInvalidValue);
   return kvf_last_error();
@@ -437,11 +453,13 @@ KVF_EXPORT int kvf_moe_identity(int dtype, float* x, const void* h, const int* s
 // The routed experts of a bf16 step without the rows that did not choose them.  x [n, K] (row
 // stride ldx), w_gate_up / w_down: the tiled forms of [E 2 ff, K] (gate and up rows interleaved)
 // and [K, E ff]; sel / wgt [n, top]; scratch: where, order [n top], tiles [3 max_tiles],
-// num_tiles [1], act [n top, ff], y [n top, K].  Needs K % 8 == 0 and ff % 32 == 0.
+// num_tiles [1], act [n top, ff], y [n top, K].  Needs K % 8 == 0 and ff % 32 == 0.  weigh_input: the
+// weights go into the experts' inputs instead of the sum over their outputs.  fresh: residual is
+// written, not added to.
 KVF_EXPORT int kvf_moe_grouped(const void* x, int ldx, const void* h, int n, int K, int E, int ff, int top,
                                const void* w_gate_up, const void* w_down, const int* sel, const float* wgt,
                                int* where, int* order, int* tiles, int* num_tiles, int max_tiles, void* act,
-                               void* y, float* residual, hipStream_t s) {
+                               void* y, float* residual, int weigh_input, int fresh, hipStream_t s) {
   if (n <= 0) return 0;
   const int pairs = n * top;
   // many rows: tiles of 64 rows (four sub-tiles share every weight fragment); few: tiles of 16
@@ -457,18 +475,19 @@ KVF_EXPORT int kvf_moe_grouped(const void* x, int ldx, const void* h, int n, int
   const int grid_tiles = many ? (pairs + 63) / 64 + E : max_tiles;
   const dim3 up_grid((up_groups + 4 * gw - 1) / (4 * gw), grid_tiles), down_grid((down_groups + 4 * gw - 1) / (4 * gw), grid_tiles);
   const bf16_t* xb = static_cast<const bf16_t*>(x);
+  const float* in_wgt = weigh_input ? wgt : nullptr;
   if (many) {
     hipLaunchKernelGGL((moe_up_kernel<4, 4>), up_grid, dim3(256), 0, s, xb, ldx, K, static_cast<const uint4*>(w_gate_up), S,
-                       order, tiles, num_tiles, top, ff, static_cast<bf16_t*>(act));
+                       order, tiles, num_tiles, top, ff, in_wgt, static_cast<bf16_t*>(act));
     hipLaunchKernelGGL((moe_down_kernel<4, 4>), down_grid, dim3(256), 0, s, static_cast<const bf16_t*>(act), ff,
                        static_cast<const uint4*>(w_down), E * (ff / 32), tiles, num_tiles, static_cast<bf16_t*>(y), K);
   } else {
     hipLaunchKernelGGL((moe_up_kernel<1, 1>), up_grid, dim3(256), 0, s, xb, ldx, K, static_cast<const uint4*>(w_gate_up), S,
-                       order, tiles, num_tiles, top, ff, static_cast<bf16_t*>(act));
+                       order, tiles, num_tiles, top, ff, in_wgt, static_cast<bf16_t*>(act));
     hipLaunchKernelGGL((moe_down_kernel<1, 1>), down_grid, dim3(256), 0, s, static_cast<const bf16_t*>(act), ff,
                        static_cast<const uint4*>(w_down), E * (ff / 32), tiles, num_tiles, static_cast<bf16_t*>(y), K);
   }
   hipLaunchKernelGGL(moe_combine_kernel<bf16_t>, dim3(n), dim3(256), 0, s, residual, static_cast<const bf16_t*>(y),
-                     static_cast<const bf16_t*>(h), sel, wgt, where, K, top, E);
+                     static_cast<const bf16_t*>(h), sel, weigh_input ? nullptr : wgt, where, K, top, E, fresh);
   return kvf_last_error();
 }

@@ -49,6 +49,7 @@ MODULES: dict[str, list[str]] = {
     "latent": ["latent.hip"],
     "wkv": ["wkv.hip"],
     "linmem": ["linmem.hip"],
+    "ssm": ["ssm.hip"],
 }
 
 

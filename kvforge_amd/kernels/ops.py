@@ -369,6 +369,21 @@ def rms_add(x: torch.Tensor, y: torch.Tensor, weight: torch.Tensor, eps: float) 
         "rms_add")
 
 
+def rms_add_cast(x: torch.Tensor, y: torch.Tensor, weight: torch.Tensor, eps: float, out: torch.Tensor) -> None:
+    """``rms_add`` and a copy of the sum in one pass: ``x[m] += y[m] * rsqrt(mean(y[m]^2) + eps) * weight``,
+    then ``out[m] = x[m]`` in ``out``'s type."""
+    _check(x, "x", F32, (None, None))
+    _check(y, "y", F32, tuple(x.shape))
+    _check(weight, "weight", F32, (x.shape[1],))
+    _check(out, "out", None, tuple(x.shape))
+    if _overlap(x, out) or _overlap(y, out):
+        raise KernelError("rms_add_cast: out must not share memory with x or y")
+    f = _fn("elementwise", "kvf_rms_add_cast", [c_int, c_void_p, c_void_p, c_void_p, c_float, c_void_p, c_int, c_int,
+                                                c_void_p])
+    _ok(f(_tcode(out.dtype), x.data_ptr(), y.data_ptr(), weight.data_ptr(), float(eps), out.data_ptr(), x.shape[0],
+          x.shape[1], _stream()), "rms_add_cast")
+
+
 def rms_add_norm(x: torch.Tensor, y: torch.Tensor, weight: torch.Tensor, eps: float, weight2: torch.Tensor,
                  eps2: float, out: torch.Tensor) -> None:
     """``rms_add`` and the norm of the sum in one pass: ``x[m] += y[m] * rsqrt(mean(y[m]^2) + eps) *
@@ -1426,33 +1441,39 @@ def mlstm_out(heads_raw: torch.Tensor, gate: torch.Tensor, weight: torch.Tensor,
 
 
 # ------------------------------------------------------------------------------ latent attention
-def latent_split(proj: torch.Tensor, qkv: torch.Tensor, norm_weight: torch.Tensor, eps: float,
+def latent_split(proj: torch.Tensor, qkv: torch.Tensor, norm_weight: torch.Tensor | None, eps: float,
                  heads: int, dim: int, rot: int, rank: int, head_dim: int) -> None:
     """A projected row ``[heads x (dim | rot) | latent (rank) | shared key part (rot)]`` becomes
     the attention kernels' row ``[heads + 2, head_dim]``: q head ``h`` gets its ``rot`` part in
     front (columns ``rot..rot+rank-1`` are left for ``head_product`` to fill, the rest is
     zero), the one k head is ``[key part | norm(latent) | 0]`` and the one v head
     ``[0 | norm(latent) | 0]``, the norm being ``x / sqrt(mean(x^2) + eps) * norm_weight`` in
-    fp32 with one rounding."""
+    fp32 with one rounding.  ``norm_weight=None``: the projected row holds q heads alone, and so
+    does the attention row, ``[heads, head_dim]`` (attention over another layer's keys)."""
     n = proj.shape[0]
     H, d = int(heads), int(head_dim)
+    own = norm_weight is not None
     _check(proj, "proj", None, (n, None), contiguous=False)
-    _check(qkv, "qkv", proj.dtype, (n, (H + 2) * d))
-    _check(norm_weight, "norm_weight", F32, (rank,))
-    if proj.stride(1) != 1 or proj.shape[1] < H * (dim + rot) + rank + rot or d < rot + rank:
+    _check(qkv, "qkv", proj.dtype, (n, (H + (2 if own else 0)) * d))
+    if own:
+        _check(norm_weight, "norm_weight", F32, (rank,))
+    if proj.stride(1) != 1 or proj.shape[1] < H * (dim + rot) + (rank + rot if own else 0) or d < rot + rank:
         raise KernelError(f"latent_split: rows of {proj.shape[1]} elements / heads of {d} do not hold "
                           f"{H} x ({dim} + {rot}) + {rank} + {rot}")
     f = _fn("latent", "kvf_latent_split", [c_int, c_void_p, c_int, c_void_p, c_int, c_void_p, c_float]
             + [c_int] * 6 + [c_void_p])
     _ok(f(_tcode(proj.dtype), proj.data_ptr(), proj.stride(0) if n > 1 else proj.shape[1], qkv.data_ptr(),
-          qkv.shape[1], norm_weight.data_ptr(), float(eps), n, H, int(dim), int(rot), int(rank), d,
+          qkv.shape[1], norm_weight.data_ptr() if own else None, float(eps), n, H, int(dim), int(rot), int(rank), d,
           _stream()), "latent_split")
 
 
-def head_product(x: torch.Tensor, in_head: int, w: torch.Tensor, out: torch.Tensor, out_head: int) -> None:
+def head_product(x: torch.Tensor, in_head: int, w: torch.Tensor, out: torch.Tensor, out_head: int,
+                 gate: torch.Tensor | None = None) -> None:
     """``out[n, h * out_head + o] = sum_i w[h, o, i] * x[n, h * in_head + i]`` for per-head
     matrices ``w [H, O, I]``: ``x`` and ``out`` are rows (views of wider rows are fine) in which
-    head ``h`` starts ``h * in_head`` / ``h * out_head`` elements in.  fp32 multiply and add."""
+    head ``h`` starts ``h * in_head`` / ``h * out_head`` elements in.  fp32 multiply and add.
+    ``gate`` (``[n, >= H]``, dense rows of ``x``'s type): what is stored is the product times
+    ``sigmoid(gate[n, h])``."""
     n = x.shape[0]
     _check(w, "w", None, (None, None, None))
     H, O, I = w.shape
@@ -1465,11 +1486,16 @@ def head_product(x: torch.Tensor, in_head: int, w: torch.Tensor, out: torch.Tens
                           f"{x.shape[1]} / {out.shape[1]}")
     if _overlap(x, out):
         raise KernelError("head_product: out must not share memory with x")
+    if gate is not None:
+        _check(gate, "gate", x.dtype, (n, None), contiguous=False)
+        if gate.stride(1) != 1 or gate.shape[1] < H:
+            raise KernelError("head_product: a gate needs a number per head in dense rows")
     f = _fn("latent", "kvf_head_product", [c_int, c_int, c_void_p, c_int, c_int, c_void_p, c_void_p]
-            + [c_int] * 6 + [c_void_p])
+            + [c_int] * 6 + [c_void_p, c_int, c_void_p])
     _ok(f(_tcode(x.dtype), _tcode(w.dtype), x.data_ptr(), x.stride(0) if n > 1 else x.shape[1], int(in_head),
           w.data_ptr(), out.data_ptr(), out.stride(0) if n > 1 else out.shape[1], int(out_head), n, H, O, I,
-          _stream()), "head_product")
+          gate.data_ptr() if gate is not None else None,
+          (gate.stride(0) if n > 1 else gate.shape[1]) if gate is not None else 0, _stream()), "head_product")
 
 
 # ------------------------------------------------------------------------------ decaying matrix memory
@@ -1617,41 +1643,50 @@ MOE_MAX_ROUTER_OUTPUTS = 512
 MOE_MAX_TOP = 16
 
 
-def moe_topk(logits: torch.Tensor, correction: torch.Tensor, chosen: torch.Tensor,
-             weights: torch.Tensor) -> None:
-    """The router's choice per token from its fp32 ``logits [N, R]``: ``s = softmax(logits)``, the
-    ``top`` outputs with the largest ``s + correction`` (the lowest index among equals) go to
-    ``chosen [N, top]`` (int32) and their ``s``, divided by the sum of the chosen ``s`` (+ 1e-20),
-    to ``weights [N, top]`` (fp32)."""
+MOE_SCORES = {"softmax": 0, "sigmoid": 1}
+
+
+def moe_topk(logits: torch.Tensor, correction: torch.Tensor | None, chosen: torch.Tensor,
+             weights: torch.Tensor, scores: str = "softmax", renormalize: bool = True) -> None:
+    """The router's choice per token from its fp32 ``logits [N, R]``: ``s = softmax(logits)`` or, with
+    ``scores="sigmoid"``, ``s = sigmoid(logits)`` of every output by itself; the ``top`` outputs with
+    the largest ``s + correction`` (``None``: ``s`` alone; the lowest index among equals) go to
+    ``chosen [N, top]`` (int32) and their ``s``, with ``renormalize`` divided by the sum of the chosen
+    ``s`` (+ 1e-20), to ``weights [N, top]`` (fp32)."""
+    if scores not in MOE_SCORES:
+        raise KernelError(f"moe_topk: unknown scores {scores!r}; known: {sorted(MOE_SCORES)}")
     n, R = logits.shape
     _check(logits, "logits", F32, (n, R), contiguous=False)
     if logits.stride(1) != 1:
         raise KernelError("moe_topk: logits rows must be dense")
-    _check(correction, "correction", F32, (R,))
+    if correction is not None:
+        _check(correction, "correction", F32, (R,))
     top = chosen.shape[1]
     _check(chosen, "chosen", I32, (n, top))
     _check(weights, "weights", F32, (n, top))
     if R > MOE_MAX_ROUTER_OUTPUTS or not 0 < top <= min(MOE_MAX_TOP, R):
         raise KernelError(f"moe_topk: up to {MOE_MAX_ROUTER_OUTPUTS} router outputs and {MOE_MAX_TOP} choices, got {R} / {top}")
-    f = _fn("moe", "kvf_moe_topk", [c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_void_p])
-    _ok(f(logits.data_ptr(), logits.stride(0) if n > 1 else R, correction.data_ptr(), chosen.data_ptr(),
-          weights.data_ptr(), n, R, top, _stream()), "moe_topk")
+    f = _fn("moe", "kvf_moe_topk", [c_void_p, c_int, c_void_p, c_void_p, c_void_p] + [c_int] * 5 + [c_void_p])
+    _ok(f(logits.data_ptr(), logits.stride(0) if n > 1 else R,
+          correction.data_ptr() if correction is not None else None, chosen.data_ptr(), weights.data_ptr(), n, R, top,
+          MOE_SCORES[scores], 1 if renormalize else 0, _stream()), "moe_topk")
 
 
 def moe_dense_act(gate_up: torch.Tensor, chosen: torch.Tensor, weights: torch.Tensor, out: torch.Tensor,
-                  experts: int, ff: int) -> None:
+                  experts: int, ff: int, weigh_input: bool = False) -> None:
     """``gate_up [N, 2 experts ff]`` holds every expert's (gate, up) pairs as neighbouring columns;
     ``out[n, e ff + j] = weight(n, e) * silu(gate) * up`` where token ``n`` chose expert ``e`` and an
-    exact zero elsewhere."""
+    exact zero elsewhere.  ``weigh_input``: ``silu(w gate) * (w up)`` with ``w = weight(n, e)`` instead
+    (the weight belongs to the expert's input)."""
     n = gate_up.shape[0]
     E, top = int(experts), chosen.shape[1]
     _check(gate_up, "gate_up", None, (n, 2 * E * ff))
     _check(out, "out", gate_up.dtype, (n, E * ff))
     _check(chosen, "chosen", I32, (n, top))
     _check(weights, "weights", F32, (n, top))
-    f = _fn("moe", "kvf_moe_dense_act", [c_int] + [c_void_p] * 4 + [c_int] * 4 + [c_void_p])
+    f = _fn("moe", "kvf_moe_dense_act", [c_int] + [c_void_p] * 4 + [c_int] * 5 + [c_void_p])
     _ok(f(_tcode(gate_up.dtype), gate_up.data_ptr(), chosen.data_ptr(), weights.data_ptr(), out.data_ptr(),
-          n, E, int(ff), top, _stream()), "moe_dense_act")
+          n, E, int(ff), top, 1 if weigh_input else 0, _stream()), "moe_dense_act")
 
 
 def moe_identity(x: torch.Tensor, h: torch.Tensor, chosen: torch.Tensor, weights: torch.Tensor,
@@ -1685,7 +1720,7 @@ def moe_grouped_tiles(rows: int, top: int, experts: int) -> int:
 
 def moe_grouped(x: torch.Tensor, w_gate_up: "StreamedWeight", w_down: "StreamedWeight", chosen: torch.Tensor,
                 weights: torch.Tensor, residual: torch.Tensor, experts: int, ff: int,
-                scratch: dict[str, torch.Tensor]) -> None:
+                scratch: dict[str, torch.Tensor], weigh_input: bool = False, fresh: bool = False) -> None:
     """``residual[n] += sum_k weights[n, k] * expert_{chosen[n, k]}(x[n])`` (a choice ``>= experts``
     stands for ``x[n]`` itself) with every expert's products taken over only the rows that chose
     it: the pairs are grouped by expert on the device, tiles of 16 rows go through the
@@ -1693,7 +1728,9 @@ def moe_grouped(x: torch.Tensor, w_gate_up: "StreamedWeight", w_down: "StreamedW
     up rows interleaved) and ``w_down`` (``[K, experts * ff]``), an expert's output row is stored
     in bf16 and the weighted sum over a token's choices is taken in fp32 in their order.
     ``scratch``: ``where order [n top]``, ``tiles [3 moe_grouped_tiles]``, ``num_tiles [1]`` (int32),
-    ``act [n top, ff]``, ``y [n top, K]`` (bf16)."""
+    ``act [n top, ff]``, ``y [n top, K]`` (bf16).  ``weigh_input``: every chosen expert reads its
+    weight times the row, ``expert(weights[n, k] * x[n])``, and the outputs are summed as they are.
+    ``fresh``: ``residual`` is written instead of added to."""
     n, k = x.shape
     top = chosen.shape[1]
     if not moe_grouped_takes(x, w_gate_up, w_down, experts, ff):
@@ -1709,12 +1746,12 @@ def moe_grouped(x: torch.Tensor, w_gate_up: "StreamedWeight", w_down: "StreamedW
                                ("num_tiles", I32, (1,)), ("act", BF16, (pairs, ff)), ("y", BF16, (pairs, k))):
         _check(scratch[name], name, dtype, shape)
     f = _fn("moe", "kvf_moe_grouped", [c_void_p, c_int, c_void_p] + [c_int] * 5 + [c_void_p] * 8 + [c_int]
-            + [c_void_p] * 4)
+            + [c_void_p] * 3 + [c_int, c_int, c_void_p])
     _ok(f(x.data_ptr(), x.stride(0) if n > 1 else k, x.data_ptr(), n, k, int(experts), int(ff), top,
           w_gate_up.tiles.data_ptr(), w_down.tiles.data_ptr(), chosen.data_ptr(), weights.data_ptr(),
           scratch["where"].data_ptr(), scratch["order"].data_ptr(), scratch["tiles"].data_ptr(),
           scratch["num_tiles"].data_ptr(), max_tiles, scratch["act"].data_ptr(), scratch["y"].data_ptr(),
-          residual.data_ptr(), _stream()), "moe_grouped")
+          residual.data_ptr(), 1 if weigh_input else 0, 1 if fresh else 0, _stream()), "moe_grouped")
 
 
 
@@ -1863,6 +1900,174 @@ def linmem_out(heads_raw: torch.Tensor, gate: torch.Tensor, weight: torch.Tensor
     _ok(f(_tcode(out.dtype), heads_raw.data_ptr(), gate.data_ptr(), gate.stride(0) if n > 1 else H * dv,
           weight.data_ptr() if weight is not None else None, float(eps), float(scale), out.data_ptr(), n, H, dv,
           _stream()), "linmem_out")
+
+
+# ------------------------------------------------------------------------------ state-space memories
+# Runs of at least SSM_CHUNK_FROM tokens are cut into chunks that go through the matrix cores; shorter
+# ones go token by token in one workgroup per head and slice of value columns.
+SSM_CHUNK_FROM = 24
+SSM_MAX_TAPS = 8
+
+
+def ssm_state_floats(heads: int, key_dim: int, value_dim: int, channels: int, taps: int) -> int:
+    """fp32 numbers of a request's slot: every head's ``S [key_dim, value_dim]``, then the
+    convolution's last ``taps - 1`` inputs of all channels."""
+    return int(heads) * int(key_dim) * int(value_dim) + (int(taps) - 1) * int(channels)
+
+
+def ssm_chunk_len(key_dim: int) -> int:
+    """Tokens of a chunk for heads of this key size."""
+    return 64 if key_dim <= 128 else 32
+
+
+def ssm_plan(q_lens, key_dim: int, chunk_from: int = SSM_CHUNK_FROM) -> tuple[list[int], list[int]]:
+    """For the runs of at least ``chunk_from`` tokens among ``q_lens`` (a step's runs in sequence
+    order): the flat rows ``(sequence, first token, tokens, 0)`` of their chunks and
+    ``(sequence, first chunk, chunks)`` of the runs, as ``ssm_scan(multi=...)`` wants them."""
+    cl = ssm_chunk_len(key_dim)
+    chunks: list[int] = []
+    runs: list[int] = []
+    start = 0
+    for seq, q in enumerate(q_lens):
+        if q >= chunk_from:
+            first = len(chunks) // 4
+            for t in range(0, q, cl):
+                chunks += [seq, start + t, min(cl, q - t), 0]
+            runs += [seq, first, len(chunks) // 4 - first]
+        start += q
+    return chunks, runs
+
+
+def ssm_scratch(n_tokens: int, n_chunks: int, heads: int, key_dim: int, value_dim: int, delta: bool) -> dict[str, tuple]:
+    """(shape, dtype) of the scratch tensors the passes over the chunks need, by name."""
+    H, dk, dv, cl = int(heads), int(key_dim), int(value_dim), ssm_chunk_len(key_dim)
+    out = {"W": ((n_chunks, H, dk, dv), F32)}
+    if delta:
+        out.update({"T": ((n_chunks, H, cl, cl), F32), "U": ((n_tokens, H, dv), F32)})
+    else:
+        out["E"] = ((n_chunks, H), F32)
+    return out
+
+
+def ssm_conv(rows: torch.Tensor, col0: int, weight: torch.Tensor, bias: torch.Tensor | None, cu_q: torch.Tensor,
+             positions: torch.Tensor, slot_ids: torch.Tensor, state: torch.Tensor, state_off: int, out: torch.Tensor,
+             n_seqs: int, longest: int, unit: int = 0, key_dim: int = 0, q_scale: float = 1.0) -> None:
+    """A short causal convolution per channel with silu over every query run: ``out[t, c] =
+    silu(sum_j weight[c, j] * x[t - (taps - 1) + j, c] + bias[c])`` with ``x`` the columns ``col0 ..
+    col0 + C - 1`` of ``rows`` and ``weight`` fp32 ``[C, taps]``.  What lies before a run is read from the
+    sequence's slot (``taps - 1`` rows of ``C`` floats from ``state_off`` on, the oldest first; zeros at
+    position 0), where the run leaves its own last inputs.  The first ``unit`` channels are heads of
+    ``key_dim`` elements that are then divided by ``sqrt(sum of squares + 1e-6)``, the first half of them
+    multiplied by ``q_scale``.  ``out`` fp32 ``[n, C]``; ``longest``: tokens of the longest run."""
+    n = rows.shape[0]
+    C, taps = weight.shape
+    _check(rows, "rows", None, (n, None), contiguous=False)
+    if rows.stride(1) != 1 or col0 < 0 or col0 + C > rows.shape[1]:
+        raise KernelError(f"ssm_conv: channels {col0}..{col0 + C} in dense rows of {rows.shape[1]}")
+    _check(weight, "weight", F32, (C, taps))
+    if not 1 <= taps <= SSM_MAX_TAPS:
+        raise KernelError(f"ssm_conv: 1 to {SSM_MAX_TAPS} taps, got {taps}")
+    if bias is not None:
+        _check(bias, "bias", F32, (C,))
+    if unit and (not 0 < key_dim <= 256 or unit % (2 * key_dim) or unit > C):
+        raise KernelError(f"ssm_conv: {unit} channels are not q and k heads of {key_dim} elements (at most 256)")
+    _check(state, "state", F32, (None, None))
+    if state_off < 0 or state_off + (taps - 1) * C > state.shape[1]:
+        raise KernelError(f"ssm_conv: slots of {state.shape[1]} floats do not hold {taps - 1} x {C} inputs from {state_off} on")
+    for t, name in ((cu_q, "cu_q"), (positions, "positions"), (slot_ids, "slot_ids")):
+        _check(t, name, I32, (None,))
+    if cu_q.shape[0] < n_seqs + 1 or slot_ids.shape[0] < n_seqs or positions.shape[0] < n or not 0 < longest <= n:
+        raise KernelError("ssm_conv: batch arrays shorter than the batch")
+    _check(out, "out", F32, (n, C))
+    f = _fn("ssm", "kvf_ssm_conv", [c_int, c_void_p] + [c_int] * 4 + [c_void_p] * 2 + [c_int, c_int, c_float]
+            + [c_void_p] * 4 + [c_int] * 3 + [c_void_p] + [c_int] * 2 + [c_void_p])
+    _ok(f(_tcode(rows.dtype), rows.data_ptr(), rows.stride(0) if n > 1 else rows.shape[1], int(col0), C, taps,
+          weight.data_ptr(), bias.data_ptr() if bias is not None else None, int(unit), int(key_dim), float(q_scale),
+          cu_q.data_ptr(), positions.data_ptr(), slot_ids.data_ptr(), state.data_ptr(), state.shape[0], state.shape[1],
+          int(state_off), out.data_ptr(), int(n_seqs), int(longest), _stream()), "ssm_conv")
+
+
+def ssm_scan(rows: torch.Tensor, q_off: int, k_off: int, v_off: int, gates: torch.Tensor, a_off: int,
+             b_off: int | None, neg_a: torch.Tensor, dt_bias: torch.Tensor, skip: torch.Tensor | None,
+             cu_q: torch.Tensor, positions: torch.Tensor, slot_ids: torch.Tensor, state: torch.Tensor, out: torch.Tensor,
+             n_seqs: int, heads: int, key_heads: int, key_dim: int, value_dim: int, multi: dict | None = None,
+             short_runs: bool = True) -> None:
+    """A matrix memory per head with one decay per head and token, over every query run, in fp32,
+    from and to the sequences' state slots (a run at position 0 starts from zeros whatever its slot
+    holds; a sequence without a slot starts from zeros and keeps nothing).  ``rows`` fp32 ``[n, ld]``
+    holds ``key_heads`` heads of q (from column ``q_off``) and of k (``k_off``), ``key_dim`` elements each, and
+    ``heads`` heads of v (``v_off``); head ``h`` uses q/k head ``h // (heads / key_heads)``.  ``gates`` fp32
+    ``[n, >= ...]``: with ``dt = softplus(gates[a_off + h] + dt_bias[h])`` the decay is ``exp(neg_a[h] * dt)``.
+    ``b_off=None``: ``S <- a S + dt k v^T`` and ``o = S^T q + skip[h] v``.  With ``b_off`` the delta rule:
+    ``beta = sigmoid(gates[b_off + h])``, ``S <- a S``, ``S <- S + k (beta (v - S^T k))^T``, ``o = S^T q``.
+    ``out`` fp32 ``[n, heads * value_dim]``.  ``multi``: ``chunks`` and ``runs`` (int32 device tensors of
+    ``ssm_plan``'s rows) and the tensors of ``ssm_scratch``: those runs go chunk by chunk and the
+    token-by-token kernel leaves them alone; it is not launched with ``short_runs=False``."""
+    n = rows.shape[0]
+    H, G, dk, dv = int(heads), int(key_heads), int(key_dim), int(value_dim)
+    delta = b_off is not None
+    _check(rows, "rows", F32, (n, None), contiguous=False)
+    if rows.stride(1) != 1 or G <= 0 or H % G or not 0 < dk <= 256 or dv <= 0:
+        raise KernelError(f"ssm_scan: dense rows, {H} heads over {G} key heads of {dk} (at most 256) x {dv}")
+    for off, size, name in ((q_off, G * dk, "q"), (k_off, G * dk, "k"), (v_off, H * dv, "v")):
+        if off < 0 or off + size > rows.shape[1]:
+            raise KernelError(f"ssm_scan: {name} at columns {off}..{off + size} lies outside rows of {rows.shape[1]}")
+    _check(gates, "gates", F32, (n, None), contiguous=False)
+    if gates.stride(1) != 1 or not 0 <= a_off <= gates.shape[1] - H or (delta and not 0 <= b_off <= gates.shape[1] - H):
+        raise KernelError("ssm_scan: gate rows too short or not dense")
+    _check(neg_a, "neg_a", F32, (H,))
+    _check(dt_bias, "dt_bias", F32, (H,))
+    if skip is not None:
+        _check(skip, "skip", F32, (H,))
+        if delta:
+            raise KernelError("ssm_scan: no skip beside the delta rule")
+    _check(out, "out", F32, (n, H * dv))
+    _check(state, "state", F32, (None, None))
+    if state.shape[1] < H * dk * dv:
+        raise KernelError(f"ssm_scan: heads of {dk} x {dv} need slots of {H * dk * dv} floats")
+    for t, name in ((cu_q, "cu_q"), (positions, "positions"), (slot_ids, "slot_ids")):
+        _check(t, name, I32, (None,))
+    if cu_q.shape[0] < n_seqs + 1 or slot_ids.shape[0] < n_seqs or positions.shape[0] < n:
+        raise KernelError("ssm_scan: batch arrays shorter than the batch")
+    common = (1 if delta else 0, rows.data_ptr(), rows.stride(0) if n > 1 else rows.shape[1], int(q_off), int(k_off),
+              int(v_off), gates.data_ptr(), gates.stride(0) if n > 1 else gates.shape[1], int(a_off),
+              int(b_off) if delta else 0, neg_a.data_ptr(), dt_bias.data_ptr(),
+              skip.data_ptr() if skip is not None else None, positions.data_ptr(), slot_ids.data_ptr(),
+              state.data_ptr(), state.shape[0], state.shape[1], out.data_ptr(), H, G, dk, dv)
+    types = ([c_int, c_void_p] + [c_int] * 4 + [c_void_p] + [c_int] * 3 + [c_void_p] * 6 + [c_int] * 2 + [c_void_p]
+             + [c_int] * 4)
+    if short_runs or multi is None:
+        f = _fn("ssm", "kvf_ssm_scan", types + [c_void_p, c_int, c_int, c_void_p])
+        _ok(f(*common, cu_q.data_ptr(), int(n_seqs), SSM_CHUNK_FROM if multi is not None else 0, _stream()), "ssm_scan")
+    if multi is None:
+        return
+    chunks, runs = multi["chunks"], multi["runs"]
+    _check(chunks, "chunks", I32, (None, 4))
+    _check(runs, "runs", I32, (None, 3))
+    nc = chunks.shape[0]
+    for name, (shape, dtype) in ssm_scratch(n, nc, H, dk, dv, delta).items():
+        _check(multi[name], name, dtype, shape)
+    f = _fn("ssm", "kvf_ssm_chunks", types + [c_void_p, c_int, c_void_p, c_int] + [c_void_p] * 5)
+    _ok(f(*common, chunks.data_ptr(), nc, runs.data_ptr(), runs.shape[0],
+          *(multi[k].data_ptr() if k in multi else None for k in ("T", "W", "U", "E")), _stream()), "ssm_chunks")
+
+
+def ssm_gate_norm(y: torch.Tensor, gate: torch.Tensor, weight: torch.Tensor, eps: float, parts: int,
+                  out: torch.Tensor) -> None:
+    """``out = weight * u / sqrt(mean(u^2) + eps)`` with ``u = y * silu(gate)``, the mean over each of ``parts``
+    equal parts of the row.  ``y`` fp32 ``[n, inner]``; ``gate``: dense rows of ``out``'s type (a view of wider
+    rows is fine)."""
+    n, inner = y.shape
+    _check(y, "y", F32, (n, inner))
+    _check(weight, "weight", F32, (inner,))
+    _check(out, "out", None, (n, inner))
+    _check(gate, "gate", out.dtype, (n, inner), contiguous=False)
+    if gate.stride(1) != 1 or parts <= 0 or inner % parts:
+        raise KernelError(f"ssm_gate_norm: dense gate rows and rows of {inner} in {parts} equal parts")
+    f = _fn("ssm", "kvf_ssm_gate_norm", [c_int, c_void_p, c_void_p, c_int, c_void_p, c_float, c_void_p] + [c_int] * 3
+            + [c_void_p])
+    _ok(f(_tcode(out.dtype), y.data_ptr(), gate.data_ptr(), gate.stride(0) if n > 1 else inner, weight.data_ptr(),
+          float(eps), out.data_ptr(), n, inner, int(parts), _stream()), "ssm_gate_norm")
 
 
 # ------------------------------------------------------------------------------ sampling

@@ -12,8 +12,9 @@ from kvforge_amd.parts.latent import LatentAttention
 from kvforge_amd.parts.wkv import DecayMemory
 from kvforge_amd.parts.linmem import LinearMemory
 from kvforge_amd.parts.pair import MixerPair
+from kvforge_amd.parts.ssm import ConvMemory, GatedDelta, Mamba2
 from kvforge_amd.parts.embedding import LMHead, TokenEmbedding
-from kvforge_amd.parts.block import ParallelBlock, PreNormBlock, SandwichBlock
+from kvforge_amd.parts.block import ParallelBlock, PostNormBlock, PreNormBlock, SandwichBlock
 
 __all__ = ["BLOCK", "PageTensor", "attention_pages", "Block", "CacheSpec", "Embedding", "FeedForward", "Head", "LayerCall", "LayerState", "Mixer", "ModelSpec",
            "Norm", "Part", "Positions", "StateSpec", "WeightSpec", "RMSNorm", "RotaryPositions",
@@ -21,4 +22,4 @@ __all__ = ["BLOCK", "PageTensor", "attention_pages", "Block", "CacheSpec", "Embe
            "PreNormBlock", "ParallelBlock", "ScalarRMSNorm", "LearnedPositions", "GatedFeedForward",
            "TokenSideInput", "OnePlusRMSNorm", "YarnStretch", "MatrixLSTM", "RoutedExperts",
            "NamedRMSNorm", "LatentAttention", "DecayMemory", "SandwichBlock", "LinearMemory", "MixerPair",
-           "PlainFeedForward"]
+           "PlainFeedForward", "ConvMemory", "GatedDelta", "Mamba2", "PostNormBlock"]

@@ -156,6 +156,54 @@ class ParallelBlock(Block):
             self.after.forward(residual, step, bias=bias)
 
 
+@register_block("post_norm")
+class PostNormBlock(Block):
+    """The sublayers read the stream itself, and what they give joins it through a norm:
+    ``x += norm(mixer(x))`` and then, if the layer has a feed-forward, ``x += ffn_norm(ffn(x))``.
+    As in a sandwich block a sublayer's last product is written to rows of its own (fp32; the
+    step holds them as ``fresh``), which stay owed to the stream until it is read next; the kernel
+    that adds them (norm and sum in fp32) also leaves the stream's copy in the sublayers' type."""
+
+    def __init__(self, mixer: Mixer, norm: Norm, ffn: FeedForward | None = None, ffn_norm: Norm | None = None) -> None:
+        if (ffn is None) != (ffn_norm is None):
+            raise ValueError("a feed-forward and its norm come together")
+        self.mixer, self.norm, self.ffn, self.ffn_norm = mixer, norm, ffn, ffn_norm
+
+    def parts(self) -> list[Part]:
+        return [p for p in (self.mixer, self.norm, self.ffn, self.ffn_norm) if p is not None]
+
+    def kernel_modules(self, dtype) -> set[str]:
+        return super().kernel_modules(dtype) | {"elementwise"}
+
+    def forward(self, residual, step, layer: LayerState) -> None:
+        branch = step.ws.buf("sublayer_out", tuple(residual.shape), torch.float32)
+        x = self._read(residual, step)
+        step.fresh = branch
+        self.mixer.forward(x, step, layer, branch)
+        SandwichBlock._join(residual, branch, self.norm, step)
+        if self.ffn is None:
+            return
+        x = self._read(residual, step)
+        step.fresh = branch
+        self.ffn.forward(x, step, branch)
+        SandwichBlock._join(residual, branch, self.ffn_norm, step)
+
+    @staticmethod
+    def _read(residual, step) -> torch.Tensor:
+        """The up-to-date stream as a sublayer reads it: itself in 32-bit, else a copy in the step's
+        activation type, made by the kernel that adds what is owed."""
+        if step.act_dtype == torch.float32:
+            step.settle()
+            return residual
+        x = step.ws.buf("stream_read", tuple(residual.shape), step.act_dtype)
+        owed = step.take_owed_normed(residual)
+        if owed is not None:
+            ops.rms_add_cast(residual, *owed, x)
+        else:
+            ops.settle_cast(residual, owed=step.take_owed(residual), copy=x)
+        return x
+
+
 @register_block("sandwich")
 class SandwichBlock(Block):
     """A norm before and after each sublayer: ``x += post(mixer(pre(x)))`` and then, if the layer
@@ -199,7 +247,8 @@ class SandwichBlock(Block):
         read next: by the norm in front of the next sublayer (one kernel for the sum and that
         norm), or by whoever settles the step."""
         if step.fresh is branch:
-            raise RuntimeError("a sublayer of a sandwich block must end in parts.base.add_product")
+            raise RuntimeError("a sublayer whose output joins the stream through a norm must write its fresh rows "
+                               "(end in parts.base.add_product)")
         step.settle()
         weight = post.fp32_weight() if hasattr(post, "fp32_weight") else None
         if weight is None:

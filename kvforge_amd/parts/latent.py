@@ -27,7 +27,11 @@ from kvforge_amd.registry import register_mixer
 
 @register_mixer("latent_attention")
 class LatentAttention(PagedAttention):
-    """``names``: checkpoint names under the prefix, by ``q dkv dkv_norm uk uv o``.  ``rotary``:
+    """``names``: checkpoint names under the prefix, by ``q dkv dkv_norm uk uv o``.  ``own_kv=False``:
+    the mixer has no ``dkv`` and uses the latents and rotated key parts that another call's pages
+    hold (of equal ``kv_rank``, ``rot_dim`` and rotation).  ``head_gate``: checkpoint name of a matrix
+    ``[heads, hidden]``; head ``h``'s output is multiplied by ``sigmoid(W_g x)_h`` where the values are
+    read out.  ``rotary``:
     the rotation of the ``rot_dim`` parts (its width must be ``rot_dim`` at most).  ``window``,
     ``sink``, ``scale``: as in ``PagedAttention``, whose launch planning and kernels this
     mixer uses with one kv head of ``rot_dim + kv_rank`` elements."""
@@ -40,7 +44,7 @@ class LatentAttention(PagedAttention):
     def __init__(self, prefix: str, hidden: int, num_heads: int, head_dim: int, rot_dim: int,
                  value_dim: int, kv_rank: int, rotary: RotaryPositions | None, scale: float,
                  norm_eps: float, window: int | None = None, sink: str | None = None,
-                 names: dict[str, str] | None = None) -> None:
+                 names: dict[str, str] | None = None, head_gate: str | None = None, own_kv: bool = True) -> None:
         self.prefix, self.hidden, self.H, self.KV = prefix, int(hidden), int(num_heads), 1
         self.dim, self.rot, self.dv_out, self.rank = int(head_dim), int(rot_dim), int(value_dim), int(kv_rank)
         if min(self.H, self.dv_out, self.rank) <= 0 or self.dim < 0 or self.rot < 0 or self.dim + self.rot <= 0:
@@ -57,11 +61,11 @@ class LatentAttention(PagedAttention):
         self.scale, self.norm_eps_c = float(scale), float(norm_eps)
         if not self.scale > 0.0:
             raise ValueError(f"scale must be positive, got {scale}")
-        self.window = int(window) if window else None
+        self.window, self.chunk = int(window) if window else None, None
         self.keep_first = 0
         self.names = dict(self.LATENT_NAMES, **(names or {}))
-        self.sink = sink
-        self.gated, self.own_kv, self.qk_norm = False, True, None
+        self.sink, self.head_gate = sink, head_gate
+        self.gated, self.own_kv, self.qk_norm = False, bool(own_kv), None
         self.score_slopes = self.slopes = self.sinks = None
         self.score_cap = self.q_temp = None
         self.cache_spec = CacheSpec(attention_pages(1, self.d), self.window, 0)
@@ -71,27 +75,36 @@ class LatentAttention(PagedAttention):
         h, H = self.hidden, self.H
         n = lambda key: self._name(self.names[key])  # noqa: E731
         out = {n("q"): WeightSpec((H * (self.dim + self.rot), h)),
-               n("dkv"): WeightSpec((self.rank + self.rot, h)),
-               n("dkv_norm"): WeightSpec((self.rank,), init="norm", std=0.1),
                n("uk"): WeightSpec((H * self.dim, self.rank)),
                n("uv"): WeightSpec((H * self.dv_out, self.rank)),
                n("o"): WeightSpec((h, H * self.dv_out))}
+        if self.own_kv:
+            out[n("dkv")] = WeightSpec((self.rank + self.rot, h))
+            out[n("dkv_norm")] = WeightSpec((self.rank,), init="norm", std=0.1)
+        if self.head_gate is not None:
+            out[self._name(self.head_gate)] = WeightSpec((H, h))
         if self.sink is not None:
             out[self._name(self.sink)] = WeightSpec((H,), std=1.0)
         return out
 
     def load(self, tensors: dict[str, torch.Tensor]) -> None:
         t = lambda key: tensors[self._name(self.names[key])]  # noqa: E731
-        q, dkv = t("q"), t("dkv")
-        if q.dtype != dkv.dtype:
-            q, dkv = q.float(), dkv.float()
-        # one product for the queries, the latent and the shared key part
-        self.w_in = torch.cat([q, dkv], dim=0).contiguous()
+        mats = [t("q")] + ([t("dkv")] if self.own_kv else [])
+        # one product for the queries, the latent, the shared key part and the heads' gates (their
+        # rows padded with zero rows, so that the product's rows start on 16 bytes)
+        self.gate_col = sum(int(m.shape[0]) for m in mats)
+        if self.head_gate is not None:
+            g = tensors[self._name(self.head_gate)]
+            mats += [g, g.new_zeros(-(self.gate_col + self.H) % 16, self.hidden)]
+        if len({m.dtype for m in mats}) > 1:
+            mats = [m.float() for m in mats]
+        self.w_in = torch.cat(mats, dim=0).contiguous()
         # the queries go through the keys' read-out transposed: [H, rank, dim]
         self.w_uk_t = t("uk").view(self.H, self.dim, self.rank).transpose(1, 2).contiguous()
         self.w_uv = t("uv").view(self.H, self.dv_out, self.rank).contiguous()
         self.w_o = t("o")
-        self.c_norm_w = t("dkv_norm").float().contiguous()
+        if self.own_kv:
+            self.c_norm_w = t("dkv_norm").float().contiguous()
         if self.sink is not None:
             self.sinks = tensors[self._name(self.sink)].float().contiguous()
 
@@ -124,13 +137,13 @@ class LatentAttention(PagedAttention):
         step.settle()
         proj = ws.buf("latent_proj", (n, self.w_in.shape[0]), act)
         ops.gemm(x, self.w_in, proj)
-        qkv = ws.buf("latent_qkv", (n, (H + 2) * d), act)
+        qkv = ws.buf("latent_qkv", (n, (H + (2 if self.own_kv else 0)) * d), act)
         ops.latent_split(proj, qkv, self.c_norm_w, self.norm_eps_c, H, dim, rot, rank, d)
         if dim:
             # q_h -> W_uk_h^T q_h, next to the head's rotated part
             ops.head_product(proj[:, :H * (dim + rot)], dim + rot, self.w_uk_t, qkv[:, rot:H * d], d)
         ops.rope_kvwrite(qkv, step.positions, step.seq_of_token, cos, sin, table, layer.k_pages,
-                         layer.v_pages, H, 1, d, write_kv=layer.owns_cache)
+                         layer.v_pages, H, 1, d, write_kv=layer.owns_cache and self.own_kv)
         out = ws.buf("attn_out", (n, H * d), act)
         bs = layer.k_pages.shape[2]
         work, rows_per_item = self._prefill_work(step, act, bs)
@@ -149,5 +162,6 @@ class LatentAttention(PagedAttention):
                             token_is_seq=step.decode_seq_ids is None and work is None, sinks=self.sinks)
         # the heads' weighted sums of the latent, read out by W_uv_h
         heads = ws.buf("latent_heads", (n, H * self.dv_out), act)
-        ops.head_product(out[:, rot:], d, self.w_uv, heads, self.dv_out)
+        gate = proj[:, self.gate_col:self.gate_col + H] if self.head_gate is not None else None
+        ops.head_product(out[:, rot:], d, self.w_uv, heads, self.dv_out, gate=gate)
         add_product(step, heads, self.w_o, residual)

@@ -11,6 +11,10 @@ weighted sum over the chosen experts, plus the shared expert's output.
 Instead of a router a *table* may make the choice: an integer tensor ``[vocab, top]`` names the
 experts of every token id (a row's entries differ), each with weight ``1 / top``.  The shared
 expert's output may be multiplied by ``sigmoid(w . x)``, one number per token.
+
+Variants of the router: ``s = sigmoid(W_r x)`` of every output by itself, weights that are the chosen
+``s`` as they are, no correction, and weights that belong to the chosen experts' inputs,
+``sum expert(w x)``, instead of their outputs.
 """
 
 from __future__ import annotations
@@ -32,7 +36,11 @@ class RoutedExperts(FeedForward):
     ``shared_gate``: the shared expert's output is multiplied by ``sigmoid(w . x)`` with ``w``
     the tensor ``[1, hidden]`` named ``shared_gate`` under the shared expert's prefix; the number
     is a product with fp32 sums and joins the expert's activation ahead of its (linear) down
-    projection."""
+    projection.  ``scores``: ``"softmax"`` over all outputs, or ``"sigmoid"`` of each; ``renormalize``:
+    whether the weights are divided by their sum; ``correct``: whether there is a ``correction``;
+    ``weigh_input``: the weights go into the experts' inputs (gate and up are linear in it, so they
+    are multiplied into those two products' fp32 sums, or into the stored products, ahead of the
+    activation)."""
 
     NAMES = {"expert": "e{e}", "gate": "gate", "up": "up", "down": "down", "router": "router",
              "correction": "correction", "shared": "shared", "table": "table", "shared_gate": "sg"}
@@ -41,7 +49,8 @@ class RoutedExperts(FeedForward):
 
     def __init__(self, prefix: str, hidden: int, ff: int, experts: int, top: int, identity: int = 0,
                  shared_ff: int = 0, names: dict[str, str] | None = None, table_vocab: int | None = None,
-                 shared_gate: bool = False) -> None:
+                 shared_gate: bool = False, scores: str = "softmax", renormalize: bool = True,
+                 correct: bool = True, weigh_input: bool = False) -> None:
         self.prefix, self.hidden, self.ff = prefix, int(hidden), int(ff)
         self.E, self.top, self.identity = int(experts), int(top), int(identity)
         self.R = self.E + self.identity
@@ -52,6 +61,12 @@ class RoutedExperts(FeedForward):
         if self.shared_gate and not shared_ff:
             raise ValueError("a gate on the shared expert goes with a shared expert")
         self.table = self.w_shared_gate = None
+        if scores not in ops.MOE_SCORES:
+            raise ValueError(f"unknown router scores {scores!r}; known: {sorted(ops.MOE_SCORES)}")
+        self.scores, self.renormalize = scores, bool(renormalize)
+        self.correct, self.weigh_input = bool(correct), bool(weigh_input)
+        if self.weigh_input and self.identity:
+            raise ValueError("weights on the experts' inputs go without identity outputs")
         if not 0 < self.top <= min(self.R, ops.MOE_MAX_TOP) or self.R > ops.MOE_MAX_ROUTER_OUTPUTS:
             raise ValueError(f"router of {self.R} outputs choosing {self.top}: the kernels take up to "
                              f"{ops.MOE_MAX_ROUTER_OUTPUTS} outputs and {ops.MOE_MAX_TOP} choices")
@@ -72,8 +87,9 @@ class RoutedExperts(FeedForward):
             out = {self._name(self.names["table"]): WeightSpec((self.table_vocab, self.top), init="choices",
                                                                 std=float(self.E), integer=True)}
         else:
-            out = {self._name(self.names["router"]): WeightSpec((self.R, h)),
-                   self._name(self.names["correction"]): WeightSpec((self.R,))}
+            out = {self._name(self.names["router"]): WeightSpec((self.R, h))}
+            if self.correct:
+                out[self._name(self.names["correction"])] = WeightSpec((self.R,))
         for e in range(self.E):
             out[self._expert(e, "gate")] = WeightSpec((ff, h))
             out[self._expert(e, "up")] = WeightSpec((ff, h))
@@ -94,7 +110,8 @@ class RoutedExperts(FeedForward):
             r = tensors[self._name(self.names["router"])]
             self.R_pad = -(-self.R // 16) * 16
             self.w_router = torch.cat([r, r.new_zeros(self.R_pad - self.R, self.hidden)], dim=0).contiguous()
-            self.correction = tensors[self._name(self.names["correction"])].float().contiguous()
+            if self.correct:
+                self.correction = tensors[self._name(self.names["correction"])].float().contiguous()
         if self.shared_gate:
             # one row, padded with zero rows to 16 (which every product kernel takes)
             g = tensors[self.shared._name(self.names["shared_gate"])]
@@ -160,7 +177,7 @@ class RoutedExperts(FeedForward):
         else:
             logits = ws.buf("moe_logits", (n, self.R_pad), torch.float32)[:, :self.R]
             ops.gemm(x, self.w_router, ws.buf("moe_logits", (n, self.R_pad), torch.float32))   # 32-bit sums, stored so
-            ops.moe_topk(logits, self.correction, chosen, weights)
+            ops.moe_topk(logits, self.correction, chosen, weights, self.scores, self.renormalize)
         if ops.moe_grouped_takes(x, self.w_gate_up, self.w_down, self.E, self.ff) and x.is_contiguous():
             # bf16: every expert over only the rows that chose it, grouped on the device
             pairs, tiles = n * self.top, ops.moe_grouped_tiles(n, self.top, self.E)
@@ -170,18 +187,25 @@ class RoutedExperts(FeedForward):
                        "num_tiles": ws.buf("moe_num_tiles", (1,), torch.int32),
                        "act": ws.buf("moe_act_rows", (pairs, self.ff), dt),
                        "y": ws.buf("moe_y_rows", (pairs, self.hidden), dt)}
-            ops.moe_grouped(x, self.w_gate_up, self.w_down, chosen, weights, residual, self.E, self.ff, scratch)
+            fresh = step.fresh is residual
+            if fresh:
+                step.fresh = None      # written here instead of added to
+            ops.moe_grouped(x, self.w_gate_up, self.w_down, chosen, weights, residual, self.E, self.ff, scratch,
+                            weigh_input=self.weigh_input, fresh=fresh)
             self._shared_forward(x, step, residual)
             return
         # otherwise (32-bit, or sizes the grouped kernels do not take): every expert over every
         # row in one product, the rows that did not choose it multiplied by an exact zero
-        if self.identity:
+        first = self.identity and step.fresh is not residual
+        if first:
             ops.moe_identity(residual, x, chosen, weights, self.E)
         gu = ws.buf("moe_gate_up", (n, 2 * self.E * self.ff), dt)
         ops.gemm(x, self.w_gate_up, gu)
         act = ws.buf("moe_act", (n, self.E * self.ff), dt)
-        ops.moe_dense_act(gu, chosen, weights, act, self.E, self.ff)
+        ops.moe_dense_act(gu, chosen, weights, act, self.E, self.ff, self.weigh_input)
         add_product(step, act, self.w_down, residual)
+        if self.identity and not first:     # fresh rows are written by the product before they are added to
+            ops.moe_identity(residual, x, chosen, weights, self.E)
         self._shared_forward(x, step, residual)
 
     def _shared_forward(self, x, step, residual) -> None:

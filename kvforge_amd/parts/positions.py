@@ -80,17 +80,22 @@ class RotaryPositions(Positions):
     """Rotary pairs over the first ``rot_dim`` elements of each head.  ``interleaved=False``: the
     checkpoint pairs element ``i`` with ``i + rot_dim/2`` (half-split); ``True``: it pairs element
     ``2i`` with ``2i + 1``, which is the order the kernels rotate in, so that a mixer has nothing
-    to permute.  ``scaling``: ``RopeScaling`` (llama3), ``YarnStretch`` or ``None``."""
+    to permute.  ``scaling``: ``RopeScaling`` (llama3), ``YarnStretch`` or ``None``.  ``rounded_once``:
+    without scaling, the frequencies ``theta^(-2i/rot_dim)`` are formed in 64 bits and rounded to fp32
+    once, instead of by fp32 operations (their error grows with the position in every angle)."""
 
     replayable = True
 
     def __init__(self, rot_dim: int, theta: float, scaling: "RopeScaling | YarnStretch | None" = None,
-                 interleaved: bool = False) -> None:
+                 interleaved: bool = False, rounded_once: bool = False) -> None:
         if rot_dim <= 0 or rot_dim % 2:
             raise ValueError(f"rotary width must be positive and even, got {rot_dim}")
         self.rot_dim, self.theta, self.scaling = int(rot_dim), float(theta), scaling
         self.interleaved = bool(interleaved)
-        self.inv_freq = scaled_inv_freq(self.rot_dim, self.theta, scaling)
+        if rounded_once and scaling is not None:
+            raise ValueError("rounded_once goes without a scaling of the frequencies")
+        self.inv_freq = ((self.theta ** (-2.0 * torch.arange(rot_dim // 2, dtype=torch.float64) / rot_dim)).float()
+                         if rounded_once else scaled_inv_freq(self.rot_dim, self.theta, scaling))
         self.magnitude = rotary_magnitude(scaling)
         self.cos: torch.Tensor | None = None
         self.sin: torch.Tensor | None = None
