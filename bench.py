@@ -652,6 +652,90 @@ def ludelix_points(dtype, batch, prompt_len, steps, warmup, use_graphs=True, onl
     return out
 
 
+# (name, width, heads of the attention layers, kv heads of Buzinex's, their head size, latent heads' plain /
+#  rotated / value size, latent rank, delta memories, q/k heads they share, their key and value size, mamba2
+#  memories, their value size, state size, groups, Buzinex's memories, their size, feed-forward, expert width,
+#  experts, chosen, groups of four layers, vocabulary)
+BALALORN_SIZES = [("w1024", 1024, 16, 4, 64, 64, 32, 64, 192, 8, 4, 128, 128, 32, 64, 128, 4, 16, 64, 4096, 1024, 16, 4, 2, 32000),
+                  ("w2048", 2048, 32, 8, 64, 64, 32, 64, 192, 16, 8, 128, 128, 64, 64, 128, 8, 32, 64, 8192, 2048, 32, 4, 2, 128256),
+                  ("w4096", 4096, 32, 8, 128, 128, 64, 128, 192, 32, 16, 128, 128, 128, 64, 128, 8, 64, 64, 14336, 3584, 32, 4, 1, 128256)]
+BALALORN_FIELDS = ("width", "heads", "kv_heads", "head_dim", "latent_dim", "latent_rot_dim", "latent_vdim", "kv_rank",
+                   "delta_heads", "delta_kv_heads", "delta_dim", "delta_vdim", "ssm_heads", "ssm_vdim", "ssm_state",
+                   "ssm_groups", "wkv_heads", "wkv_dim", "ff", "expert_ff", "experts", "top", "groups", "vocab")
+
+
+def balalorn_points(dtype, batch, prompt_len, steps, warmup, use_graphs=True, only=None, models=None):
+    """Balalorn at a few sizes that resemble a real model's layers (groups of a gated delta rule
+    with a dense feed-forward, latent attention with experts, Mamba-2 with experts, latent
+    attention over the same latents with a dense feed-forward), beside the engine's closest
+    existing model, Buzinex, of the same width, heads, latents, feed-forward (as wide as the chosen
+    experts together) and number of layers; random weights drawn on the device.  Per size and
+    model: ms per decode step, its share of the HBM roofline, tokens a second of a 2,048-token
+    prefill and its share of the matrix-core peak.  A Balalorn decode step has to read: the
+    mixers and dense feed-forwards once, the experts that the batch's tokens are expected to
+    choose (a share ``1 - (1 - top/experts)^batch`` of them), one latent row (``rot_dim + kv_rank``) per
+    token in each latent layer, and every sequence's memories (read and written)."""
+    import torch
+    from kvforge_amd.config.presets import balalorn_stack, buzinex_stack
+
+    elem = 2 if dtype == "bfloat16" else 4
+    out = {}
+    for (name, w, H, KV, d, ld, lr, lv, rank, Hd, Gd, dk, dv, Hs, sv, N, Gs, Hm, dm, ff, eff, E, top, groups,
+         vocab) in BALALORN_SIZES:
+        if only and name not in only:
+            continue
+        bal = balalorn_stack(vocab=vocab, width=w, groups=groups, heads=H, latent_dim=ld, rot_dim=lr, kv_rank=rank,
+                             mem_heads=Hd, mem_kv_heads=Gd, mem_dim=dk, mem_vdim=dv, ssm_heads=Hs, ssm_vdim=sv,
+                             state=N, ssm_groups=Gs, ff=ff, moe_ff=eff, experts=E, top=top, max_positions=CONTEXT_CAP)
+        buz = buzinex_stack(vocab=vocab, width=w, groups=groups, heads=H, kv_heads=KV, dim=d, latent_dim=ld,
+                            rot_dim=lr, kv_rank=rank, window=BUZINEX_WINDOW, wkv_heads=Hm, wkv_dim=dm, ff=ff,
+                            max_positions=CONTEXT_CAP)
+        for layer in bal["layers"] + buz["layers"]:
+            if layer["type"] == "latent_attention":
+                layer["mixer"]["vdim"] = lv
+        latent_q = w * H * (ld + lr) + H * (ld + lv) * rank + H * lv * w
+        latent_kv = w * (rank + lr)
+        delta = w * (2 * Gd * dk + 3 * Hd * dv + 2 * Hd)
+        ssm = w * (3 * Hs * sv + 2 * Gs * N + Hs)
+        routed = 3 * w * eff
+        touched = E * (1.0 - (1.0 - top / E) ** batch)
+        bal_fixed = groups * (delta + ssm + 2 * (latent_q + w * H) + latent_kv + 2 * 3 * w * ff + 2 * w * E)
+        bal_state = groups * (Hd * dk * dv + 3 * (2 * Gd * dk + Hd * dv) + Hs * sv * N + 3 * (Hs * sv + 2 * Gs * N)) * 4 * 2
+        attn = w * d * (2 * H + 2 * KV)
+        memory = 5 * w * Hm * dm + BUZINEX_DECAY_RANK * (w + Hm * dm)
+        buz_fixed = groups * (attn + 2 * (latent_q + latent_kv) + memory + 3 * 3 * w * ff)
+        buz_state = groups * (Hm * dm * dm + w) * 4 * 2
+        n = PREFILL_TOKENS
+        full = n * n / 2.0                                                   # (query, key) pairs, causal
+        seen = min(n, BUZINEX_WINDOW)
+        windowed = n * seen - seen * seen / 2.0
+        per_pair = 2.0 * H * (lr + 2 * rank)                                 # latent scores and sums
+        rows = {"balalorn": (bal, bal_fixed, 2 * groups, 2 * groups * (lr + rank), None, bal_state,
+                             2 * groups * full * per_pair + groups * n * (6.0 * Hd * dk * dv + 4.0 * Hs * sv * N)),
+                "buzinex": (buz, buz_fixed, 0, 2 * groups * (lr + rank), BUZINEX_WINDOW, buz_state,
+                            2 * groups * windowed * per_pair + groups * (full * 4.0 * H * d + n * 4.0 * Hm * dm * dm))}
+        for model, (cfg, fixed, routed_layers, latent_row, window, state_bytes, mixing) in rows.items():
+            if models and model not in models:
+                continue
+            need = batch * (prompt_len + steps + warmup + early_tokens(batch, prompt_len) + 32)
+            engine = build_engine(cfg, dtype, batch, max(need, PREFILL_TOKENS + 64), use_graphs=use_graphs)
+            r = decode_run(engine, vocab, batch, prompt_len, steps, warmup)
+            s = prefill_run(engine, vocab, PREFILL_TOKENS, repeats=2)
+            ctx = min(r["mean_ctx"], window) if window else r["mean_ctx"]
+            keys = r["mean_ctx"] * groups * 2 * KV * d if model == "buzinex" else 0.0
+            read = ((fixed + routed_layers * touched * routed + vocab * w) * elem
+                    + batch * ((ctx * latent_row + keys) * elem + state_bytes))
+            flops = 2.0 * n * (fixed + routed_layers * top * routed) + 2.0 * vocab * w + mixing
+            out[f"{name}_{model}"] = {
+                "decode_ms": round(r["ms_per_step"], 4), "decode_tok_s": round(r["tok_s"], 1),
+                "decode_hbm_frac": round(read / (r["seconds"] / steps) / 1e9 / HBM_PEAK_GBS, 4),
+                "prefill_tok_s": round(PREFILL_TOKENS / s, 1), "prefill_ms": round(s * 1e3, 3),
+                "prefill_frac": round(flops / s / MFMA_PEAK[dtype], 4)}
+            del engine
+            torch.cuda.empty_cache()
+    return out
+
+
 def model_numbers(cfg, layers_run):
     h, H, KV, d, I, V = (cfg["hidden_size"], cfg["num_attention_heads"], cfg["num_key_value_heads"],
                          cfg["head_dim"], cfg["intermediate_size"], cfg["vocab_size"])
@@ -680,7 +764,7 @@ def main() -> int:
     ap.add_argument("--no-graphs", action="store_true")
     ap.add_argument("--decode-run-steps", type=int, default=None,
                     help="decode steps the device takes between two looks of the host (engine default: 8)")
-    ap.add_argument("--phase", choices=["all", "decode", "prefill", "mixed", "burst", "products", "fogorax", "rudorax", "buzinex", "ludelix"],
+    ap.add_argument("--phase", choices=["all", "decode", "prefill", "mixed", "burst", "products", "fogorax", "rudorax", "buzinex", "ludelix", "balalorn"],
                     default="all",
                     help="for profiles: only the decode steps at --batch, or only the prefill; "
                          "mixed: --batch requests with prompts of 128 to 4,096 tokens, chunked "
@@ -691,8 +775,9 @@ def main() -> int:
                          "(launch to launch, so short ones show the host's time); fogorax: the "
                          "Fogorax design at a few layer sizes beside a Llama model of equal sizes; "
                          "rudorax: the Rudorax design likewise (--sizes names some of them); "
-                         "buzinex: the Buzinex design likewise; ludelix: the Ludelix design beside Rudorax")
-    ap.add_argument("--sizes", default="", help="with --phase rudorax, buzinex or ludelix: the sizes to run, with commas")
+                         "buzinex: the Buzinex design likewise; ludelix: the Ludelix design beside Rudorax; "
+                         "balalorn: the Balalorn design beside Buzinex")
+    ap.add_argument("--sizes", default="", help="with --phase rudorax, buzinex, ludelix or balalorn: the sizes to run, with commas")
     args = ap.parse_args()
     if args.gpus != 1:
         print(f"bench.py measures one GPU; --gpus {args.gpus} is not supported by this engine")
@@ -750,6 +835,16 @@ def main() -> int:
                           **ludelix_points(args.dtype, args.batch, args.prompt_len, steps,
                                            min(args.warmup, 8), not args.no_graphs,
                                            [x for x in args.sizes.split(",") if x] or None)}))
+        return 0
+    if args.phase == "balalorn":
+        steps = min(args.steps, 64)
+        print(json.dumps({"phase": "balalorn", "dtype": args.dtype, "batch": args.batch,
+                          "prompt_len": args.prompt_len, "steps": steps, "buzinex_window": BUZINEX_WINDOW,
+                          "prefill_tokens": PREFILL_TOKENS,
+                          "sizes": {r[0]: dict(zip(BALALORN_FIELDS, r[1:])) for r in BALALORN_SIZES},
+                          **balalorn_points(args.dtype, args.batch, args.prompt_len, steps,
+                                            min(args.warmup, 8), not args.no_graphs,
+                                            [x for x in args.sizes.split(",") if x] or None)}))
         return 0
     if args.preset == "small" and args.phase != "burst":
         print("--preset small goes with --phase burst")

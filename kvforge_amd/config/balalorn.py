@@ -19,6 +19,7 @@ from kvforge_amd.config.rudorax import DEFAULT_MAX_POSITIONS, RotaryConfig, _num
 
 MAX_KEY_SIZE = 256     # key size of a memory's head, as the kernels take it
 MAX_TAPS = 8           # taps of a short convolution
+MAX_LATENT_ROW = 640   # rotated key part and latent of a token together, as the attention kernels take them
 
 
 def _taps(d: dict[str, Any], where: str) -> int:
@@ -119,6 +120,8 @@ class GatedLatentConfig:
         rot = RotaryConfig.from_dict(rot, where) if rot else None
         if rot is not None and rot.dims > sizes["rot_dim"]:
             raise ConfigError(f"{where}: rot.dims ({rot.dims}) exceeds rot_dim ({sizes['rot_dim']})")
+        if sizes["rot_dim"] + _positive(d, "kv_rank", where) > MAX_LATENT_ROW:
+            raise ConfigError(f"{where}: rot_dim + kv_rank must not exceed {MAX_LATENT_ROW} (the attention kernels' head size)")
         src = d.get("kv_from")
         if src is not None and (not isinstance(src, int) or isinstance(src, bool) or src < 0):
             raise ConfigError(f"{where}: 'kv_from' must name an earlier layer, got {src!r}")

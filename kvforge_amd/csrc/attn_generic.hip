@@ -1,5 +1,6 @@
 // Paged attention of the true 32-bit path: every product and sum in fp32.  It takes bf16
-// operands as well (widened exactly), for caches whose pages the bf16 kernels do not take.
+// operands as well (widened exactly), for caches whose pages the bf16 kernels do not take and for
+// heads of more than 256 elements (up to 640: one latent row of a wide latent attention).
 //
 // Query runs of any length (attn_mfma32_kernel): fp32 on the matrix cores with
 // v_mfma_f32_16x16x4_f32, which multiplies and adds in fp32.  Row r of a sequence is
@@ -23,6 +24,7 @@
 
 namespace {
 constexpr int ITEM_ROWS = 64;   // rows per work item: four waves of 16
+constexpr int MAX_HEAD = 640;   // elements of a head
 
 // The first key a query at position `pos` sees: with a window w > 0 the key w - 1 before it, with
 // chunks (window < 0, chunks of -window positions counted from position 0) the first key of its
@@ -77,7 +79,7 @@ __global__ __launch_bounds__(256) void attn_mfma32_kernel(
     const int* __restrict__ ctx_lens, const int* __restrict__ work, T* __restrict__ out,
     AttnArgs a) {
   constexpr int DT = DMAX / 16;                // 16-element tiles of the head
-  constexpr int BK = DMAX > 128 ? 32 : 64;     // keys per tile
+  constexpr int BK = DMAX > 256 ? 16 : DMAX > 128 ? 32 : 64;   // keys per tile
   constexpr int ST = BK / 16;                  // 16-key blocks per tile
   constexpr int KLD = DMAX + 4, VLD = BK + 4;  // LDS rows 16 bytes apart in the banks
   constexpr int FLOATS = BK * KLD > DMAX * VLD ? BK * KLD : DMAX * VLD;
@@ -293,7 +295,8 @@ int launch(const void* q, const void* k_pages, const void* v_pages, const int* b
                      static_cast<T*>(out), a)
   if (a.d <= 64) GO(64);
   else if (a.d <= 128) GO(128);
-  else GO(256);
+  else if (a.d <= 256) GO(256);
+  else GO(MAX_HEAD);
 #undef GO
   return kvf_last_error();
 }
@@ -319,8 +322,8 @@ struct DecodeArgs {
   float cap;            // as in AttnArgs
 };
 
-// GT: heads of the group handled together (a power of two, at most 8; a larger group is taken
-// in chunks of 8 heads by workgroups of their own); DQ: elements of the head per lane
+// GT: heads of the group handled together (a power of two, at most 8, or 4 for heads of more than
+// 256 elements; a larger group is taken in chunks of so many heads by workgroups of their own); DQ: elements of the head per lane
 // (ceil(d / 64)).
 template <typename T, int GT, int DQ>
 __global__ __launch_bounds__(DEC_WAVES * KVF_WAVE) void attn_decode_kernel(
@@ -328,7 +331,7 @@ __global__ __launch_bounds__(DEC_WAVES * KVF_WAVE) void attn_decode_kernel(
     const int* __restrict__ block_table, const int* __restrict__ seq_ids,
     const int* __restrict__ cu_q, const int* __restrict__ ctx_lens, T* __restrict__ out,
     float* __restrict__ part_acc, float* __restrict__ part_ml, DecodeArgs a) {
-  __shared__ float Qs[GT][256];
+  __shared__ float Qs[GT][DQ * KVF_WAVE];
   __shared__ float Ps[DEC_WAVES][GT][DEC_KEYS];
   __shared__ float Ms[DEC_WAVES][GT], Ls[DEC_WAVES][GT];
   __shared__ float Os[DEC_WAVES][GT][DQ * KVF_WAVE];
@@ -561,7 +564,9 @@ int launch_decode_g(const void* q, const void* k_pages, const void* v_pages, con
                      static_cast<T*>(out), part_acc, part_ml, a)
   if (a.d <= 64) GO(1);
   else if (a.d <= 128) GO(2);
-  else GO(4);
+  else if (a.d <= 256) GO(4);
+  else if constexpr (GT <= 4) GO(MAX_HEAD / KVF_WAVE);
+  else return static_cast<int>(hipErrorInvalidValue);
 #undef GO
   int code = kvf_last_error();
   if (code != 0 || a.splits == 1) return code;
@@ -580,7 +585,7 @@ int launch_decode(const void* q, const void* k_pages, const void* v_pages, const
                                 part_acc, part_ml, num_seqs, a, s)
   if (G <= 1) GO(1);
   if (G <= 2) GO(2);
-  if (G <= 4) GO(4);
+  if (G <= 4 || a.d > 256) GO(4);
   GO(8);
 #undef GO
 }
@@ -600,7 +605,7 @@ KVF_EXPORT int kvf_attn_generic_decode(int dtype, const void* q, const void* k_p
                                        const float* slopes, const float* sinks, float cap, hipStream_t s) {
   if (num_seqs <= 0) return 0;
   if (!(cap >= 0.f)) return static_cast<int>(hipErrorInvalidValue);
-  if (keep < 0 || d % 16 != 0 || d > 256 || d <= 0 || KV <= 0 || H % KV != 0 || splits < 1 ||
+  if (keep < 0 || d % 16 != 0 || d > MAX_HEAD || d <= 0 || KV <= 0 || H % KV != 0 || splits < 1 ||
       (splits > 1 && (!part_acc || !part_ml)) || block_size <= 0)
     return static_cast<int>(hipErrorInvalidValue);
   DecodeArgs a{H, KV, d, block_size, num_blocks, table_stride, q_stride, o_stride, window, n_seqs,
@@ -614,7 +619,7 @@ KVF_EXPORT int kvf_attn_generic_decode(int dtype, const void* q, const void* k_p
   return static_cast<int>(hipErrorInvalidValue);
 }
 
-// dtype: 0 = fp32, 1 = bf16.  d must be a multiple of 16 and at most 256 (checked by the caller
+// dtype: 0 = fp32, 1 = bf16.  d must be a multiple of 16 and at most 640 (checked by the caller
 // and here).  `work` holds num_work rows (sequence, item, item or -1), an item being
 // kvf_attn_generic_rows_per_item() rows of (query token, head in the kv head's group).
 KVF_EXPORT int kvf_attn_generic(int dtype, const void* q, const void* k_pages, const void* v_pages,
@@ -624,7 +629,7 @@ KVF_EXPORT int kvf_attn_generic(int dtype, const void* q, const void* k_pages, c
                                 int o_stride, int window, int keep, int n_seqs, float scale,
                                 const float* slopes, const float* sinks, float cap, hipStream_t s) {
   if (!(cap >= 0.f)) return static_cast<int>(hipErrorInvalidValue);
-  if (keep < 0 || d % 16 != 0 || d > 256 || d <= 0 || KV <= 0 || H % KV != 0 || !work || block_size <= 0 ||
+  if (keep < 0 || d % 16 != 0 || d > MAX_HEAD || d <= 0 || KV <= 0 || H % KV != 0 || !work || block_size <= 0 ||
       q_stride % 4 != 0 || o_stride % 4 != 0)
     return static_cast<int>(hipErrorInvalidValue);
   AttnArgs a{H, KV, d, block_size, num_blocks, table_stride, q_stride, o_stride, window, n_seqs,

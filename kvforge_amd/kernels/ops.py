@@ -1057,9 +1057,12 @@ def set_gemm_waves(waves: int, rows: int = 0) -> None:
 
 
 # ------------------------------------------------------------------------------ attention
+ATTENTION_MAX_HEAD = 640     # elements of a head; beyond 256 the fp32 kernels alone
+
+
 def _attn_common(q, k_pages, v_pages, block_table, cu_q, ctx_lens, out, H, KV, d):
-    if d % 16 or d > 256 or d <= 0:
-        raise KernelError(f"attention kernels take head sizes in steps of 16 up to 256, got {d}")
+    if d % 16 or d > ATTENTION_MAX_HEAD or d <= 0:
+        raise KernelError(f"attention kernels take head sizes in steps of 16 up to {ATTENTION_MAX_HEAD}, got {d}")
     if H % KV:
         raise KernelError(f"query heads ({H}) must be a multiple of kv heads ({KV})")
     _check(q, "q", None, (None, None), contiguous=False)
@@ -1143,17 +1146,17 @@ def _gate_args(gate, q: torch.Tensor, cols: int):
     return gate.data_ptr(), gate.stride(0)
 
 
-def attention_on_matrix_cores(dtype: torch.dtype, block_size: int) -> bool:
-    """The MFMA attention kernels take bf16 and pages of a multiple of 8 tokens; everything else
-    (the true 32-bit path above all) runs the vector-ALU kernel."""
-    return dtype == BF16 and block_size % 8 == 0
+def attention_on_matrix_cores(dtype: torch.dtype, block_size: int, head_dim: int) -> bool:
+    """The bf16 MFMA attention kernels take bf16, pages of a multiple of 8 tokens and heads of up to
+    256 elements; everything else (the true 32-bit path above all) runs the fp32 kernels."""
+    return dtype == BF16 and block_size % 8 == 0 and head_dim <= 256
 
 
 def prefill_rows_per_item(dtype: torch.dtype, head_dim: int, block_size: int, row_tiles: int = 1) -> int:
     """Rows of (query token, head in group) that one entry of a prefill work list covers.
     ``row_tiles``: 1 or 2 tiles of 16 rows per wave of the matrix-core kernel (two where the head
     size allows them; they pay when the work fills the chip anyway, see ``attn_mfma.hip``)."""
-    if attention_on_matrix_cores(dtype, block_size):
+    if attention_on_matrix_cores(dtype, block_size, head_dim):
         return int(_fn("attn_mfma", "kvf_attn_mfma_rows_per_item", [c_int, c_int])(int(head_dim), int(row_tiles)))
     return int(_fn("attn_generic", "kvf_attn_generic_rows_per_item", [])())
 
@@ -1168,7 +1171,7 @@ def prefill_blocks_per_cu(dtype: torch.dtype, head_dim: int, block_size: int, ro
     key = (dtype, int(head_dim), int(block_size) % 8 == 0, int(row_tiles))
     if key not in _blocks_per_cu:
         n = 4
-        if attention_on_matrix_cores(dtype, block_size):
+        if attention_on_matrix_cores(dtype, block_size, head_dim):
             n = int(_fn("attn_mfma", "kvf_attn_mfma_prefill_blocks_per_cu", [c_int, c_int])(int(head_dim), int(row_tiles)))
         _blocks_per_cu[key] = max(1, n)
     return _blocks_per_cu[key]
@@ -1202,7 +1205,7 @@ def attn_prefill(q: torch.Tensor, k_pages: torch.Tensor, v_pages: torch.Tensor,
     H, KV, d = num_heads, num_kv_heads, head_dim
     window = _mask_arg(window, chunk)
     n_seqs = _attn_common(q, k_pages, v_pages, block_table, cu_q, ctx_lens, out, H, KV, d)
-    cap = _score_cap(score_cap, sinks, slopes, attention_on_matrix_cores(q.dtype, k_pages.shape[2]))
+    cap = _score_cap(score_cap, sinks, slopes, attention_on_matrix_cores(q.dtype, k_pages.shape[2], d))
     _check(work, "work", I32, (None, 3))
     keep = _keep_first(window, keep_first)
     gp, gs = _gate_args(gate, q, H * d)
@@ -1211,8 +1214,8 @@ def attn_prefill(q: torch.Tensor, k_pages: torch.Tensor, v_pages: torch.Tensor,
     nb, _, bs, _ = k_pages.shape
     if rows_per_item is None:
         rows_per_item = prefill_rows_per_item(q.dtype, d, bs)
-    _no_sinks_with_slopes(sinks, slopes, attention_on_matrix_cores(q.dtype, bs))
-    if attention_on_matrix_cores(q.dtype, bs):
+    _no_sinks_with_slopes(sinks, slopes, attention_on_matrix_cores(q.dtype, bs, d))
+    if attention_on_matrix_cores(q.dtype, bs, d):
         if window < 0 and (sinks is not None or slopes is not None or cap > 0.0):
             raise KernelError("attn_prefill: the matrix-core kernel has chunks of positions with plain scores "
                               "only (no sinks, slopes or score cap beside them)")
@@ -1261,7 +1264,7 @@ def attn_decode(q: torch.Tensor, k_pages: torch.Tensor, v_pages: torch.Tensor,
     H, KV, d = num_heads, num_kv_heads, head_dim
     window = _mask_arg(window, chunk)
     n_seqs = _attn_common(q, k_pages, v_pages, block_table, cu_q, ctx_lens, out, H, KV, d)
-    cap = _score_cap(score_cap, sinks, slopes, attention_on_matrix_cores(q.dtype, k_pages.shape[2]))
+    cap = _score_cap(score_cap, sinks, slopes, attention_on_matrix_cores(q.dtype, k_pages.shape[2], d))
     sl = _slopes_ptr(slopes, H, q)
     sk = _sinks_ptr(sinks, H, q)
     keep = _keep_first(window, keep_first)
@@ -1286,8 +1289,8 @@ def attn_decode(q: torch.Tensor, k_pages: torch.Tensor, v_pages: torch.Tensor,
         _check(pm, "workspace[1]", F32)
         if pa.numel() < num_seqs * H * splits * d or pm.numel() < num_seqs * H * splits * 2:
             raise KernelError("attn_decode: workspace too small")
-    _no_sinks_with_slopes(sinks, slopes, attention_on_matrix_cores(q.dtype, bs))
-    if not attention_on_matrix_cores(q.dtype, bs):
+    _no_sinks_with_slopes(sinks, slopes, attention_on_matrix_cores(q.dtype, bs, d))
+    if not attention_on_matrix_cores(q.dtype, bs, d):
         if gate is not None:
             raise KernelError("attn_decode: the 32-bit kernel takes no gate; gate its rows afterwards")
         f = _fn("attn_generic", "kvf_attn_generic_decode",

@@ -461,14 +461,14 @@ class PagedAttention(Mixer):
         work, rows_per_item = self._prefill_work(step, act, bs)
         gate = qkv[:, g0:g0 + H * d] if self.gated else None
         # the matrix-core kernels gate their output as they store it
-        gate_in_kernel = gate if gate is not None and ops.attention_on_matrix_cores(act, bs) else None
+        gate_in_kernel = gate if gate is not None and ops.attention_on_matrix_cores(act, bs, d) else None
         if work is not None:
             ops.attn_prefill(qkv, layer.k_pages, layer.v_pages, table, step.cu_q, step.ctx_lens,
                              work, out, H, KV, d, self.scale, window, self.slopes, rows_per_item,
                              keep_first=self.keep_first, gate=gate_in_kernel, sinks=self.sinks,
                              score_cap=self.score_cap, chunk=chunk)
         if step.n_decode:
-            splits = self._decode_cuts(step, ops.attention_on_matrix_cores(act, bs))
+            splits = self._decode_cuts(step, ops.attention_on_matrix_cores(act, bs, d))
             workspace = None
             if splits > 1:
                 workspace = (ws.buf("decode_part_acc", (step.n_decode * H * splits * d,), torch.float32),

@@ -11,7 +11,8 @@ queries are taken through ``W_uk_h^T`` once (``ops.head_product``), attention ru
 key/value head over pages of ``[k_r | c]`` (the built-in paged kernels, window and sink
 included), and the weighted sums of ``c`` are read out per head by ``W_uv_h`` before the output
 projection.  A page row is ``rot_dim + kv_rank`` elements (rounded up to the kernels' step of
-16) whatever the number of heads.
+16) whatever the number of heads; rows of more than 256 elements (up to 640) take the fp32 attention
+kernels in either mode.
 """
 
 from __future__ import annotations
@@ -51,9 +52,9 @@ class LatentAttention(PagedAttention):
             raise ValueError(f"latent attention: sizes must be positive, got heads {num_heads}, "
                              f"{head_dim} + {rot_dim}, values {value_dim}, rank {kv_rank}")
         self.d = -(-(self.rot + self.rank) // 16) * 16
-        if self.d > 256:
-            raise ValueError(f"attention kernels take heads up to 256 elements; rot_dim + kv_rank is "
-                             f"{self.rot + self.rank}")
+        if self.d > ops.ATTENTION_MAX_HEAD:
+            raise ValueError(f"attention kernels take heads up to {ops.ATTENTION_MAX_HEAD} elements; rot_dim + "
+                             f"kv_rank is {self.rot + self.rank}")
         self.dk = self.dv = self.d
         self.rotary = rotary
         if rotary is not None and (rotary.rot_dim > self.rot or not rotary.interleaved):
@@ -152,7 +153,7 @@ class LatentAttention(PagedAttention):
             ops.attn_prefill(qkv, layer.k_pages, layer.v_pages, table, step.cu_q, step.ctx_lens, work,
                              out, H, 1, d, self.scale, window, None, rows_per_item, sinks=self.sinks)
         if step.n_decode:
-            splits = self._decode_cuts(step, ops.attention_on_matrix_cores(act, bs))
+            splits = self._decode_cuts(step, ops.attention_on_matrix_cores(act, bs, d))
             workspace = None
             if splits > 1:
                 workspace = (ws.buf("decode_part_acc", (step.n_decode * H * splits * d,), torch.float32),

@@ -52,14 +52,9 @@ def silu(x: torch.Tensor) -> torch.Tensor:
 def short_conv(x: torch.Tensor, taps: torch.Tensor, bias: torch.Tensor | None) -> torch.Tensor:
     """``y_t[c] = silu(sum_j taps[c, j] x_(t - (n - 1) + j)[c] + bias[c])`` for ``n`` taps, the last of
     which meets the token itself; inputs before the first token are zeros."""
-    T, C = x.shape
     n = taps.shape[1]
-    y = x.new_zeros(T, C)
-    for t in range(T):
-        for j in range(n):
-            s = t - (n - 1) + j
-            if s >= 0:
-                y[t] += taps[:, j] * x[s]
+    before = torch.cat([x.new_zeros(n - 1, x.shape[1]), x])
+    y = torch.stack([(taps.T * before[t:t + n]).sum(0) for t in range(x.shape[0])])
     if bias is not None:
         y = y + bias
     return silu(y)
@@ -70,19 +65,22 @@ def unit(x: torch.Tensor) -> torch.Tensor:
 
 
 # ---------------------------------------------------------------------------------- memories
+def of_group(x: torch.Tensor, heads: int) -> torch.Tensor:
+    """``x [T, G, n]`` as ``[T, heads, n]``: head ``h`` gets group ``h // (heads / G)``'s."""
+    return x.repeat_interleave(heads // x.shape[1], dim=1)
+
+
 def delta_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, g: torch.Tensor, beta: torch.Tensor) -> torch.Tensor:
     """``q, k [T, G, dk]`` (head ``h`` uses ``h // (H / G)``), ``v [T, H, dv]``, ``g, beta [T, H]``."""
     T, H, dv = v.shape
-    G, dk = q.shape[1], q.shape[2]
+    q, k = of_group(q, H), of_group(k, H)
+    S = v.new_zeros(H, q.shape[2], dv)
     out = v.new_zeros(T, H, dv)
-    for h in range(H):
-        a = h // (H // G)
-        S = v.new_zeros(dk, dv)
-        for t in range(T):
-            S = g[t, h] * S
-            u = beta[t, h] * (v[t, h] - S.T @ k[t, a])
-            S = S + torch.outer(k[t, a], u)
-            out[t, h] = S.T @ q[t, a]
+    for t in range(T):
+        S = g[t][:, None, None] * S
+        u = beta[t][:, None] * (v[t] - (S * k[t][:, :, None]).sum(1))
+        S = S + k[t][:, :, None] * u[:, None, :]
+        out[t] = (S * q[t][:, :, None]).sum(1)
     return out
 
 
@@ -90,14 +88,12 @@ def ssd_scan(C: torch.Tensor, B: torch.Tensor, x: torch.Tensor, a: torch.Tensor,
     """``C, B [T, G, N]`` (head ``h`` uses group ``h // (H / G)``), ``x [T, H, dv]``, decays ``a`` and
     step sizes ``dt [T, H]``: ``S_t = a_t S_(t-1) + dt_t B_t x_t^T``, ``y_t = S_t^T C_t``."""
     T, H, dv = x.shape
-    G, N = B.shape[1], B.shape[2]
+    B, C = of_group(B, H), of_group(C, H)
+    S = x.new_zeros(H, B.shape[2], dv)
     out = x.new_zeros(T, H, dv)
-    for h in range(H):
-        g = h // (H // G)
-        S = x.new_zeros(N, dv)
-        for t in range(T):
-            S = a[t, h] * S + dt[t, h] * torch.outer(B[t, g], x[t, h])
-            out[t, h] = S.T @ C[t, g]
+    for t in range(T):
+        S = a[t][:, None, None] * S + dt[t][:, None, None] * B[t][:, :, None] * x[t][:, None, :]
+        out[t] = (S * C[t][:, :, None]).sum(1)
     return out
 
 
