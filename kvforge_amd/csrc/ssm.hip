@@ -335,26 +335,72 @@ __device__ __forceinline__ void chunk_gates(const float* __restrict__ z, const S
   }
 }
 
-// rows tb .. tb + cnt - 1 of a head of q or k (columns off .. off + dk - 1) into LDS, [CL][DKP + 4],
-// zeros past the tokens and past dk
-template <int DKP, int CL>
-__device__ __forceinline__ void stage_rows(const float* __restrict__ rows, const SsmArgs& a, int off, int tb, int cnt,
-                                           float* dst) {
-  constexpr int QLD = DKP + 4;
-  if (a.dk % 4 == 0 && a.ld % 4 == 0 && off % 4 == 0) {
-    for (int i = threadIdx.x; i < CL * (DKP / 4); i += blockDim.x) {
-      const int t = i / (DKP / 4), e = 4 * (i - t * (DKP / 4));
-      f32x4 v = zero4();
-      if (t < cnt && e < a.dk) v = *reinterpret_cast<const f32x4*>(rows + static_cast<size_t>(tb + t) * a.ld + off + e);
-      *reinterpret_cast<f32x4*>(dst + t * QLD + e) = v;
-    }
+// Loads on their way into LDS are never predicated: a lane without an element of its own reads the
+// rows' first one and the value is cleared when it is put down, so that no load waits for another.
+//
+// Four neighbouring elements e .. e + 3 of a head's row p; VEC: heads and rows start on 16 bytes and dk
+// is a multiple of four, so that they are one load and lie inside the row or outside it together.
+template <bool VEC>
+__device__ __forceinline__ f32x4 load_four(const float* __restrict__ safe, const float* p, int e, int dk, bool ok) {
+  if constexpr (VEC) {
+    return *reinterpret_cast<const f32x4*>(ok && e < dk ? p + e : safe);
   } else {
-    for (int i = threadIdx.x; i < CL * DKP; i += blockDim.x) {
-      const int t = i / DKP, e = i - t * DKP;
-      dst[t * QLD + e] = (t < cnt && e < a.dk) ? rows[static_cast<size_t>(tb + t) * a.ld + off + e] : 0.f;
-    }
+    f32x4 v;
+#pragma unroll
+    for (int y = 0; y < 4; ++y) v[y] = *(ok && e + y < dk ? p + e + y : safe);
+    return v;
   }
 }
+__device__ __forceinline__ f32x4 clear_past(f32x4 v, int e, int dk, bool ok) {
+#pragma unroll
+  for (int y = 0; y < 4; ++y) v[y] = ok && e + y < dk ? v[y] : 0.f;
+  return v;
+}
+
+// Rows tb .. tb + cnt - 1 of a head of q or k (columns off .. off + dk - 1) on their way from memory into
+// LDS, [CL][DKP + 4], by NT threads: all loads are asked for (`ask`) before the first is put down
+// (`put`).  Zeros past the tokens and past dk.
+template <int DKP, int CL, int NT, bool VEC> struct StagedRows {
+  static constexpr int N = CL * (DKP / 4) / NT;
+  static constexpr int ROWS = NT / (DKP / 4);     // a round's rows; a thread has the same elements in every round
+  static_assert(N >= 1 && N * NT == CL * (DKP / 4) && ROWS * (DKP / 4) == NT, "whole rounds of threads");
+  f32x4 v[N];
+  __device__ __forceinline__ void ask(const float* __restrict__ rows, const SsmArgs& a, int off, int tb, int cnt) {
+    const int t0 = threadIdx.x / (DKP / 4), e = 4 * (threadIdx.x % (DKP / 4));
+    const float* p = rows + static_cast<size_t>(tb + t0) * a.ld + off;
+    const size_t step = static_cast<size_t>(ROWS) * a.ld;
+#pragma unroll
+    for (int x = 0; x < N; ++x, p += step) v[x] = load_four<VEC>(rows, p, e, a.dk, t0 + ROWS * x < cnt);
+  }
+  __device__ __forceinline__ void put(float* dst, int cnt, int dk) const {
+    const int t0 = threadIdx.x / (DKP / 4), e = 4 * (threadIdx.x % (DKP / 4));
+    float* d = dst + t0 * (DKP + 4) + e;
+#pragma unroll
+    for (int x = 0; x < N; ++x)
+      *reinterpret_cast<f32x4*>(d + x * ROWS * (DKP + 4)) = clear_past(v[x], e, dk, t0 + ROWS * x < cnt);
+  }
+};
+
+// COLS columns of R rows of `ld` floats from p on, on their way into LDS turned round, [COLS][LLD]:
+// element (r, c) lies at c * LLD + r.  Zeros past `rows_ok` rows and `cols_ok` columns (both at least one).
+template <int R, int COLS, int NT, int LLD> struct StagedTurned {
+  static constexpr int N = R * COLS / NT, ROWS = NT / COLS;
+  static_assert(N >= 1 && N * NT == R * COLS && ROWS * COLS == NT, "whole rounds of threads");
+  float v[N];
+  __device__ __forceinline__ void ask(const float* __restrict__ p, size_t ld, int rows_ok, int cols_ok) {
+    const int r0 = threadIdx.x / COLS, c = threadIdx.x % COLS;
+    const float* q = p + static_cast<size_t>(r0) * ld + c;
+#pragma unroll
+    for (int x = 0; x < N; ++x, q += static_cast<size_t>(ROWS) * ld)
+      v[x] = *(r0 + ROWS * x < rows_ok && c < cols_ok ? q : p);
+  }
+  __device__ __forceinline__ void put(float* dst, int rows_ok, int cols_ok) const {
+    const int r0 = threadIdx.x / COLS, c = threadIdx.x % COLS;
+    float* d = dst + c * LLD + r0;
+#pragma unroll
+    for (int x = 0; x < N; ++x) d[x * ROWS] = r0 + ROWS * x < rows_ok && c < cols_ok ? v[x] : 0.f;
+  }
+};
 
 // acc += A B^T over k = 0 .. K - 1 (K a multiple of 16): `ra` and `rb` point at the lane's row of
 // either operand, at element 4 (l / 16)
@@ -365,8 +411,20 @@ __device__ __forceinline__ f32x4 mma16(const float* ra, const float* rb, f32x4 a
   return acc;
 }
 template <int K> __device__ __forceinline__ f32x4 mma_rows(const float* ra, const float* rb, f32x4 acc) {
-#pragma unroll 4
-  for (int k0 = 0; k0 < K; k0 += 16) acc = mma16(ra + k0, rb + k0, acc);
+  constexpr int AHEAD = K < 128 ? K / 16 : 8;      // steps whose operands are asked for together
+#pragma unroll
+  for (int k0 = 0; k0 < K; k0 += 16 * AHEAD) {
+    f32x4 a4[AHEAD], b4[AHEAD];
+#pragma unroll
+    for (int u = 0; u < AHEAD; ++u) {
+      a4[u] = *reinterpret_cast<const f32x4*>(ra + k0 + 16 * u);
+      b4[u] = *reinterpret_cast<const f32x4*>(rb + k0 + 16 * u);
+    }
+#pragma unroll
+    for (int u = 0; u < AHEAD; ++u)
+#pragma unroll
+      for (int e = 0; e < 4; ++e) acc = __builtin_amdgcn_mfma_f32_16x16x4f32(a4[u][e], b4[u][e], acc, 0, 0, 0);
+  }
   return acc;
 }
 __device__ __forceinline__ f32x4 mma_rows(const float* ra, const float* rb, int K, f32x4 acc) {
@@ -375,13 +433,13 @@ __device__ __forceinline__ f32x4 mma_rows(const float* ra, const float* rb, int 
 }
 
 // chunks: rows (sequence, first token, tokens, 0).  T [chunks, H, CL, CL]: blocks above the diagonal
-// are not written.
-template <int DKP, int CL>
+// are not written.  B [chunks, H, 2, CL]: e^(b_t), then e^(b_L - b_t) (zero past the chunk's tokens).
+template <int DKP, int CL, bool VEC>
 __global__ __launch_bounds__(256) void ssm_solve_kernel(const float* __restrict__ rows, const float* __restrict__ z,
                                                         const float* __restrict__ neg_a,
                                                         const float* __restrict__ dt_bias,
                                                         const int* __restrict__ chunks, float* __restrict__ T,
-                                                        SsmArgs a) {
+                                                        float* __restrict__ B, SsmArgs a) {
   extern __shared__ __align__(16) float lds[];
   constexpr int QLD = DKP + 4, TLD = CL + 4, RT = CL / 16;
   double* bc = reinterpret_cast<double*>(lds);   // [CL]
@@ -392,8 +450,17 @@ __global__ __launch_bounds__(256) void ssm_solve_kernel(const float* __restrict_
   const int chunk = blockIdx.y, head = blockIdx.x, kh = head / (a.H / a.G);
   const int tb = chunks[4 * chunk + 1], cnt = chunks[4 * chunk + 2];
   const int tid = threadIdx.x, lane = tid % KVF_WAVE, wave = tid / KVF_WAVE, l16 = lane % 16, lq = lane / 16;
-  stage_rows<DKP, CL>(rows, a, a.k_off + kh * a.dk, tb, cnt, Ks);
-  if (wave == 0) chunk_gates<true, CL>(z, a, head, neg_a[head], dt_bias[head], tb, cnt, bc, sw);
+  StagedRows<DKP, CL, 256, VEC> ks;
+  ks.ask(rows, a, a.k_off + kh * a.dk, tb, cnt);
+  if (wave == 0) {
+    chunk_gates<true, CL>(z, a, head, neg_a[head], dt_bias[head], tb, cnt, bc, sw);
+    if (lane < CL) {
+      float* Bg = B + (static_cast<size_t>(chunk) * a.H + head) * 2 * CL;
+      Bg[lane] = expf(static_cast<float>(bc[lane]));
+      Bg[CL + lane] = lane < cnt ? expf(static_cast<float>(bc[CL - 1] - bc[lane])) : 0.f;
+    }
+  }
+  ks.put(Ks, cnt, a.dk);
   __syncthreads();
   for (int tile = wave; tile < RT * RT; tile += 4) {
     const int rt = tile / RT, ct = tile - rt * RT;
@@ -452,18 +519,16 @@ __global__ __launch_bounds__(256) void ssm_solve_kernel(const float* __restrict_
 }
 
 // runs: rows (sequence, first chunk, chunks).  Workgroup (16 value columns, head, run).  A chunk's K,
-// T and V are asked for while the chunk before is worked on.  W [chunks, H, dk, dv] receives the
+// T, V and B are asked for while the chunk before is worked on.  W [chunks, H, dk, dv] receives the
 // state before every chunk, U [tokens, H, dv] the chunks' u.
 constexpr int DCOLS = 16;
-template <int DKP, int CL>
-__global__ __launch_bounds__(256) void ssm_delta_kernel(const float* __restrict__ rows, const float* __restrict__ z,
-                                                        const float* __restrict__ neg_a,
-                                                        const float* __restrict__ dt_bias,
-                                                        const int* __restrict__ chunks, const int* __restrict__ runs,
+template <int DKP, int CL, bool VEC>
+__global__ __launch_bounds__(256) void ssm_delta_kernel(const float* __restrict__ rows, const int* __restrict__ chunks,
+                                                        const int* __restrict__ runs,
                                                         const int* __restrict__ positions,
                                                         const int* __restrict__ slot_ids, float* __restrict__ state,
-                                                        const float* __restrict__ T, float* __restrict__ W,
-                                                        float* __restrict__ U, SsmArgs a) {
+                                                        const float* __restrict__ T, const float* __restrict__ B,
+                                                        float* __restrict__ W, float* __restrict__ U, SsmArgs a) {
   extern __shared__ __align__(16) float lds[];
   constexpr int QLD = DKP + 4, TLD = CL + 4, RT = CL / 16;
   float* eb = lds;                               // [CL] e^(b_t)
@@ -472,7 +537,7 @@ __global__ __launch_bounds__(256) void ssm_delta_kernel(const float* __restrict_
   float* Tb = Ks + CL * QLD;                     // [CL][TLD]
   float* Vt = Tb + CL * TLD;                     // [DCOLS][TLD]
   float* Rt = Vt + DCOLS * TLD;                  // [DCOLS][TLD]
-  float* Ut = Rt + DCOLS * TLD;                  // [DCOLS][TLD]
+  float* Ut = Rt + DCOLS * TLD;                  // [DCOLS][TLD] u times wl
   float* St = Ut + DCOLS * TLD;                  // [DCOLS][QLD]
   const int head = blockIdx.y, col0 = blockIdx.x * DCOLS, kh = head / (a.H / a.G);
   const int seq = runs[3 * blockIdx.z], c0 = runs[3 * blockIdx.z + 1], nc = runs[3 * blockIdx.z + 2];
@@ -487,68 +552,35 @@ __global__ __launch_bounds__(256) void ssm_delta_kernel(const float* __restrict_
     const int r = i / DCOLS, cl = i % DCOLS, c = col0 + cl;
     St[cl * QLD + r] = (resume && r < dk && c < dv) ? S_slot[static_cast<size_t>(r) * dv + c] : 0.f;
   }
-  const float na = neg_a[head], db = dt_bias[head];
   const int k_off = a.k_off + kh * dk, v_off = a.v_off + head * dv;
-  const bool vec = dk % 4 == 0 && a.ld % 4 == 0 && k_off % 4 == 0;
-  constexpr int NK = CL * DKP / 4 / 256, NT = CL * CL / 4 / 256, NV = CL * DCOLS / 256;
-  f32x4 kreg[NK], treg[NT];
-  float vreg[NV], zreg = 0.f;
-  auto ask = [&](int ch) {
-    const int tb = chunks[4 * ch + 1], cnt = chunks[4 * ch + 2];
-#pragma unroll
-    for (int x = 0; x < NK; ++x) {
-      const int i = tid + 256 * x, t = i / (DKP / 4), e = 4 * (i - t * (DKP / 4));
-      const float* p = rows + static_cast<size_t>(tb + t) * a.ld + k_off + e;
-      kreg[x] = zero4();
-      if (t < cnt) {
-        if (vec) {
-          if (e < dk) kreg[x] = *reinterpret_cast<const f32x4*>(p);
-        } else {
-#pragma unroll
-          for (int y = 0; y < 4; ++y)
-            if (e + y < dk) kreg[x][y] = p[y];
-        }
-      }
-    }
+  constexpr int NT = CL * CL / 4 / 256;
+  StagedRows<DKP, CL, 256, VEC> ks;
+  StagedTurned<CL, DCOLS, 256, TLD> vs;
+  f32x4 treg[NT];
+  float breg = 0.f;
+  auto ask = [&](int ch, int tb, int cnt) {
+    ks.ask(rows, a, k_off, tb, cnt);
     const float* Tg = T + (static_cast<size_t>(ch) * a.H + head) * CL * CL;
 #pragma unroll
     for (int x = 0; x < NT; ++x) treg[x] = *reinterpret_cast<const f32x4*>(Tg + 4 * (tid + 256 * x));
-#pragma unroll
-    for (int x = 0; x < NV; ++x) {
-      const int i = tid + 256 * x, t = i / DCOLS, c = col0 + i % DCOLS;
-      vreg[x] = (t < cnt && c < dv) ? rows[static_cast<size_t>(tb + t) * a.ld + v_off + c] : 0.f;
-    }
-    if (wave == 0) zreg = lane < cnt ? z[static_cast<size_t>(tb + lane) * a.z_ld + a.a_off + head] : 0.f;
+    vs.ask(rows + static_cast<size_t>(tb) * a.ld + v_off + col0, a.ld, cnt, dv - col0);
+    breg = B[(static_cast<size_t>(ch) * a.H + head) * 2 * CL + tid % (2 * CL)];
   };
-  ask(c0);
+  int tb = chunks[4 * c0 + 1], cnt = chunks[4 * c0 + 2];
+  ask(c0, tb, cnt);
   for (int j = 0; j < nc; ++j) {
-    const int ch = c0 + j, tb = chunks[4 * ch + 1], cnt = chunks[4 * ch + 2];
+    const int ch = c0 + j;
+    // the next chunk's place, asked for early
+    const int tb_next = j + 1 < nc ? chunks[4 * (ch + 1) + 1] : 0, cnt_next = j + 1 < nc ? chunks[4 * (ch + 1) + 2] : 0;
     __syncthreads();   // the chunk before is done with everything
+    ks.put(Ks, cnt, dk);
 #pragma unroll
-    for (int x = 0; x < NK; ++x) {
-      const int i = tid + 256 * x, t = i / (DKP / 4), e = 4 * (i - t * (DKP / 4));
-      *reinterpret_cast<f32x4*>(Ks + t * QLD + e) = kreg[x];
-    }
-#pragma unroll
-    for (int x = 0; x < NT; ++x) {
-      const int i = 4 * (tid + 256 * x), t = i / CL, s = i - t * CL;
-      *reinterpret_cast<f32x4*>(Tb + t * TLD + s) = treg[x];
-    }
-#pragma unroll
-    for (int x = 0; x < NV; ++x) {
-      const int i = tid + 256 * x;
-      Vt[(i % DCOLS) * TLD + i / DCOLS] = vreg[x];
-    }
-    if (wave == 0) {
-      const double b = running_sum(lane < cnt ? na * softplus(zreg + db) : 0.f);
-      const double b_last = __shfl(b, KVF_WAVE - 1, KVF_WAVE);
-      if (lane < CL) {
-        eb[lane] = expf(static_cast<float>(b));
-        wl[lane] = lane < cnt ? expf(static_cast<float>(b_last - b)) : 0.f;
-      }
-    }
+    for (int x = 0; x < NT; ++x)
+      *reinterpret_cast<f32x4*>(Tb + (4 * tid / CL + x * (1024 / CL)) * TLD + 4 * tid % CL) = treg[x];
+    vs.put(Vt, cnt, dv - col0);
+    if (tid < 2 * CL) eb[tid] = breg;            // (wl lies behind eb)
     __syncthreads();
-    if (j + 1 < nc) ask(ch + 1);
+    if (j + 1 < nc) ask(ch + 1, tb_next, cnt_next);
     // R = V - diag(e^b) K S
     if (wave < RT) {
       const f32x4 acc = mma_rows<DKP>(Ks + (16 * wave + l16) * QLD + 4 * lq, St + l16 * QLD + 4 * lq, zero4());
@@ -561,12 +593,22 @@ __global__ __launch_bounds__(256) void ssm_delta_kernel(const float* __restrict_
       *reinterpret_cast<f32x4*>(Rt + l16 * TLD + t) = r;
     }
     __syncthreads();
-    // U = T R
+    // U = T R, over the blocks of T up to the diagonal
     if (wave < RT) {
-      const f32x4 u = mma_rows(Tb + (16 * wave + l16) * TLD + 4 * lq, Rt + l16 * TLD + 4 * lq, 16 * (wave + 1),
-                               zero4());
       const int t = 16 * wave + 4 * lq, c = col0 + l16;
-      *reinterpret_cast<f32x4*>(Ut + l16 * TLD + t) = u;
+      f32x4 a4[RT], b4[RT], u = zero4();
+#pragma unroll
+      for (int k = 0; k < RT; ++k) {
+        a4[k] = *reinterpret_cast<const f32x4*>(Tb + (16 * wave + l16) * TLD + 16 * k + 4 * lq);
+        b4[k] = *reinterpret_cast<const f32x4*>(Rt + l16 * TLD + 16 * k + 4 * lq);
+      }
+#pragma unroll
+      for (int k = 0; k < RT; ++k) {
+        if (k > wave) break;
+#pragma unroll
+        for (int e = 0; e < 4; ++e) u = __builtin_amdgcn_mfma_f32_16x16x4f32(a4[k][e], b4[k][e], u, 0, 0, 0);
+      }
+      *reinterpret_cast<f32x4*>(Ut + l16 * TLD + t) = u * *reinterpret_cast<const f32x4*>(wl + t);
 #pragma unroll
       for (int v = 0; v < 4; ++v)
         if (t + v < cnt && c < dv) U[(static_cast<size_t>(tb + t + v) * a.H + head) * dv + c] = u[v];
@@ -575,26 +617,33 @@ __global__ __launch_bounds__(256) void ssm_delta_kernel(const float* __restrict_
     // S <- e^(b_L) S + K^T diag(e^(b_L - b)) U; the state as it was goes to W
     const float g_last = eb[CL - 1];
     float* Wg = W + (static_cast<size_t>(ch) * a.H + head) * dk * dv;
+    f32x4 b4[RT];
+#pragma unroll
+    for (int k = 0; k < RT; ++k) b4[k] = *reinterpret_cast<const f32x4*>(Ut + l16 * TLD + 16 * k + 4 * lq);
     for (int kt = wave; kt < DKP / 16; kt += 4) {
       f32x4* mine = reinterpret_cast<f32x4*>(St + l16 * QLD + 16 * kt + 4 * lq);
+      const float* ka = Ks + (4 * lq) * QLD + 16 * kt + l16;
+      float kv[RT][4];
+#pragma unroll
+      for (int k = 0; k < RT; ++k)
+#pragma unroll
+        for (int e = 0; e < 4; ++e) kv[k][e] = ka[(16 * k + e) * QLD];
       const f32x4 old = *mine;
+      f32x4 acc = old * g_last;
+#pragma unroll
+      for (int k = 0; k < RT; ++k)
+#pragma unroll
+        for (int e = 0; e < 4; ++e) acc = __builtin_amdgcn_mfma_f32_16x16x4f32(kv[k][e], b4[k][e], acc, 0, 0, 0);
       const int c = col0 + l16;
 #pragma unroll
       for (int v = 0; v < 4; ++v) {
         const int r = 16 * kt + 4 * lq + v;
         if (r < dk && c < dv) Wg[static_cast<size_t>(r) * dv + c] = old[v];
       }
-      f32x4 acc = old * g_last;
-      const float* ka = Ks + (4 * lq) * QLD + 16 * kt + l16;
-      const float* ub = Ut + l16 * TLD + 4 * lq;
-#pragma unroll
-      for (int k0 = 0; k0 < CL; k0 += 16) {
-        const f32x4 b4 = *reinterpret_cast<const f32x4*>(ub + k0) * *reinterpret_cast<const f32x4*>(wl + k0 + 4 * lq);
-#pragma unroll
-        for (int e = 0; e < 4; ++e) acc = __builtin_amdgcn_mfma_f32_16x16x4f32(ka[(k0 + e) * QLD], b4[e], acc, 0, 0, 0);
-      }
       *mine = acc;
     }
+    tb = tb_next;
+    cnt = cnt_next;
   }
   __syncthreads();
   if (S_slot != nullptr) {
@@ -608,7 +657,7 @@ __global__ __launch_bounds__(256) void ssm_delta_kernel(const float* __restrict_
 // The plain form's chunks alone: W [chunks, H, dk, dv] = K^T diag(e^(b_L - b_s) s_s) V, and E [chunks, H] =
 // e^(b_L).  Workgroup (64 value columns, head, chunk).
 constexpr int VCOLS = 64;
-template <int DKP, int CL>
+template <int DKP, int CL, bool VEC>
 __global__ __launch_bounds__(256) void ssm_local_kernel(const float* __restrict__ rows, const float* __restrict__ z,
                                                         const float* __restrict__ neg_a,
                                                         const float* __restrict__ dt_bias,
@@ -625,36 +674,47 @@ __global__ __launch_bounds__(256) void ssm_local_kernel(const float* __restrict_
   const int tb = chunks[4 * chunk + 1], cnt = chunks[4 * chunk + 2];
   const int tid = threadIdx.x, lane = tid % KVF_WAVE, wave = tid / KVF_WAVE, l16 = lane % 16, lq = lane / 16;
   const int dk = a.dk, dv = a.dv;
-  stage_rows<DKP, CL>(rows, a, a.k_off + kh * dk, tb, cnt, Ks);
-  for (int i = tid; i < CL * VCOLS; i += 256) {
-    const int t = i / VCOLS, cl = i % VCOLS, c = col0 + cl;
-    Vt[cl * TLD + t] = (t < cnt && c < dv) ? rows[static_cast<size_t>(tb + t) * a.ld + a.v_off + head * dv + c] : 0.f;
-  }
+  StagedRows<DKP, CL, 256, VEC> ks;
+  StagedTurned<CL, VCOLS, 256, TLD> vs;
+  ks.ask(rows, a, a.k_off + kh * dk, tb, cnt);
+  vs.ask(rows + static_cast<size_t>(tb) * a.ld + a.v_off + head * dv + col0, a.ld, cnt, dv - col0);
   if (wave == 0) {
     chunk_gates<false, CL>(z, a, head, neg_a[head], dt_bias[head], tb, cnt, bc, sw);
     if (lane < CL) wl[lane] = sw[lane] * expf(static_cast<float>(bc[CL - 1] - bc[lane]));
     if (lane == 0 && blockIdx.x == 0)
       E[static_cast<size_t>(chunk) * a.H + head] = expf(static_cast<float>(bc[CL - 1]));
   }
+  ks.put(Ks, cnt, dk);
+  vs.put(Vt, cnt, dv - col0);
   __syncthreads();
   float* Wg = W + (static_cast<size_t>(chunk) * a.H + head) * dk * dv;
-  const int col_tiles = min(VCOLS / 16, (dv - col0 + 15) / 16), row_tiles = (dk + 15) / 16;
-  for (int tile = wave; tile < row_tiles * col_tiles; tile += 4) {
-    const int kt = tile / col_tiles, ct = tile - kt * col_tiles;
-    f32x4 acc = zero4();
+  const int col_tiles = min(VCOLS / 16, (dv - col0 + 15) / 16);
+  constexpr int RT = CL / 16;
+  for (int kt = wave; 16 * kt < dk; kt += 4) {
+    // the tile's rows of K^T, weighted, serve all column tiles
     const float* ka = Ks + (4 * lq) * QLD + 16 * kt + l16;
-    const float* vb = Vt + (16 * ct + l16) * TLD + 4 * lq;
+    float kv[RT][4];
 #pragma unroll
-    for (int k0 = 0; k0 < CL; k0 += 16) {
-      const f32x4 b4 = *reinterpret_cast<const f32x4*>(vb + k0) * *reinterpret_cast<const f32x4*>(wl + k0 + 4 * lq);
+    for (int k = 0; k < RT; ++k) {
+      const f32x4 w4 = *reinterpret_cast<const f32x4*>(wl + 16 * k + 4 * lq);
 #pragma unroll
-      for (int e = 0; e < 4; ++e) acc = __builtin_amdgcn_mfma_f32_16x16x4f32(ka[(k0 + e) * QLD], b4[e], acc, 0, 0, 0);
+      for (int e = 0; e < 4; ++e) kv[k][e] = ka[(16 * k + e) * QLD] * w4[e];
     }
-    const int c = col0 + 16 * ct + l16;
+    for (int ct = 0; ct < col_tiles; ++ct) {
+      f32x4 acc = zero4();
+      const float* vb = Vt + (16 * ct + l16) * TLD + 4 * lq;
 #pragma unroll
-    for (int v = 0; v < 4; ++v) {
-      const int r = 16 * kt + 4 * lq + v;
-      if (r < dk && c < dv) Wg[static_cast<size_t>(r) * dv + c] = acc[v];
+      for (int k = 0; k < RT; ++k) {
+        const f32x4 b4 = *reinterpret_cast<const f32x4*>(vb + 16 * k);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) acc = __builtin_amdgcn_mfma_f32_16x16x4f32(kv[k][e], b4[e], acc, 0, 0, 0);
+      }
+      const int c = col0 + 16 * ct + l16;
+#pragma unroll
+      for (int v = 0; v < 4; ++v) {
+        const int r = 16 * kt + 4 * lq + v;
+        if (r < dk && c < dv) Wg[static_cast<size_t>(r) * dv + c] = acc[v];
+      }
     }
   }
 }
@@ -701,45 +761,57 @@ __global__ __launch_bounds__(256) void ssm_carry_kernel(const int* __restrict__ 
 
 // Workgroup of eight waves (64 value columns, head, chunk): the chunk's outputs from the state
 // before it (W) and its u (U, or for the plain form v itself with the steps among the weights).
-template <int DKP, int CL, bool DELTA>
-__global__ __launch_bounds__(512) void ssm_read_kernel(const float* __restrict__ rows, const float* __restrict__ z,
-                                                       const float* __restrict__ neg_a,
-                                                       const float* __restrict__ dt_bias,
-                                                       const float* __restrict__ Dskip, const int* __restrict__ chunks,
-                                                       const float* __restrict__ W, const float* __restrict__ U,
-                                                       float* __restrict__ out, SsmArgs a) {
+// Wave w has the chunk's rows 16 (w % RT) .. + 15, whose q it keeps in registers for both products;
+// K's place in LDS takes the state's columns once the weights are made.
+template <int DKP, int CL, bool DELTA, bool VEC>
+__global__ __launch_bounds__(512, DKP <= 128 ? 4 : 2) void ssm_read_kernel(
+    const float* __restrict__ rows, const float* __restrict__ z, const float* __restrict__ neg_a,
+    const float* __restrict__ dt_bias, const float* __restrict__ Dskip, const int* __restrict__ chunks,
+    const float* __restrict__ W, const float* __restrict__ U, float* __restrict__ out, SsmArgs a) {
   extern __shared__ __align__(16) float lds[];
-  constexpr int QLD = DKP + 4, TLD = CL + 4, RT = CL / 16, KS = CL > VCOLS ? CL : VCOLS;
+  constexpr int QLD = DKP + 4, TLD = CL + 4, RT = CL / 16, KS = CL > VCOLS ? CL : VCOLS, SHARES = 8 / RT;
   double* bc = reinterpret_cast<double*>(lds);   // [CL]
   float* sw = lds + 2 * CL;                      // [CL]
   float* eb = sw + CL;                           // [CL]
-  float* Qs = eb + CL;                           // [CL][QLD]
-  float* Ks = Qs + CL * QLD;                     // [CL][QLD], then the state's columns [VCOLS][QLD]
+  float* Ks = eb + CL;                           // [CL][QLD], then the state's columns [VCOLS][QLD]
   float* As = Ks + KS * QLD;                     // [CL][TLD]
   float* Ut = As + CL * TLD;                     // [VCOLS][TLD]
   const int chunk = blockIdx.z, head = blockIdx.y, col0 = blockIdx.x * VCOLS, kh = head / (a.H / a.G);
   const int tb = chunks[4 * chunk + 1], cnt = chunks[4 * chunk + 2];
   const int tid = threadIdx.x, lane = tid % KVF_WAVE, wave = tid / KVF_WAVE, l16 = lane % 16, lq = lane / 16;
-  const int dk = a.dk, dv = a.dv;
-  stage_rows<DKP, CL>(rows, a, a.q_off + kh * dk, tb, cnt, Qs);
-  stage_rows<DKP, CL>(rows, a, a.k_off + kh * dk, tb, cnt, Ks);
-  for (int i = tid; i < CL * VCOLS; i += 512) {
-    const int t = i / VCOLS, cl = i % VCOLS, c = col0 + cl;
-    float v = 0.f;
-    if (t < cnt && c < dv)
-      v = DELTA ? U[(static_cast<size_t>(tb + t) * a.H + head) * dv + c]
-                : rows[static_cast<size_t>(tb + t) * a.ld + a.v_off + head * dv + c];
-    Ut[cl * TLD + t] = v;
+  const int dk = a.dk, dv = a.dv, rt = wave % RT, share = wave / RT;
+  StagedRows<DKP, CL, 512, VEC> ks;
+  StagedTurned<CL, VCOLS, 512, TLD> us;
+  StagedTurned<DKP, VCOLS, 512, QLD> ws;
+  ks.ask(rows, a, a.k_off + kh * dk, tb, cnt);
+  f32x4 q4[DKP / 16];
+  const bool q_ok = 16 * rt + l16 < cnt;
+  {
+    const float* p = rows + static_cast<size_t>(tb + 16 * rt + l16) * a.ld + a.q_off + kh * dk;
+#pragma unroll
+    for (int u = 0; u < DKP / 16; ++u) q4[u] = load_four<VEC>(rows, p, 16 * u + 4 * lq, dk, q_ok);
   }
+  if (DELTA) us.ask(U + (static_cast<size_t>(tb) * a.H + head) * dv + col0, static_cast<size_t>(a.H) * dv, cnt, dv - col0);
+  else us.ask(rows + static_cast<size_t>(tb) * a.ld + a.v_off + head * dv + col0, a.ld, cnt, dv - col0);
+  ws.ask(W + (static_cast<size_t>(chunk) * a.H + head) * dk * dv + col0, dv, dk, dv - col0);
   if (wave == 0) {
     chunk_gates<DELTA, CL>(z, a, head, neg_a[head], dt_bias[head], tb, cnt, bc, sw);
     if (lane < CL) eb[lane] = expf(static_cast<float>(bc[lane]));
   }
+  ks.put(Ks, cnt, dk);
+  us.put(Ut, cnt, dv - col0);
+#pragma unroll
+  for (int u = 0; u < DKP / 16; ++u) q4[u] = clear_past(q4[u], 16 * u + 4 * lq, dk, q_ok);
   __syncthreads();
-  for (int tile = wave; tile < RT * RT; tile += 8) {
-    const int rt = tile / RT, ct = tile - rt * RT;
-    if (ct > rt) continue;
-    const f32x4 acc = mma_rows<DKP>(Qs + (16 * rt + l16) * QLD + 4 * lq, Ks + (16 * ct + l16) * QLD + 4 * lq, zero4());
+  for (int ct = share; ct <= rt; ct += SHARES) {
+    f32x4 acc = zero4();
+    const float* kb = Ks + (16 * ct + l16) * QLD + 4 * lq;
+#pragma unroll
+    for (int u = 0; u < DKP / 16; ++u) {
+      const f32x4 b4 = *reinterpret_cast<const f32x4*>(kb + 16 * u);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) acc = __builtin_amdgcn_mfma_f32_16x16x4f32(q4[u][e], b4[e], acc, 0, 0, 0);
+    }
     const int s = 16 * ct + l16;
 #pragma unroll
     for (int v = 0; v < 4; ++v) {
@@ -753,20 +825,21 @@ __global__ __launch_bounds__(512) void ssm_read_kernel(const float* __restrict__
     }
   }
   __syncthreads();   // K is read; its place takes the state
-  const float* Wg = W + (static_cast<size_t>(chunk) * a.H + head) * dk * dv;
-  for (int i = tid; i < DKP * VCOLS; i += 512) {
-    const int r = i / VCOLS, cl = i % VCOLS, c = col0 + cl;
-    Ks[cl * QLD + r] = (r < dk && c < dv) ? Wg[static_cast<size_t>(r) * dv + c] : 0.f;
-  }
+  ws.put(Ks, dk, dv - col0);
   __syncthreads();
   const float dskip = Dskip ? Dskip[head] : 0.f;
-  const int col_tiles = min(VCOLS / 16, (dv - col0 + 15) / 16);
-  for (int tile = wave; tile < RT * col_tiles; tile += 8) {
-    const int rt = tile / col_tiles, ct = tile - rt * col_tiles;
-    f32x4 acc = mma_rows<DKP>(Qs + (16 * rt + l16) * QLD + 4 * lq, Ks + (16 * ct + l16) * QLD + 4 * lq, zero4());
-    const int t4 = 16 * rt + 4 * lq;
-    acc *= *reinterpret_cast<const f32x4*>(eb + t4);
-    acc = mma_rows(As + (16 * rt + l16) * TLD + 4 * lq, Ut + (16 * ct + l16) * TLD + 4 * lq, 16 * (rt + 1), acc);
+  const int col_tiles = min(VCOLS / 16, (dv - col0 + 15) / 16), t4 = 16 * rt + 4 * lq;
+  const f32x4 e4 = *reinterpret_cast<const f32x4*>(eb + t4);
+  for (int ct = share; ct < col_tiles; ct += SHARES) {
+    f32x4 acc = zero4();
+    const float* sb = Ks + (16 * ct + l16) * QLD + 4 * lq;
+#pragma unroll
+    for (int u = 0; u < DKP / 16; ++u) {
+      const f32x4 b4 = *reinterpret_cast<const f32x4*>(sb + 16 * u);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) acc = __builtin_amdgcn_mfma_f32_16x16x4f32(q4[u][e], b4[e], acc, 0, 0, 0);
+    }
+    acc = mma_rows(As + (16 * rt + l16) * TLD + 4 * lq, Ut + (16 * ct + l16) * TLD + 4 * lq, 16 * (rt + 1), acc * e4);
     const int c = col0 + 16 * ct + l16;
 #pragma unroll
     for (int v = 0; v < 4; ++v) {
@@ -785,7 +858,7 @@ template <int DKP, int CL> constexpr size_t delta_lds() {
 }
 template <int DKP, int CL> constexpr size_t local_lds() { return 4 * (4 * CL + CL * (DKP + 4) + VCOLS * (CL + 4)); }
 template <int DKP, int CL> constexpr size_t read_lds() {
-  return 4 * (4 * CL + CL * (DKP + 4) + (CL > VCOLS ? CL : VCOLS) * (DKP + 4) + CL * (CL + 4) + VCOLS * (CL + 4));
+  return 4 * (4 * CL + (CL > VCOLS ? CL : VCOLS) * (DKP + 4) + CL * (CL + 4) + VCOLS * (CL + 4));
 }
 
 // more LDS than a kernel gets unasked is asked for once per kernel
@@ -797,83 +870,134 @@ template <typename F> hipError_t allow_lds(F* kernel, size_t bytes) {
 struct ChunkPtrs {
   const float *rows, *z, *neg_a, *dt_bias, *dskip;
   const int *positions, *slot_ids, *chunks, *runs;
-  float *state, *out, *T, *W, *U, *E;
+  float *state, *out, *T, *B, *W, *U, *E;
   int n_chunks, n_runs;
 };
 
-template <int DKP, int CL>
+template <int DKP, int CL, bool VEC>
 int chunks_go(bool delta, const ChunkPtrs& p, SsmArgs a, hipStream_t s) {
   static bool allowed = false;
+  constexpr size_t lds_solve = solve_lds<DKP, CL>(), lds_delta = delta_lds<DKP, CL>(), lds_local = local_lds<DKP, CL>(),
+                   lds_read = read_lds<DKP, CL>();
   if (!allowed) {
-    hipError_t e = allow_lds(&ssm_solve_kernel<DKP, CL>, solve_lds<DKP, CL>());
-    if (e == hipSuccess) e = allow_lds(&ssm_delta_kernel<DKP, CL>, delta_lds<DKP, CL>());
-    if (e == hipSuccess) e = allow_lds(&ssm_local_kernel<DKP, CL>, local_lds<DKP, CL>());
-    if (e == hipSuccess) e = allow_lds(&ssm_read_kernel<DKP, CL, true>, read_lds<DKP, CL>());
-    if (e == hipSuccess) e = allow_lds(&ssm_read_kernel<DKP, CL, false>, read_lds<DKP, CL>());
+    hipError_t e = allow_lds(&ssm_solve_kernel<DKP, CL, VEC>, lds_solve);
+    if (e == hipSuccess) e = allow_lds(&ssm_delta_kernel<DKP, CL, VEC>, lds_delta);
+    if (e == hipSuccess) e = allow_lds(&ssm_local_kernel<DKP, CL, VEC>, lds_local);
+    if (e == hipSuccess) e = allow_lds(&ssm_read_kernel<DKP, CL, true, VEC>, lds_read);
+    if (e == hipSuccess) e = allow_lds(&ssm_read_kernel<DKP, CL, false, VEC>, lds_read);
     if (e != hipSuccess) return static_cast<int>(e);
     allowed = true;
   }
-  const unsigned slices = static_cast<unsigned>((a.dv + VCOLS - 1) / VCOLS);
-  constexpr size_t lds_solve = solve_lds<DKP, CL>(), lds_delta = delta_lds<DKP, CL>(), lds_local = local_lds<DKP, CL>(),
-                   lds_read = read_lds<DKP, CL>();
+  const dim3 slices((a.dv + VCOLS - 1) / VCOLS, a.H, p.n_chunks);
   if (delta) {
-    hipLaunchKernelGGL((ssm_solve_kernel<DKP, CL>), dim3(a.H, p.n_chunks), dim3(256), lds_solve, s, p.rows, p.z,
-                       p.neg_a, p.dt_bias, p.chunks, p.T, a);
-    hipLaunchKernelGGL((ssm_delta_kernel<DKP, CL>), dim3((a.dv + DCOLS - 1) / DCOLS, a.H, p.n_runs), dim3(256),
-                       lds_delta, s, p.rows, p.z, p.neg_a, p.dt_bias, p.chunks, p.runs, p.positions, p.slot_ids,
-                       p.state, p.T, p.W, p.U, a);
-    hipLaunchKernelGGL((ssm_read_kernel<DKP, CL, true>), dim3(slices, a.H, p.n_chunks), dim3(512), lds_read, s, p.rows,
-                       p.z, p.neg_a, p.dt_bias, p.dskip, p.chunks, p.W, p.U, p.out, a);
+    hipLaunchKernelGGL((ssm_solve_kernel<DKP, CL, VEC>), dim3(a.H, p.n_chunks), dim3(256), lds_solve, s, p.rows, p.z,
+                       p.neg_a, p.dt_bias, p.chunks, p.T, p.B, a);
+    hipLaunchKernelGGL((ssm_delta_kernel<DKP, CL, VEC>), dim3((a.dv + DCOLS - 1) / DCOLS, a.H, p.n_runs), dim3(256),
+                       lds_delta, s, p.rows, p.chunks, p.runs, p.positions, p.slot_ids, p.state, p.T, p.B, p.W, p.U,
+                       a);
+    hipLaunchKernelGGL((ssm_read_kernel<DKP, CL, true, VEC>), slices, dim3(512), lds_read, s, p.rows, p.z, p.neg_a,
+                       p.dt_bias, p.dskip, p.chunks, p.W, p.U, p.out, a);
   } else {
-    hipLaunchKernelGGL((ssm_local_kernel<DKP, CL>), dim3(slices, a.H, p.n_chunks), dim3(256), lds_local, s, p.rows,
-                       p.z, p.neg_a, p.dt_bias, p.chunks, p.W, p.E, a);
+    hipLaunchKernelGGL((ssm_local_kernel<DKP, CL, VEC>), slices, dim3(256), lds_local, s, p.rows, p.z, p.neg_a,
+                       p.dt_bias, p.chunks, p.W, p.E, a);
     hipLaunchKernelGGL(ssm_carry_kernel, dim3((a.dk * a.dv + 255) / 256, a.H, p.n_runs), dim3(256), 0, s, p.chunks,
                        p.runs, p.positions, p.slot_ids, p.state, p.W, p.E, a);
-    hipLaunchKernelGGL((ssm_read_kernel<DKP, CL, false>), dim3(slices, a.H, p.n_chunks), dim3(512), lds_read, s,
-                       p.rows, p.z, p.neg_a, p.dt_bias, p.dskip, p.chunks, p.W, p.U, p.out, a);
+    hipLaunchKernelGGL((ssm_read_kernel<DKP, CL, false, VEC>), slices, dim3(512), lds_read, s, p.rows, p.z, p.neg_a,
+                       p.dt_bias, p.dskip, p.chunks, p.W, p.U, p.out, a);
   }
   return kvf_last_error();
 }
 
 // ---------------------------------------------------------------------------------- gate and norm
 // out[t, :] = w * u / sqrt(mean(u^2) + eps), u = y silu(z), the mean over each of `parts` equal parts of
-// the row.  Workgroup (token, part).
-template <typename T>
+// the row.  Workgroup (token, part), or with fewer threads a part.  A thread takes eight neighbouring
+// elements a load where the rows and parts allow it (V = 8), else one.
+template <typename T, int V>
 __global__ __launch_bounds__(256) void ssm_gate_norm_kernel(const float* __restrict__ y, const T* __restrict__ z,
                                                             int z_ld, const float* __restrict__ w, float eps,
                                                             T* __restrict__ out, int inner, int size) {
   __shared__ float scratch[16];
-  const int t = blockIdx.x, c0 = blockIdx.y * size;
+  const int t = blockIdx.x, c0 = blockIdx.y * size, step = V * blockDim.x;
   const float* yr = y + static_cast<size_t>(t) * inner + c0;
   const T* zr = z + static_cast<size_t>(t) * z_ld + c0;
   T* o = out + static_cast<size_t>(t) * inner + c0;
-  constexpr int N = 8;      // parts of up to 2,048 elements stay in registers
-  float u[N];
+  auto gated = [&](int i, float (&u)[V]) {
+    float g[V];
+    if constexpr (V == 8) {
+      load8(yr + i, u);
+      load8(zr + i, g);
+    } else {
+      u[0] = yr[i];
+      g[0] = Elem<T>::load(zr + i);
+    }
+#pragma unroll
+    for (int e = 0; e < V; ++e) u[e] *= g[e] * sigmoidf(g[e]);
+  };
+  constexpr int N = V == 8 ? 2 : 8;      // what a thread keeps in registers (the rest is formed twice)
+  float u[N][V];
   float ss = 0.f;
 #pragma unroll
   for (int k = 0; k < N; ++k) {
-    const int i = threadIdx.x + 256 * k;
-    u[k] = 0.f;
-    if (i < size) {
-      const float g = Elem<T>::load(zr + i);
-      u[k] = yr[i] * (g * sigmoidf(g));
-      ss = fmaf(u[k], u[k], ss);
-    }
+    const int i = V * threadIdx.x + step * k;
+    if (i >= size) continue;
+    gated(i, u[k]);
+#pragma unroll
+    for (int e = 0; e < V; ++e) ss = fmaf(u[k][e], u[k][e], ss);
   }
-  for (int i = threadIdx.x + 256 * N; i < size; i += 256) {
-    const float g = Elem<T>::load(zr + i), v = yr[i] * (g * sigmoidf(g));
-    ss = fmaf(v, v, ss);
+  for (int i = V * threadIdx.x + step * N; i < size; i += step) {
+    float v[V];
+    gated(i, v);
+#pragma unroll
+    for (int e = 0; e < V; ++e) ss = fmaf(v[e], v[e], ss);
   }
   const float r = 1.f / sqrtf(block_sum(ss, scratch) / static_cast<float>(size) + eps);
+  auto put = [&](int i, const float (&v)[V]) {
+    if constexpr (V == 8) {
+      float wv[8];
+      load8(w + c0 + i, wv);
+#pragma unroll
+      for (int e = 0; e < 8; ++e) wv[e] *= v[e] * r;
+      if constexpr (sizeof(T) == 4) {
+        *reinterpret_cast<float4*>(o + i) = make_float4(wv[0], wv[1], wv[2], wv[3]);
+        *reinterpret_cast<float4*>(o + i + 4) = make_float4(wv[4], wv[5], wv[6], wv[7]);
+      } else {
+        uint32_t p[4];
+#pragma unroll
+        for (int e = 0; e < 4; ++e)
+          p[e] = static_cast<uint32_t>(f32_to_bf16(wv[2 * e])) | (static_cast<uint32_t>(f32_to_bf16(wv[2 * e + 1])) << 16);
+        *reinterpret_cast<uint4*>(o + i) = make_uint4(p[0], p[1], p[2], p[3]);
+      }
+    } else {
+      Elem<T>::store(o + i, v[0] * r * w[c0 + i]);
+    }
+  };
 #pragma unroll
   for (int k = 0; k < N; ++k) {
-    const int i = threadIdx.x + 256 * k;
-    if (i < size) Elem<T>::store(o + i, u[k] * r * w[c0 + i]);
+    const int i = V * threadIdx.x + step * k;
+    if (i < size) put(i, u[k]);
   }
-  for (int i = threadIdx.x + 256 * N; i < size; i += 256) {
-    const float g = Elem<T>::load(zr + i), v = yr[i] * (g * sigmoidf(g));
-    Elem<T>::store(o + i, v * r * w[c0 + i]);
+  for (int i = V * threadIdx.x + step * N; i < size; i += step) {
+    float v[V];
+    gated(i, v);
+    put(i, v);
   }
+}
+
+template <typename T>
+int gate_norm_launch(const float* y, const void* z, int z_ld, const float* w, float eps, void* out, int n, int inner,
+                     int parts, hipStream_t s) {
+  const int size = inner / parts;
+  const auto on = [](const void* p, size_t bytes) { return reinterpret_cast<uintptr_t>(p) % bytes == 0; };
+  const T* zt = static_cast<const T*>(z);
+  T* o = static_cast<T*>(out);
+  if (size % 8 == 0 && z_ld % 8 == 0 && on(y, 32) && on(z, 8 * sizeof(T)) && on(w, 32) && on(out, 16)) {
+    const int need = (size / 8 + KVF_WAVE - 1) / KVF_WAVE * KVF_WAVE;
+    hipLaunchKernelGGL((ssm_gate_norm_kernel<T, 8>), dim3(n, parts), dim3(need < 256 ? need : 256), 0, s, y, zt, z_ld, w,
+                       eps, o, inner, size);
+  } else {
+    hipLaunchKernelGGL((ssm_gate_norm_kernel<T, 1>), dim3(n, parts), dim3(256), 0, s, y, zt, z_ld, w, eps, o, inner, size);
+  }
+  return kvf_last_error();
 }
 
 bool args_ok(const SsmArgs& a, bool delta) {
@@ -938,34 +1062,33 @@ KVF_EXPORT int kvf_ssm_scan(SSM_ARGS_DECL, const int* cu_q, int n_seqs, int chun
 
 // The runs named in `runs` (sequence, first chunk, chunks), cut into `chunks` (sequence, first token,
 // tokens, 0; at most kvf_ssm_chunk_len(dk) tokens each, a run's chunks in order and one after another).
-// Scratch: W [n_chunks, H, dk, dv]; for the delta rule T [n_chunks, H, CL, CL] and U [tokens, H, dv]; for the
+// Scratch: W [n_chunks, H, dk, dv]; for the delta rule T [n_chunks, H, CL, CL], B [n_chunks, H, 2, CL] and
+// U [tokens, H, dv]; for the
 // plain form E [n_chunks, H].
 KVF_EXPORT int kvf_ssm_chunks(SSM_ARGS_DECL, const int* chunks, int n_chunks, const int* runs, int n_runs, float* T,
-                              float* W, float* U, float* E, hipStream_t s) {
+                              float* B, float* W, float* U, float* E, hipStream_t s) {
   if (n_chunks <= 0 || n_runs <= 0) return 0;
   const SsmArgs a{H, G, dk, dv, ld, q_off, k_off, v_off, z_ld, a_off, b_off, n_slots, slot_floats, 0};
   if (!args_ok(a, delta != 0) || n_chunks > 65535 || n_runs > 65535 || !chunks || !runs || !W ||
-      (delta ? (!T || !U) : !E))
+      (delta ? (!T || !B || !U) : !E))
     return static_cast<int>(hipErrorInvalidValue);
-  const ChunkPtrs p{rows, z, neg_a, dt_bias, dskip, positions, slot_ids, chunks, runs, state, out, T, W, U, E,
+  const ChunkPtrs p{rows, z, neg_a, dt_bias, dskip, positions, slot_ids, chunks, runs, state, out, T, B, W, U, E,
                     n_chunks, n_runs};
-  if (dk <= 32) return chunks_go<32, 64>(delta != 0, p, a, s);
-  if (dk <= 64) return chunks_go<64, 64>(delta != 0, p, a, s);
-  if (dk <= 128) return chunks_go<128, 64>(delta != 0, p, a, s);
-  return chunks_go<256, 32>(delta != 0, p, a, s);
+  const bool vec = dk % 4 == 0 && ld % 4 == 0 && q_off % 4 == 0 && k_off % 4 == 0 &&
+                   reinterpret_cast<uintptr_t>(rows) % 16 == 0;
+#define GO(DKP, CL) return vec ? chunks_go<DKP, CL, true>(delta != 0, p, a, s) : chunks_go<DKP, CL, false>(delta != 0, p, a, s)
+  if (dk <= 32) GO(32, 64);
+  if (dk <= 64) GO(64, 64);
+  if (dk <= 128) GO(128, 64);
+  GO(256, 32);
+#undef GO
 }
 
 KVF_EXPORT int kvf_ssm_gate_norm(int dtype, const float* y, const void* z, int z_ld, const float* w, float eps, void* out,
                                  int n, int inner, int parts, hipStream_t s) {
   if (n <= 0) return 0;
   if (inner <= 0 || parts <= 0 || inner % parts || parts > 65535) return static_cast<int>(hipErrorInvalidValue);
-  if (dtype == 0)
-    hipLaunchKernelGGL(ssm_gate_norm_kernel<float>, dim3(n, parts), dim3(256), 0, s, y, static_cast<const float*>(z), z_ld,
-                       w, eps, static_cast<float*>(out), inner, inner / parts);
-  else if (dtype == 1)
-    hipLaunchKernelGGL(ssm_gate_norm_kernel<bf16_t>, dim3(n, parts), dim3(256), 0, s, y, static_cast<const bf16_t*>(z),
-                       z_ld, w, eps, static_cast<bf16_t*>(out), inner, inner / parts);
-  else
-    return static_cast<int>(hipErrorInvalidValue);
-  return kvf_last_error();
+  if (dtype == 0) return gate_norm_launch<float>(y, z, z_ld, w, eps, out, n, inner, parts, s);
+  if (dtype == 1) return gate_norm_launch<bf16_t>(y, z, z_ld, w, eps, out, n, inner, parts, s);
+  return static_cast<int>(hipErrorInvalidValue);
 }

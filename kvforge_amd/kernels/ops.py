@@ -1946,7 +1946,7 @@ def ssm_scratch(n_tokens: int, n_chunks: int, heads: int, key_dim: int, value_di
     H, dk, dv, cl = int(heads), int(key_dim), int(value_dim), ssm_chunk_len(key_dim)
     out = {"W": ((n_chunks, H, dk, dv), F32)}
     if delta:
-        out.update({"T": ((n_chunks, H, cl, cl), F32), "U": ((n_tokens, H, dv), F32)})
+        out.update({"T": ((n_chunks, H, cl, cl), F32), "B": ((n_chunks, H, 2, cl), F32), "U": ((n_tokens, H, dv), F32)})
     else:
         out["E"] = ((n_chunks, H), F32)
     return out
@@ -2050,9 +2050,9 @@ def ssm_scan(rows: torch.Tensor, q_off: int, k_off: int, v_off: int, gates: torc
     nc = chunks.shape[0]
     for name, (shape, dtype) in ssm_scratch(n, nc, H, dk, dv, delta).items():
         _check(multi[name], name, dtype, shape)
-    f = _fn("ssm", "kvf_ssm_chunks", types + [c_void_p, c_int, c_void_p, c_int] + [c_void_p] * 5)
+    f = _fn("ssm", "kvf_ssm_chunks", types + [c_void_p, c_int, c_void_p, c_int] + [c_void_p] * 6)
     _ok(f(*common, chunks.data_ptr(), nc, runs.data_ptr(), runs.shape[0],
-          *(multi[k].data_ptr() if k in multi else None for k in ("T", "W", "U", "E")), _stream()), "ssm_chunks")
+          *(multi[k].data_ptr() if k in multi else None for k in ("T", "B", "W", "U", "E")), _stream()), "ssm_chunks")
 
 
 def ssm_gate_norm(y: torch.Tensor, gate: torch.Tensor, weight: torch.Tensor, eps: float, parts: int,
