@@ -32,8 +32,12 @@ __global__ __launch_bounds__(256) void latent_split_kernel(const T* __restrict__
   const T* in = proj + static_cast<size_t>(n) * ld_in;
   T* out = qkv + static_cast<size_t>(n) * ld_out;
   const T* down = in + H * (dim + rot);
+  // few tokens: a token's heads are shared among workgroups, of which the first has the key and value
+  const int h0 = static_cast<int>(static_cast<long>(H) * blockIdx.y / gridDim.y);
+  const int h1 = static_cast<int>(static_cast<long>(H) * (blockIdx.y + 1) / gridDim.y);
+  const bool own = w != nullptr && blockIdx.y == 0;
   float r = 0.f;
-  if (w != nullptr) {   // the same for the whole grid
+  if (own) {   // the same for the whole workgroup
     float ss = 0.f;
     for (int i = tid; i < rank; i += blockDim.x) {
       const float v = Elem<T>::load(down + i);
@@ -42,14 +46,14 @@ __global__ __launch_bounds__(256) void latent_split_kernel(const T* __restrict__
     r = 1.f / sqrtf(block_sum(ss, scratch) / static_cast<float>(rank) + eps);
   }
   // q heads: the rotated part to the front, zeros behind what head_product fills
-  for (int i = tid; i < H * d; i += blockDim.x) {
+  for (int i = h0 * d + tid; i < h1 * d; i += blockDim.x) {
     const int h = i / d, e = i - h * d;
     if (e < rot)
       out[i] = in[h * (dim + rot) + dim + e];
     else if (e >= rot + rank || dim == 0)   // (heads without a plain part: nothing fills the middle)
       Elem<T>::store(out + i, 0.f);
   }
-  if (w == nullptr) return;
+  if (!own) return;
   T* k = out + H * d;
   T* v = k + d;
   for (int e = tid; e < d; e += blockDim.x) {
@@ -271,11 +275,14 @@ KVF_EXPORT int kvf_latent_split(int dtype, const void* proj, int ld_in, void* qk
   if (H <= 0 || dim < 0 || rot < 0 || rank <= 0 || d < rot + rank || ld_in < H * (dim + rot) + (w ? rank + rot : 0) ||
       ld_out < (H + (w ? 2 : 0)) * d)
     return static_cast<int>(hipErrorInvalidValue);
+  int shares = n >= 512 ? 1 : 512 / n;
+  if (shares > 8) shares = 8;
+  if (shares > H) shares = H;
   if (dtype == 0)
-    hipLaunchKernelGGL(latent_split_kernel<float>, dim3(n), dim3(256), 0, s, static_cast<const float*>(proj), ld_in,
+    hipLaunchKernelGGL(latent_split_kernel<float>, dim3(n, shares), dim3(256), 0, s, static_cast<const float*>(proj), ld_in,
                        static_cast<float*>(qkv), ld_out, w, eps, H, dim, rot, rank, d);
   else if (dtype == 1)
-    hipLaunchKernelGGL(latent_split_kernel<bf16_t>, dim3(n), dim3(256), 0, s, static_cast<const bf16_t*>(proj), ld_in,
+    hipLaunchKernelGGL(latent_split_kernel<bf16_t>, dim3(n, shares), dim3(256), 0, s, static_cast<const bf16_t*>(proj), ld_in,
                        static_cast<bf16_t*>(qkv), ld_out, w, eps, H, dim, rot, rank, d);
   else
     return static_cast<int>(hipErrorInvalidValue);

@@ -128,9 +128,10 @@ __global__ __launch_bounds__(256) void ssm_conv_kernel(const T* __restrict__ row
       for (int j = 0; j < TAPS - 1; ++j)
         x[j] = Elem<T>::load(src + static_cast<size_t>(t0 - (TAPS - 1) + j) * a.ld_in);
     }
+    // (past the run's end its last row is read again and not used, so that no load is predicated)
 #pragma unroll
     for (int i = 0; i < CONV_TILE; ++i)
-      x[TAPS - 1 + i] = i < cnt ? Elem<T>::load(src + static_cast<size_t>(t0 + i) * a.ld_in) : 0.f;
+      x[TAPS - 1 + i] = Elem<T>::load(src + static_cast<size_t>(t0 + min(i, cnt - 1)) * a.ld_in);
     float wt[TAPS];
 #pragma unroll
     for (int j = 0; j < TAPS; ++j) wt[j] = w[static_cast<size_t>(c) * TAPS + j];
