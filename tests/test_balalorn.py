@@ -145,8 +145,8 @@ def test_one_layers_pages_serve_both_latent_layers_and_memories_have_slots():
 
 
 def test_frequencies_are_rounded_once():
-    r = RotaryPositions(16, 250000.0, interleaved=True, rounded_once=True)
-    want = torch.tensor([250000.0 ** (-2.0 * i / 16) for i in range(8)], dtype=torch.float64).float()
+    r = RotaryPositions(12, 70000.0, interleaved=True, rounded_once=True)
+    want = torch.tensor([70000.0 ** (-2.0 * i / 12) for i in range(6)], dtype=torch.float64).float()
     assert torch.equal(r.inv_freq, want)
 
 

@@ -194,9 +194,8 @@ def test_writes_that_repeat_a_key_replace_what_it_answers():
     """With beta near one and no decay, the delta rule's memory answers a key with the last value
     written under it, however often it was overwritten, also across chunks."""
     H, dk, dv, n = 1, 16, 16, 130
-    k = plain.unit(rand(4, dk, seed=1))
     which = [i % 4 for i in range(n)]
-    keys = torch.linalg.qr(rand(dk, dk, seed=2))[0][:4] if dk >= 4 else k
+    keys = torch.linalg.qr(rand(dk, dk, seed=2))[0][:4]       # four orthogonal unit vectors
     kk = torch.stack([keys[i] for i in which])
     v = rand(n, dv, seed=3)
     za, zb = torch.full((n, H), -60.0), torch.full((n, H), 40.0)
