@@ -16,7 +16,7 @@
 // sequence stay visible behind the window; the walk over the key tiles then has two pieces, the
 // tiles of the kept keys and the tiles from the window's first key on).  Scores are scaled after the dot
 // product; with `slopes` (one number per q head) slopes[h] * (j - p) is added to them, a bias by
-// distance.  The order of every sum is fixed by the positions alone.
+// distance, or with `dist` (a table [H, n_dist]) dist[h][min(p - j, n_dist - 1)].  The order of every sum is fixed by the positions alone.
 //
 // K pages are [num_blocks, KV, block_size, d], V pages are transposed [num_blocks, KV, d,
 // block_size]; a key whose page entry is negative or out of range reads as zeros.
@@ -42,10 +42,17 @@ struct AttnArgs {
   const float* slopes;  // null, or one number per q head: slopes[h] * (key - query position) is added to a score
   const float* sinks;   // null, or one number per q head: exp(sinks[h]) joins the softmax's denominator (a key without a value)
   float cap;            // 0, or the scaled score s becomes cap * tanh(s / cap)
+  const float* dist;    // null, or [H, n_dist]: dist[h][min(query position - key, n_dist - 1)] is added to a score
+  int n_dist;
 };
 
 // the scaled score under the cap (0: none)
 __device__ __forceinline__ float capped(float s, float cap) { return cap > 0.f ? cap * tanhf(s / cap) : s; }
+
+// the entry for distance n of a head's row of biases (a key behind the query is masked and reads the first)
+__device__ __forceinline__ float dist_bias(const float* row, int n_dist, int n) {
+  return row ? row[min(max(n, 0), n_dist - 1)] : 0.f;
+}
 
 typedef float f32x4 __attribute__((ext_vector_type(4)));
 
@@ -111,6 +118,7 @@ __global__ __launch_bounds__(256) void attn_mfma32_kernel(
   const int pos = start + tok;
   const int first_vis = first_seen(a.window, pos);      // the first key this row sees
   const float slope = a.slopes && row_ok ? a.slopes[head] : 0.f;
+  const float* drow = a.dist ? a.dist + static_cast<size_t>(head) * a.n_dist : nullptr;
   // key ranges: of the workgroup's rows (what is staged) and of this wave's (what it works on)
   int last = item0 + ITEM_ROWS - 1;
   if (last >= rows_total) last = rows_total - 1;
@@ -193,7 +201,9 @@ __global__ __launch_bounds__(256) void attn_mfma32_kernel(
           const int j = t0 + 16 * st + 4 * g4 + v;
           bool vis = row_ok && j <= pos && j < ctx;
           if (a.window != 0) vis = vis && (j >= first_vis || j < keep);
-          sc[v] = vis ? fmaf(slope, static_cast<float>(j - pos), capped(sc[v] * a.scale, a.cap)) : -INFINITY;
+          sc[v] = vis ? fmaf(slope, static_cast<float>(j - pos), capped(sc[v] * a.scale, a.cap)) +
+                            dist_bias(drow, a.n_dist, pos - j)
+                      : -INFINITY;
           tmax = fmaxf(tmax, sc[v]);
         }
         p[st] = sc;
@@ -320,6 +330,8 @@ struct DecodeArgs {
   const float* slopes;  // as in AttnArgs
   const float* sinks;   // as in AttnArgs
   float cap;            // as in AttnArgs
+  const float* dist;    // as in AttnArgs
+  int n_dist;
 };
 
 // GT: heads of the group handled together (a power of two, at most 8, or 4 for heads of more than
@@ -419,7 +431,8 @@ __global__ __launch_bounds__(DEC_WAVES * KVF_WAVE) void attn_decode_kernel(
     float corr[GT];
 #pragma unroll
     for (int g = 0; g < GT; ++g) {
-      const float sc = (vis && page >= 0) ? fmaf(slope[g], static_cast<float>(j - pos), capped(s[g] * a.scale, a.cap)) : -INFINITY;
+      float sc = (vis && page >= 0) ? fmaf(slope[g], static_cast<float>(j - pos), capped(s[g] * a.scale, a.cap)) : -INFINITY;
+      if (a.dist && g0 + g < G) sc += dist_bias(a.dist + static_cast<size_t>(kvh * G + g0 + g) * a.n_dist, a.n_dist, pos - j);
       const float m_new = fmaxf(m_run[g], wave_max(sc));
       float p = 0.f;
       corr[g] = 1.f;
@@ -602,14 +615,15 @@ KVF_EXPORT int kvf_attn_generic_decode(int dtype, const void* q, const void* k_p
                                        int H, int KV, int d, int block_size, int num_blocks,
                                        int table_stride, int q_stride, int o_stride, int window,
                                        int keep, int n_seqs, int splits, float scale,
-                                       const float* slopes, const float* sinks, float cap, hipStream_t s) {
+                                       const float* slopes, const float* sinks, float cap,
+                                       const float* dist, int n_dist, hipStream_t s) {
   if (num_seqs <= 0) return 0;
-  if (!(cap >= 0.f)) return static_cast<int>(hipErrorInvalidValue);
+  if (!(cap >= 0.f) || (dist && n_dist <= 0)) return static_cast<int>(hipErrorInvalidValue);
   if (keep < 0 || d % 16 != 0 || d > MAX_HEAD || d <= 0 || KV <= 0 || H % KV != 0 || splits < 1 ||
       (splits > 1 && (!part_acc || !part_ml)) || block_size <= 0)
     return static_cast<int>(hipErrorInvalidValue);
   DecodeArgs a{H, KV, d, block_size, num_blocks, table_stride, q_stride, o_stride, window, n_seqs,
-               splits, keep, scale, slopes, sinks, cap};
+               splits, keep, scale, slopes, sinks, cap, dist, n_dist};
   if (dtype == 0)
     return launch_decode<float>(q, k_pages, v_pages, block_table, seq_ids, cu_q, ctx_lens, out,
                                 part_acc, part_ml, num_seqs, a, s);
@@ -627,13 +641,14 @@ KVF_EXPORT int kvf_attn_generic(int dtype, const void* q, const void* k_pages, c
                                 const int* work, int num_work, void* out, int H, int KV, int d,
                                 int block_size, int num_blocks, int table_stride, int q_stride,
                                 int o_stride, int window, int keep, int n_seqs, float scale,
-                                const float* slopes, const float* sinks, float cap, hipStream_t s) {
-  if (!(cap >= 0.f)) return static_cast<int>(hipErrorInvalidValue);
+                                const float* slopes, const float* sinks, float cap, const float* dist,
+                                int n_dist, hipStream_t s) {
+  if (!(cap >= 0.f) || (dist && n_dist <= 0)) return static_cast<int>(hipErrorInvalidValue);
   if (keep < 0 || d % 16 != 0 || d > MAX_HEAD || d <= 0 || KV <= 0 || H % KV != 0 || !work || block_size <= 0 ||
       q_stride % 4 != 0 || o_stride % 4 != 0)
     return static_cast<int>(hipErrorInvalidValue);
   AttnArgs a{H, KV, d, block_size, num_blocks, table_stride, q_stride, o_stride, window, n_seqs,
-             keep, scale, slopes, sinks, cap};
+             keep, scale, slopes, sinks, cap, dist, n_dist};
   if (dtype == 0)
     return launch<float>(q, k_pages, v_pages, block_table, cu_q, ctx_lens, work, num_work, out, a, s);
   if (dtype == 1)

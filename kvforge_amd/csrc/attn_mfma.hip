@@ -29,6 +29,9 @@
 // the gap.
 // With `slopes` (one number per q head) a score also gets slopes[h] * (j - p), a bias by distance;
 // the kernels are instantiated with and without it, so that attention without it pays nothing.
+// With `dist` (a table [H, n_dist]) it gets dist[h][min(p - j, n_dist - 1)] instead, any bias by distance.
+// The table of the workgroup's heads is staged in LDS, padded at both ends: a lane's eight keys are
+// eight neighbouring distances, read at one base with fixed offsets.
 // The softmax reference of a row (what is subtracted before exp) is raised only when some score
 // of the wave exceeds it by more than LAZY (in log2 units): exp(s - ref) then stays below
 // 2^LAZY, sums and accumulators need no rescaling in most blocks, and the result is the same
@@ -88,7 +91,40 @@ struct MArgs {
   // sequence: a query sees the keys of its own chunk alone.  chunk_magic: floor(2^32 / c), and
   // 2^32 - 1 for c == 1.
   unsigned chunk_magic;
+  // null, or a bias by distance [H, n_dist] (kernels with BIAS == 4): dist[h][min(pos - key, n_dist - 1)] joins
+  // the scaled score.  dist_lds: the table goes through LDS.
+  const float* dist;
+  int n_dist, dist_lds;
 };
+
+// ---- the table of biases by distance.  A head's row in LDS holds the distances -DIST_PAD .. n_dist - 1 +
+// DIST_PAD in log2 units: zeros in front (keys behind the query, which are masked), the last one
+// repeated behind.
+constexpr int DIST_PAD = 7;
+__host__ __device__ __forceinline__ int dist_row(int n_dist) { return n_dist + 2 * DIST_PAD; }
+struct DistTable {
+  const float* lds;    // rows of dist_row(n) floats, or null: the table in memory is read
+  const float* mem;    // [H, n]
+  int n;
+};
+__device__ __forceinline__ void stage_dist(const MArgs& a, int head0, int heads, float* lds) {
+  const int row = dist_row(a.n_dist);
+  for (int i = threadIdx.x; i < heads * row; i += blockDim.x) {
+    const int h = i / row, d = i - h * row - DIST_PAD;
+    lds[i] = d < 0 ? 0.f : a.dist[static_cast<size_t>(head0 + h) * a.n_dist + min(d, a.n_dist - 1)] * LOG2E;
+  }
+}
+// biases (log2 units) of the keys at distances n0, n0 - 1, .., n0 - 7; `off`: the head's row in the table
+__device__ __forceinline__ void dist_eight(const DistTable& t, int off, int n0, float (&b)[8]) {
+  if (t.lds) {
+    const float* p = t.lds + off + DIST_PAD + min(max(n0, 0), t.n - 1 + DIST_PAD);
+#pragma unroll
+    for (int j = 0; j < 8; ++j) b[j] = p[-j];
+  } else {
+#pragma unroll
+    for (int j = 0; j < 8; ++j) b[j] = t.mem[off + min(max(n0 - j, 0), t.n - 1)] * LOG2E;
+  }
+}
 
 // The first key of the chunk that position `pos` lies in.  No division: the quotient's estimate
 // mulhi(pos, floor(2^32 / c)) is at most two short, so the remainder is below 3 c and two
@@ -219,18 +255,21 @@ template <int RT> struct Rows {
   int keep[RT];        // and the keys below this (kept behind a window; 0 for a row that is none)
   int pos[RT];         // the row's own position; with slope2, only for kernels with BIAS
   float slope2[RT];    // the head's slope in log2 units
+  int drow[RT];        // the head's row in the table of biases by distance (BIAS 4 alone)
 };
 
 // One key block for the row tiles of a wave: scores, lazy softmax update, P * V.
 // References live in log2 units: scale2 = scale * log2(e) > 0 is applied inside the exponent.
 // BIAS 1: a score also gets its head's slope times the key's distance from the row's position;
 // the scores are then brought to log2 units before the maximum is taken.  BIAS 2: the scaled
-// score s becomes cap * tanh(s / cap), likewise before the maximum.
+// score s becomes cap * tanh(s / cap), likewise before the maximum.  BIAS 4: a score also gets its head's
+// entry for the key's distance, likewise.
 template <int DT, int RT, int BIAS>
 __device__ __forceinline__ void block_update(const bf16x8 (&kf)[2][(DT + 1) / 2], const bf16x8 (&vf)[DT],
                                              const bf16x8 (&qf)[RT][(DT + 1) / 2], const Rows<RT>& rows,
                                              int kb, int kg, bool edge, float scale_log2, float (&m_ref)[RT], float (&l_run)[RT],
-                                             f32x4 (&acc)[RT][DT], float cap = 0.f) {
+                                             f32x4 (&acc)[RT][DT], float cap = 0.f,
+                                             const DistTable& dist = DistTable{nullptr, nullptr, 0}) {
   constexpr int DC = (DT + 1) / 2;
   const float scale2 = BIAS != 0 ? 1.f : scale_log2;
   f32x4 s[RT][2];
@@ -274,6 +313,17 @@ __device__ __forceinline__ void block_update(const bf16x8 (&kf)[2][(DT + 1) / 2]
 #pragma unroll
         for (int r = 0; r < 4; ++r)
           s[rt][t][r] = fmaf(s[rt][t][r], scale_log2, fmaf(rows.slope2[rt], static_cast<float>(4 * t + r), at0));
+    }
+  }
+  if constexpr (BIAS == 4) {
+#pragma unroll
+    for (int rt = 0; rt < RT; ++rt) {
+      float b[8];
+      dist_eight(dist, rows.drow[rt], rows.pos[rt] - (kb + 8 * kg), b);
+#pragma unroll
+      for (int t = 0; t < 2; ++t)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) s[rt][t][r] = fmaf(s[rt][t][r], scale_log2, b[4 * t + r]);
     }
   }
 #pragma unroll
@@ -408,6 +458,12 @@ __global__ __launch_bounds__(256) KVF_VGPR_FORM(DT <= 8) void attn_mfma_runs_ker
   const bool seq_ok = qlen > 0 && start >= 0;
   const Pages pg{k_pages, vt_pages, block_table + static_cast<size_t>(seq) * a.table_stride, kvh, ctx,
                  j16, kg};
+  float* dist_space = reinterpret_cast<float*>(frag_lds + (SHARE ? 2 * N_FRAG * KVF_WAVE : 0));
+  if (SCORE == 4 && a.dist_lds) {
+    stage_dist(a, kvh * G, G, dist_space);
+    __syncthreads();
+  }
+  const DistTable dist{SCORE == 4 && a.dist_lds ? dist_space : nullptr, a.dist, a.n_dist};
   for (int part = 0; part < 2; ++part) {
   const int item = work[3 * wrow + 1 + part];
   if (item < 0) continue;
@@ -418,6 +474,11 @@ __global__ __launch_bounds__(256) KVF_VGPR_FORM(DT <= 8) void attn_mfma_runs_ker
   int pos_min, pos_max;
   setup_rows<DT, RT, CHUNK>(q, a, q0, qlen, start, kvh, wg_tile + wave * RT, j16, kg, seq_ok, rows, qf, pos_min,
                      pos_max);
+  if constexpr (SCORE == 4) {
+#pragma unroll
+    for (int rt = 0; rt < RT; ++rt)
+      rows.drow[rt] = a.dist_lds ? (rows.head[rt] - kvh * G) * dist_row(a.n_dist) : rows.head[rt] * a.n_dist;
+  }
   // key range of this wave, and of the workgroup (tiles wg_tile .. wg_tile + 4*RT - 1)
   int lo_w = 0, hi_w = -1;
   if (pos_max >= 0) {
@@ -527,7 +588,7 @@ __global__ __launch_bounds__(256) KVF_VGPR_FORM(DT <= 8) void attn_mfma_runs_ker
 #pragma unroll
         for (int t = 0; t < DT; ++t) vf[t] = as_frag(frag_lds[(buf * N_FRAG + N_K + t) * KVF_WAVE + lane]);
         const bool edge = kb + 31 > pos_min || kb + 32 > ctx || a.window > 0 || CHUNK;
-        block_update<DT, RT, SCORE>(kf, vf, qf, rows, kb, kg, edge, scale2, m_ref, l_run, acc, a.cap);
+        block_update<DT, RT, SCORE>(kf, vf, qf, rows, kb, kg, edge, scale2, m_ref, l_run, acc, a.cap, dist);
       }
     };
     const int kb_first = wk.first;
@@ -611,7 +672,7 @@ __global__ __launch_bounds__(256) KVF_VGPR_FORM(DT <= 8) void attn_mfma_runs_ker
 #pragma unroll
       for (int t = 0; t < DT; ++t) vf[t] = as_frag(keep_first(vr[t], vl));
       const bool edge = kb + 31 > pos_min || kb + 32 > ctx || a.window > 0 || CHUNK;
-      block_update<DT, RT, SCORE>(kf, vf, qf, rows, kb, kg, edge, scale2, m_ref, l_run, acc, a.cap);
+      block_update<DT, RT, SCORE>(kf, vf, qf, rows, kb, kg, edge, scale2, m_ref, l_run, acc, a.cap, dist);
     }
   }
 
@@ -644,7 +705,7 @@ __global__ __launch_bounds__(NW * KVF_WAVE) KVF_VGPR_FORM(DT <= 6) void attn_mfm
     const int* __restrict__ seq_ids, const int* __restrict__ cu_q, const int* __restrict__ ctx_lens,
     bf16_t* __restrict__ out, float* __restrict__ part_acc, float* __restrict__ part_ml, MArgs a) {
   constexpr int DC = (DT + 1) / 2;
-  extern __shared__ float lds[];  // [NW][DT][64][4] accumulators, then [NW][16][2]
+  extern __shared__ float lds[];  // [NW][DT][64][4] accumulators, [NW][16][2], then the table of biases by distance
 
   const int lane = threadIdx.x % KVF_WAVE;
   const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x / KVF_WAVE);  // the same in all lanes
@@ -670,7 +731,15 @@ __global__ __launch_bounds__(NW * KVF_WAVE) KVF_VGPR_FORM(DT <= 6) void attn_mfm
   Rows<1> rows;
   bf16x8 qf[1][DC];
   int pos_min, pos_max;
+  float* dist_space = lds + NW * DT * KVF_WAVE * 4 + NW * 16 * 2;
+  if (BIAS == 4 && a.dist_lds) stage_dist(a, kvh * G + tile * 16, min(16, G - tile * 16), dist_space);
+  const DistTable dist{BIAS == 4 && a.dist_lds ? dist_space : nullptr, a.dist, a.n_dist};
   setup_rows<DT, 1>(q, a, q0, qlen, start, kvh, tile, j16, kg, seq_ok, rows, qf, pos_min, pos_max);
+  if constexpr (BIAS == 4) {
+    rows.drow[0] = !rows.ok[0] ? 0 : a.dist_lds ? (rows.head[0] - kvh * G - tile * 16) * dist_row(a.n_dist)
+                                                : rows.head[0] * a.n_dist;
+    if (a.dist_lds) __syncthreads();
+  }
   if (a.window < 0 && rows.ok[0]) {   // chunks of positions: the rows see from their chunk's first key
     rows.first[0] = chunk_first(a, rows.pos[0]);
     rows.span[0] = static_cast<unsigned>(rows.pos[0] - rows.first[0]);
@@ -730,7 +799,7 @@ __global__ __launch_bounds__(NW * KVF_WAVE) KVF_VGPR_FORM(DT <= 6) void attn_mfm
 #pragma unroll
     for (int t = 0; t < DT; ++t) vf[t] = as_frag(keep_first(r.v[t], r.vl));
     const bool edge = kb + 31 > pos_min || kb + 32 > ctx || a.window != 0;
-    block_update<DT, 1, BIAS>(kf, vf, qf, rows, kb, kg, edge, scale2, m_ref, l_run, acc, a.cap);
+    block_update<DT, 1, BIAS>(kf, vf, qf, rows, kb, kg, edge, scale2, m_ref, l_run, acc, a.cap, dist);
   };
   // Without a window the page lookups of the first blocks are asked for together with the
   // query and the context length, not after them: one round trip to memory less.
@@ -881,6 +950,11 @@ bool args_ok(int H, int KV, int d, int bs, int nb, int table_stride, float scale
          static_cast<unsigned long long>(nb) * KV * bs * d / 8 < limit && nb < (1 << 24) &&
          static_cast<unsigned long long>(KV) * bs * d / 8 < (1ull << 24);
 }
+// a table of biases by distance goes with none of the other things done to scores; its offsets fit 32 bits
+bool dist_ok(const float* dist, int n_dist, int H, const float* slopes, const float* sinks, float cap, int window) {
+  return !dist || (n_dist > 0 && static_cast<long long>(H) * n_dist < (1ll << 31) && !slopes && !sinks && !(cap > 0.f) &&
+                   window >= 0);
+}
 unsigned magic_of(int bs) { return static_cast<unsigned>((1ull << 32) / bs) + 1u; }
 // for chunks of c = -window positions: floor(2^32 / c), which for c == 1 is the largest 32-bit number
 unsigned chunk_magic_of(int window) {
@@ -897,6 +971,7 @@ unsigned chunk_magic_of(int window) {
 // has and by kvf_attn_mfma_prefill_blocks_per_cu.
 constexpr int runs_max_rt(int dt) { return dt <= 8 ? 2 : 1; }
 constexpr bool runs_share(int dt) { return dt <= 12; }
+constexpr size_t DIST_LDS_MOST = 64 * 1024;   // LDS a launch may ask for together with its table of biases
 
 template <int DT, int RT>
 void launch_runs_rt(dim3 grid, hipStream_t s, const void* q, const void* k_pages, const void* vt_pages,
@@ -915,7 +990,15 @@ void launch_runs_rt(dim3 grid, hipStream_t s, const void* q, const void* k_pages
                        static_cast<const bf16_t*>(q), static_cast<const bf16_t*>(k_pages),
                        static_cast<const bf16_t*>(vt_pages), block_table, work, cu_q, ctx_lens,
                        static_cast<bf16_t*>(out), a);
-  else if (a.sinks)   // (never with slopes: the exported entry refuses the pair)
+  else if (a.dist) {   // (never with any of the others)
+    MArgs b = a;
+    const size_t table = static_cast<size_t>(a.H / a.KV) * dist_row(a.n_dist) * sizeof(float);
+    b.dist_lds = lds + table <= DIST_LDS_MOST;
+    hipLaunchKernelGGL((attn_mfma_runs_kernel<DT, RT, SHARE, 4, false>), grid, dim3(256), b.dist_lds ? lds + table : lds, s,
+                       static_cast<const bf16_t*>(q), static_cast<const bf16_t*>(k_pages),
+                       static_cast<const bf16_t*>(vt_pages), block_table, work, cu_q, ctx_lens,
+                       static_cast<bf16_t*>(out), b);
+  } else if (a.sinks)   // (never with slopes: the exported entry refuses the pair)
     hipLaunchKernelGGL((attn_mfma_runs_kernel<DT, RT, SHARE, 0, true>), grid, dim3(256), lds, s,
                        static_cast<const bf16_t*>(q), static_cast<const bf16_t*>(k_pages),
                        static_cast<const bf16_t*>(vt_pages), block_table, work, cu_q, ctx_lens,
@@ -955,7 +1038,16 @@ void launch_split_waves(dim3 grid, hipStream_t s, const void* q, const void* k_p
                        static_cast<const bf16_t*>(q), static_cast<const bf16_t*>(k_pages),
                        static_cast<const bf16_t*>(vt_pages), block_table, seq_ids, cu_q, ctx_lens,
                        static_cast<bf16_t*>(out), part_acc, part_ml, a);
-  else if (a.sinks)
+  else if (a.dist) {
+    MArgs b = a;
+    const int G = a.H / a.KV;
+    const size_t table = static_cast<size_t>(G < 16 ? G : 16) * dist_row(a.n_dist) * sizeof(float);
+    b.dist_lds = lds + table <= DIST_LDS_MOST;
+    hipLaunchKernelGGL((attn_mfma_split_kernel<DT, (DT <= 8), NW, 4, false>), grid, dim3(NW * KVF_WAVE),
+                       b.dist_lds ? lds + table : lds, s, static_cast<const bf16_t*>(q),
+                       static_cast<const bf16_t*>(k_pages), static_cast<const bf16_t*>(vt_pages), block_table, seq_ids,
+                       cu_q, ctx_lens, static_cast<bf16_t*>(out), part_acc, part_ml, b);
+  } else if (a.sinks)
     hipLaunchKernelGGL((attn_mfma_split_kernel<DT, (DT <= 8), NW, 0, true>), grid, dim3(NW * KVF_WAVE), lds, s,
                        static_cast<const bf16_t*>(q), static_cast<const bf16_t*>(k_pages),
                        static_cast<const bf16_t*>(vt_pages), block_table, seq_ids, cu_q, ctx_lens,
@@ -1042,8 +1134,9 @@ KVF_EXPORT int kvf_attn_mfma_prefill(const void* q, const void* k_pages, const v
                                      int bs, int nb, int table_stride, int q_stride, int o_stride,
                                      int window, int keep, int n_seqs, float scale, const float* slopes,
                                      const void* gate, int gate_stride, const float* sinks, float cap,
-                                     hipStream_t s) {
+                                     const float* dist, int n_dist, hipStream_t s) {
   if (num_work <= 0) return 0;
+  if (!dist_ok(dist, n_dist, H, slopes, sinks, cap, window)) return static_cast<int>(hipErrorInvalidValue);
   if (sinks && slopes) return static_cast<int>(hipErrorInvalidValue);   // no kernel has both
   if (!(cap >= 0.f) || (cap > 0.f && (sinks || slopes))) return static_cast<int>(hipErrorInvalidValue);
   // chunks of positions (window < 0): the kernel for query runs has them with plain scores only
@@ -1059,7 +1152,7 @@ KVF_EXPORT int kvf_attn_mfma_prefill(const void* q, const void* k_pages, const v
   // of one head and finds them in its own L2 after the first workgroup has brought them in.
   const int kv_fastest = num_work <= 65535 ? 1 : 0;
   const MArgs a{H, KV, d, bs, nb, table_stride, q_stride, o_stride, window, n_seqs, 1, keep, kv_fastest, scale, magic_of(bs), slopes,
-                static_cast<const bf16_t*>(gate), gate_stride, sinks, cap, chunk_magic_of(window)};
+                static_cast<const bf16_t*>(gate), gate_stride, sinks, cap, chunk_magic_of(window), dist, n_dist, 0};
   const dim3 grid = kv_fastest ? dim3(KV, num_work) : dim3(num_work, KV);
   switch (d / 16) {
 #define GO(DT) \
@@ -1080,8 +1173,9 @@ KVF_EXPORT int kvf_attn_mfma_decode(const void* q, const void* k_pages, const vo
                                     int table_stride, int q_stride, int o_stride, int window,
                                     int keep, int n_seqs, int splits, float scale, const float* slopes,
                                     const void* gate, int gate_stride, const float* sinks, float cap,
-                                    hipStream_t s) {
+                                    const float* dist, int n_dist, hipStream_t s) {
   if (num_seqs <= 0) return 0;
+  if (!dist_ok(dist, n_dist, H, slopes, sinks, cap, window)) return static_cast<int>(hipErrorInvalidValue);
   if (sinks && slopes) return static_cast<int>(hipErrorInvalidValue);
   if (!(cap >= 0.f) || (cap > 0.f && (sinks || slopes))) return static_cast<int>(hipErrorInvalidValue);
   if (keep < 0 || (gate && (gate_stride % 4 != 0 || gate_stride < H * d || reinterpret_cast<uintptr_t>(gate) % 8 != 0)))
@@ -1090,7 +1184,7 @@ KVF_EXPORT int kvf_attn_mfma_decode(const void* q, const void* k_pages, const vo
       splits > KVF_WAVE || (splits > 1 && (!part_acc || !part_ml)))
     return static_cast<int>(hipErrorInvalidValue);
   const MArgs a{H, KV, d, bs, nb, table_stride, q_stride, o_stride, window, n_seqs, splits, keep, 0, scale, magic_of(bs), slopes,
-                static_cast<const bf16_t*>(gate), gate_stride, sinks, cap, chunk_magic_of(window)};
+                static_cast<const bf16_t*>(gate), gate_stride, sinks, cap, chunk_magic_of(window), dist, n_dist, 0};
   const int G = H / KV, chunks = (G + 15) / 16;
   if (num_seqs > 65535) return static_cast<int>(hipErrorInvalidValue);
   const dim3 grid(KV * chunks, num_seqs, splits);

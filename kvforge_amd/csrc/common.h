@@ -90,4 +90,26 @@ __device__ __forceinline__ float block_sum(float v, float* scratch) {
   return t;
 }
 
+// How a gated feed-forward joins its (gate, up) pairs.  act 0: silu(g) u; 1: gelu(g) u (the tanh form);
+// 2: both limited, g = min(g, limit), u = clamp(u, -limit, limit), g sigmoid(1.702 g) (u + 1).  What is
+// stored is that times `scale`.
+struct GateForm {
+  int act;
+  float limit, scale;
+};
+constexpr int GATE_LIMITED = 2;
+constexpr float LIMITED_SLOPE = 1.702f;
+// one pair under act 2, without the scale
+__device__ __forceinline__ float limited_pair(float g, float u, float limit) {
+  g = fminf(g, limit);
+  u = fminf(fmaxf(u, -limit), limit);
+  return g / (1.f + __expf(-LIMITED_SLOPE * g)) * (u + 1.f);
+}
+// the same with the exact exponential, for the 32-bit kernels
+__device__ __forceinline__ float limited_pair_exact(float g, float u, float limit) {
+  g = fminf(g, limit);
+  u = fminf(fmaxf(u, -limit), limit);
+  return g / (1.f + expf(-LIMITED_SLOPE * g)) * (u + 1.f);
+}
+
 static inline int kvf_last_error() { return static_cast<int>(hipGetLastError()); }

@@ -38,7 +38,7 @@ KVF_EXPORT int kvf_embed_bf16(const int* ids, const void* t, float* o, int n, in
 // null when the weight has been folded into the matrix that consumes y.
 // `delta` (may be null, [x_rows, h] of T) is a sum still owed to the stream: the norm is taken of
 // x + delta, and without `rows` the sum is also written back to x, which saves the pass of an
-// add kernel of its own.
+// add kernel of its own.  `bias` (fp32, may be null): a vector owed to every row, likewise.
 __device__ __forceinline__ float4 load4(const float* p) { return *reinterpret_cast<const float4*>(p); }
 __device__ __forceinline__ float4 load4(const bf16_t* p) {
   const uint2 r = *reinterpret_cast<const uint2*>(p);
@@ -57,8 +57,9 @@ constexpr int NORM_KEEP = 4;  // float4s a thread keeps in registers between the
 
 template <typename T, typename W, typename D>
 __global__ void rmsnorm_kernel(float* __restrict__ x, const int* __restrict__ rows,
-                               const D* __restrict__ delta, const W* __restrict__ w, float eps,
-                               T* __restrict__ out, int h, int x_rows, int aligned) {
+                               const D* __restrict__ delta, const float* __restrict__ bias,
+                               const W* __restrict__ w, float eps, T* __restrict__ out, int h, int x_rows,
+                               int aligned) {
   __shared__ float scratch[16];
   const int m = blockIdx.x;
   int src = rows ? rows[m] : m;
@@ -69,7 +70,7 @@ __global__ void rmsnorm_kernel(float* __restrict__ x, const int* __restrict__ ro
   }
   float* xr = x + static_cast<size_t>(src) * h;
   const D* dr = delta ? delta + static_cast<size_t>(src) * h : nullptr;
-  const bool write_back = dr && !rows;
+  const bool write_back = (dr || bias) && !rows;
   float ss = 0.f;
   if (aligned && h <= static_cast<int>(blockDim.x) * 4 * NORM_KEEP) {
     // the row stays in registers: one read of x (and delta), one write of y (and x)
@@ -83,8 +84,12 @@ __global__ void rmsnorm_kernel(float* __restrict__ x, const int* __restrict__ ro
         if (dr) {
           const float4 d = load4(dr + i);
           v[k].x += d.x; v[k].y += d.y; v[k].z += d.z; v[k].w += d.w;
-          if (write_back) store4(xr + i, v[k]);
         }
+        if (bias) {
+          const float4 d = load4(bias + i);
+          v[k].x += d.x; v[k].y += d.y; v[k].z += d.z; v[k].w += d.w;
+        }
+        if (write_back) store4(xr + i, v[k]);
         ss += v[k].x * v[k].x + v[k].y * v[k].y + v[k].z * v[k].z + v[k].w * v[k].w;
       }
     }
@@ -106,10 +111,9 @@ __global__ void rmsnorm_kernel(float* __restrict__ x, const int* __restrict__ ro
   }
   for (int i = threadIdx.x; i < h; i += blockDim.x) {
     float v = xr[i];
-    if (dr) {
-      v += Elem<D>::load(dr + i);
-      if (write_back) xr[i] = v;
-    }
+    if (dr) v += Elem<D>::load(dr + i);
+    if (bias) v += bias[i];
+    if (write_back) xr[i] = v;
     ss += v * v;
   }
   ss = block_sum(ss, scratch);
@@ -117,38 +121,39 @@ __global__ void rmsnorm_kernel(float* __restrict__ x, const int* __restrict__ ro
   for (int i = threadIdx.x; i < h; i += blockDim.x) {
     float v = xr[i];  // already the sum where it was written back (by this same thread)
     if (dr && !write_back) v += Elem<D>::load(dr + i);
+    if (bias && !write_back) v += bias[i];
     Elem<T>::store(o + i, w ? v * r * Elem<W>::load(w + i) : v * r);
   }
 }
 
 template <typename T, typename D>
-static int rmsnorm_launch(float* x, const int* rows, const void* delta, const void* w, int w_is_f32,
-                          float eps, void* out, int m, int h, int x_rows, hipStream_t s) {
+static int rmsnorm_launch(float* x, const int* rows, const void* delta, const float* bias, const void* w,
+                          int w_is_f32, float eps, void* out, int m, int h, int x_rows, hipStream_t s) {
   if (m <= 0) return 0;
   const int threads = h >= 1024 ? 256 : (h >= 256 ? 128 : 64);
   auto at = [](const void* p, size_t a) { return reinterpret_cast<uintptr_t>(p) % a == 0; };
-  const int aligned = h % 4 == 0 && at(x, 16) && at(out, 4 * sizeof(T)) && at(delta, 4 * sizeof(D)) &&
+  const int aligned = h % 4 == 0 && at(x, 16) && at(out, 4 * sizeof(T)) && at(delta, 4 * sizeof(D)) && at(bias, 16) &&
                       at(w, w_is_f32 ? 16 : 4 * sizeof(T));
   if (w_is_f32)
     hipLaunchKernelGGL((rmsnorm_kernel<T, float, D>), dim3(m), dim3(threads), 0, s, x, rows,
-                       static_cast<const D*>(delta), static_cast<const float*>(w), eps,
+                       static_cast<const D*>(delta), bias, static_cast<const float*>(w), eps,
                        static_cast<T*>(out), h, x_rows, aligned);
   else
     hipLaunchKernelGGL((rmsnorm_kernel<T, T, D>), dim3(m), dim3(threads), 0, s, x, rows,
-                       static_cast<const D*>(delta), static_cast<const T*>(w), eps,
+                       static_cast<const D*>(delta), bias, static_cast<const T*>(w), eps,
                        static_cast<T*>(out), h, x_rows, aligned);
   return kvf_last_error();
 }
 // delta (may be null): a sum still owed to x, in the type of `out` or (delta_f32) in fp32
-KVF_EXPORT int kvf_rmsnorm_f32(float* x, const int* rows, const void* delta, int delta_f32, const void* w,
-                               int wf, float eps, void* out, int m, int h, int xr, hipStream_t s) {
+KVF_EXPORT int kvf_rmsnorm_f32(float* x, const int* rows, const void* delta, int delta_f32, const float* bias,
+                               const void* w, int wf, float eps, void* out, int m, int h, int xr, hipStream_t s) {
   (void)delta_f32;
-  return rmsnorm_launch<float, float>(x, rows, delta, w, wf, eps, out, m, h, xr, s);
+  return rmsnorm_launch<float, float>(x, rows, delta, bias, w, wf, eps, out, m, h, xr, s);
 }
-KVF_EXPORT int kvf_rmsnorm_bf16(float* x, const int* rows, const void* delta, int delta_f32, const void* w,
-                                int wf, float eps, void* out, int m, int h, int xr, hipStream_t s) {
-  if (delta_f32) return rmsnorm_launch<bf16_t, float>(x, rows, delta, w, wf, eps, out, m, h, xr, s);
-  return rmsnorm_launch<bf16_t, bf16_t>(x, rows, delta, w, wf, eps, out, m, h, xr, s);
+KVF_EXPORT int kvf_rmsnorm_bf16(float* x, const int* rows, const void* delta, int delta_f32, const float* bias,
+                                const void* w, int wf, float eps, void* out, int m, int h, int xr, hipStream_t s) {
+  if (delta_f32) return rmsnorm_launch<bf16_t, float>(x, rows, delta, bias, w, wf, eps, out, m, h, xr, s);
+  return rmsnorm_launch<bf16_t, bf16_t>(x, rows, delta, bias, w, wf, eps, out, m, h, xr, s);
 }
 
 // Two norms of the same row in one pass: y1 = v r w1 and y2 = v r w2 with v = x (+ delta, which is
@@ -795,7 +800,7 @@ KVF_EXPORT int kvf_norm_shift_bf16(NORM_SHIFT_DECL) {
 // ----------------------------------------------------------------------------- gated activations
 // out[m, i] = act(gate_i + bg[i]) * (up_i + bu[i]) in fp32; the input row holds gate at 2i and
 // up at 2i + 1 (`paired`) or gate at i and up at I + i.  act: 0 silu, 1 the tanh form of gelu.
-// The biases are fp32 vectors and may be null.
+// The biases are fp32 vectors and may be null.  act 2 and the scale: see GateForm.
 __device__ __forceinline__ float gelu_tanh_f(float z) {
   const float u = 0.7978845608028654f * (z + 0.044715f * z * z * z);
   return 0.5f * z * (1.f + tanhf(u));
@@ -806,7 +811,7 @@ __device__ __forceinline__ float act_f(int act, float z) {
 template <typename T>
 __global__ void gated_act_kernel(const T* __restrict__ gu, const float* __restrict__ bg,
                                  const float* __restrict__ bu, T* __restrict__ out, int inter,
-                                 size_t total, int paired, int act) {
+                                 size_t total, int paired, GateForm f) {
   const size_t idx = static_cast<size_t>(blockIdx.x) * blockDim.x + threadIdx.x;
   if (idx >= total) return;
   const size_t m = idx / inter;
@@ -816,13 +821,13 @@ __global__ void gated_act_kernel(const T* __restrict__ gu, const float* __restri
   float u = Elem<T>::load(paired ? row + 2 * i + 1 : row + inter + i);
   if (bg) g += bg[i];
   if (bu) u += bu[i];
-  Elem<T>::store(out + idx, act_f(act, g) * u);
+  Elem<T>::store(out + idx, (f.act == GATE_LIMITED ? limited_pair_exact(g, u, f.limit) : act_f(f.act, g) * u) * f.scale);
 }
 // bf16, paired: a thread takes four neighbouring (gate, up) pairs (16 bytes in, 8 bytes out)
 // (the grid's x runs along a row, its y over the rows, so that no index is divided)
 __global__ void gated_act_pairs4_kernel(const bf16_t* __restrict__ gu, const float* __restrict__ bg,
                                         const float* __restrict__ bu, bf16_t* __restrict__ out,
-                                        int inter, int rows, int act) {
+                                        int inter, int rows, GateForm f) {
   const int i0 = (blockIdx.x * blockDim.x + threadIdx.x) * 4;
   if (i0 >= inter) return;
   float4 b_g = make_float4(0.f, 0.f, 0.f, 0.f), b_u = b_g;
@@ -836,15 +841,17 @@ __global__ void gated_act_pairs4_kernel(const bf16_t* __restrict__ gu, const flo
 #pragma unroll
   for (int i = 0; i < 4; ++i) {
     const float g = v[2 * i] + gb[i], u = v[2 * i + 1] + ub[i];
-    float a;
-    if (act == 1) {
+    float y;
+    if (f.act == GATE_LIMITED) {
+      y = limited_pair(g, u, f.limit);
+    } else if (f.act == 1) {
       // tanh(t) = 1 - 2 / (1 + exp(2 t)); exp overflows to +inf for large t, which gives 1
       const float t = 0.7978845608028654f * (g + 0.044715f * g * g * g);
-      a = 0.5f * g * (2.f - 2.f / (1.f + __expf(2.f * t)));
+      y = 0.5f * g * (2.f - 2.f / (1.f + __expf(2.f * t))) * u;
     } else {
-      a = g / (1.f + __expf(-g));
+      y = g / (1.f + __expf(-g)) * u;
     }
-    hh[i] = f32_to_bf16(a * u);
+    hh[i] = f32_to_bf16(y * f.scale);
   }
   uint2 packed;
   packed.x = hh[0] | (hh[1] << 16);
@@ -855,7 +862,9 @@ __global__ void gated_act_pairs4_kernel(const bf16_t* __restrict__ gu, const flo
 
 template <typename T>
 static int gated_act_launch(const void* gu, const float* bg, const float* bu, void* out, int m,
-                            int inter, int paired, int act, hipStream_t s) {
+                            int inter, int paired, GateForm f, hipStream_t s) {
+  if (f.act < 0 || f.act > GATE_LIMITED || (f.act == GATE_LIMITED && !(f.limit > 0.f)))
+    return static_cast<int>(hipErrorInvalidValue);
   const size_t total = static_cast<size_t>(m) * inter;
   if (total == 0) return 0;
   auto at16 = [](const void* p) { return reinterpret_cast<uintptr_t>(p) % 16 == 0; };
@@ -864,20 +873,20 @@ static int gated_act_launch(const void* gu, const float* bg, const float* bu, vo
     const int threads = inter / 4 >= 256 ? 256 : 64;
     const dim3 grid((inter / 4 + threads - 1) / threads, m < 65535 ? m : 65535);
     hipLaunchKernelGGL(gated_act_pairs4_kernel, grid, dim3(threads), 0, s, static_cast<const bf16_t*>(gu), bg,
-                       bu, static_cast<bf16_t*>(out), inter, m, act);
+                       bu, static_cast<bf16_t*>(out), inter, m, f);
     return kvf_last_error();
   }
   hipLaunchKernelGGL(gated_act_kernel<T>, dim3(static_cast<unsigned>((total + 255) / 256)), dim3(256), 0, s,
-                     static_cast<const T*>(gu), bg, bu, static_cast<T*>(out), inter, total, paired, act);
+                     static_cast<const T*>(gu), bg, bu, static_cast<T*>(out), inter, total, paired, f);
   return kvf_last_error();
 }
 KVF_EXPORT int kvf_gated_act_f32(const void* gu, const float* bg, const float* bu, void* out, int m,
-                                 int inter, int paired, int act, hipStream_t s) {
-  return gated_act_launch<float>(gu, bg, bu, out, m, inter, paired, act, s);
+                                 int inter, int paired, int act, float limit, float scale, hipStream_t s) {
+  return gated_act_launch<float>(gu, bg, bu, out, m, inter, paired, GateForm{act, limit, scale}, s);
 }
 KVF_EXPORT int kvf_gated_act_bf16(const void* gu, const float* bg, const float* bu, void* out, int m,
-                                  int inter, int paired, int act, hipStream_t s) {
-  return gated_act_launch<bf16_t>(gu, bg, bu, out, m, inter, paired, act, s);
+                                  int inter, int paired, int act, float limit, float scale, hipStream_t s) {
+  return gated_act_launch<bf16_t>(gu, bg, bu, out, m, inter, paired, GateForm{act, limit, scale}, s);
 }
 
 // ----------------------------------------------------------------------------- sigmoid gate
@@ -1231,6 +1240,68 @@ __global__ __launch_bounds__(256) void rms_add_kernel(float* __restrict__ x, con
 KVF_EXPORT int kvf_rms_add(float* x, const float* y, const float* w, float eps, int m, int h, hipStream_t s) {
   if (m <= 0) return 0;
   hipLaunchKernelGGL(rms_add_kernel, dim3(m), dim3(256), 0, s, x, y, w, eps, h);
+  return kvf_last_error();
+}
+
+// The rows of two sublayers side by side join the stream, each through a norm of its own, in one pass:
+// x += ya rsqrt(mean(ya^2) + eps) wa + yb rsqrt(mean(yb^2) + eps) wb.  Q > 0: rows of a multiple of four and at
+// most 1024 Q elements, which a thread then holds in registers, four neighbours a load.
+template <int Q>
+__global__ __launch_bounds__(256) void rms_add_two_kernel(float* __restrict__ x, const float* __restrict__ ya,
+                                                          const float* __restrict__ wa, const float* __restrict__ yb,
+                                                          const float* __restrict__ wb, float eps, int h) {
+  __shared__ float scratch[2][16];
+  const size_t at = static_cast<size_t>(blockIdx.x) * h;
+  float sa = 0.f, sb = 0.f;
+  if constexpr (Q > 0) {
+    float4 va[Q], vb[Q], vx[Q];
+#pragma unroll
+    for (int k = 0; k < Q; ++k) {
+      const int i = 4 * (threadIdx.x + 256 * k);
+      va[k] = vb[k] = vx[k] = make_float4(0.f, 0.f, 0.f, 0.f);
+      if (i < h) {
+        va[k] = load4(ya + at + i);
+        vb[k] = load4(yb + at + i);
+        vx[k] = load4(x + at + i);
+      }
+      sa += va[k].x * va[k].x + va[k].y * va[k].y + va[k].z * va[k].z + va[k].w * va[k].w;
+      sb += vb[k].x * vb[k].x + vb[k].y * vb[k].y + vb[k].z * vb[k].z + vb[k].w * vb[k].w;
+    }
+    const float ra = rsqrtf(block_sum(sa, scratch[0]) / static_cast<float>(h) + eps);
+    const float rb = rsqrtf(block_sum(sb, scratch[1]) / static_cast<float>(h) + eps);
+#pragma unroll
+    for (int k = 0; k < Q; ++k) {
+      const int i = 4 * (threadIdx.x + 256 * k);
+      if (i >= h) continue;
+      const float4 a = load4(wa + i), b = load4(wb + i);
+      vx[k].x += va[k].x * ra * a.x + vb[k].x * rb * b.x;
+      vx[k].y += va[k].y * ra * a.y + vb[k].y * rb * b.y;
+      vx[k].z += va[k].z * ra * a.z + vb[k].z * rb * b.z;
+      vx[k].w += va[k].w * ra * a.w + vb[k].w * rb * b.w;
+      store4(x + at + i, vx[k]);
+    }
+  } else {
+    for (int i = threadIdx.x; i < h; i += 256) {
+      sa = fmaf(ya[at + i], ya[at + i], sa);
+      sb = fmaf(yb[at + i], yb[at + i], sb);
+    }
+    const float ra = rsqrtf(block_sum(sa, scratch[0]) / static_cast<float>(h) + eps);
+    const float rb = rsqrtf(block_sum(sb, scratch[1]) / static_cast<float>(h) + eps);
+    for (int i = threadIdx.x; i < h; i += 256) x[at + i] += ya[at + i] * ra * wa[i] + yb[at + i] * rb * wb[i];
+  }
+}
+KVF_EXPORT int kvf_rms_add_two(float* x, const float* ya, const float* wa, const float* yb, const float* wb, float eps,
+                               int m, int h, hipStream_t s) {
+  if (m <= 0) return 0;
+  bool vec = h % 4 == 0 && h <= 8192;
+  for (const float* p : {static_cast<const float*>(x), ya, wa, yb, wb}) vec = vec && reinterpret_cast<uintptr_t>(p) % 16 == 0;
+#define GO(Q) hipLaunchKernelGGL(rms_add_two_kernel<Q>, dim3(m), dim3(256), 0, s, x, ya, wa, yb, wb, eps, h)
+  if (!vec) GO(0);
+  else if (h <= 1024) GO(1);
+  else if (h <= 2048) GO(2);
+  else if (h <= 4096) GO(4);
+  else GO(8);
+#undef GO
   return kvf_last_error();
 }
 

@@ -65,9 +65,10 @@ struct RopeEpi {
   bf16_t* k_pages;
   bf16_t* v_pages;
   int H, KV, d, rot, table_len, block_size, table_stride, num_blocks, write_kv, n_seqs;
-  // EPI 3: the gate's activation (0 silu, 1 the tanh form of gelu) and fp32 biases of the gate and
-  // up columns (by pair, may be null)
+  // EPI 3: how a pair is joined (GateForm's act and limit), what it is multiplied by, and fp32 biases
+  // of the gate and up columns (by pair, may be null)
   int act;
+  float act_limit, act_scale;
   const float* gate_bias;
   const float* up_bias;
 };
@@ -359,14 +360,16 @@ __device__ __forceinline__ void store_tile(const f32x4& s, int m, int n, int N, 
       float g = s[2 * pr], u = s[2 * pr + 1];
       if (rp.gate_bias) g += rp.gate_bias[n / 2 + pr];
       if (rp.up_bias) u += rp.up_bias[n / 2 + pr];
-      float a;
-      if (rp.act == 1) {
+      float y;
+      if (rp.act == GATE_LIMITED) {
+        y = limited_pair(g, u, rp.act_limit) * rp.act_scale;
+      } else if (rp.act == 1) {
         const float t = 0.7978845608028654f * (g + 0.044715f * g * g * g);
-        a = 0.5f * g * (1.f + tanhf(t));
+        y = 0.5f * g * (1.f + tanhf(t)) * u * rp.act_scale;
       } else {
-        a = g / (1.f + __expf(-g));
+        y = g / (1.f + __expf(-g)) * u * rp.act_scale;
       }
-      o[pr].bits = f32_to_bf16(a * u);
+      o[pr].bits = f32_to_bf16(y);
     }
   } else {
     // fused q/k/v projection: d is a multiple of 4, so the four columns lie in one head; pairs
@@ -759,7 +762,8 @@ KVF_EXPORT int kvf_gemm_bf16(const void* A, int a_type, const void* W, int w_til
     return static_cast<int>(hipErrorInvalidValue);
   if (((c_add || half_out) && epi != 2) || (half_out && (a_type != 0 || K < 64)))
     return static_cast<int>(hipErrorInvalidValue);
-  const RopeEpi none{};
+  RopeEpi none{};
+  none.act_scale = 1.f;
   const Riders rd{nullptr, static_cast<const bf16_t*>(c_add), static_cast<bf16_t*>(half_out)};
   const bf16_t* w = static_cast<const bf16_t*>(W);
   if (a_type == 0) return launch_epi<0>(A, w, C, epi, M, N, K, lda, ldc, eps, w_tiled, rd, none, s);
@@ -769,15 +773,18 @@ KVF_EXPORT int kvf_gemm_bf16(const void* A, int a_type, const void* W, int w_til
 
 // The gated pair epilogue (epi 3) with its activation chosen and biases: out[m, j] =
 // act(c[2j] + gate_bias[j]) * (c[2j+1] + up_bias[j]) as bf16 [M, N/2]; act 0 silu, 1 the tanh form
-// of gelu; the biases are fp32 [N/2] and may be null.
+// of gelu, 2 the limited form (GateForm), the whole times `scale`; the biases are fp32 [N/2] and may be null.
 KVF_EXPORT int kvf_gemm_bf16_gated(const void* A, int a_type, const void* W, int w_tiled, void* C,
                                    int M, int N, int K, int lda, int ldc, float eps, int act,
-                                   const float* gate_bias, const float* up_bias, hipStream_t s) {
+                                   float limit, float scale, const float* gate_bias, const float* up_bias, hipStream_t s) {
   if (M <= 0 || N <= 0) return 0;
-  if (K <= 0 || K % 8 != 0 || lda % 8 != 0 || N % 4 != 0 || act < 0 || act > 1)
+  if (K <= 0 || K % 8 != 0 || lda % 8 != 0 || N % 4 != 0 || act < 0 || act > GATE_LIMITED ||
+      (act == GATE_LIMITED && !(limit > 0.f)))
     return static_cast<int>(hipErrorInvalidValue);
   RopeEpi rp{};
   rp.act = act;
+  rp.act_limit = limit;
+  rp.act_scale = scale;
   rp.gate_bias = gate_bias;
   rp.up_bias = up_bias;
   const Riders rd{nullptr, nullptr, nullptr};
@@ -810,7 +817,7 @@ KVF_EXPORT int kvf_gemm_bf16_qkv_rope(const void* A, int a_type, const void* W, 
   const Riders rd{static_cast<const bf16_t*>(a_add), nullptr, nullptr};
   const RopeEpi rp{positions, seq_of_token, cos_t, sin_t, block_table,
                    static_cast<bf16_t*>(k_pages), static_cast<bf16_t*>(v_pages), H, KV, d, rot,
-                   table_len, block_size, table_stride, num_blocks, write_kv, n_seqs, 0, nullptr, nullptr};
+                   table_len, block_size, table_stride, num_blocks, write_kv, n_seqs, 0, 0.f, 1.f, nullptr, nullptr};
   const int N = (H + 2 * KV) * d + extra_cols;
   const bf16_t* w = static_cast<const bf16_t*>(W);
   if (a_type == 0) return launch_rows<0, 4>(A, w, q_out, M, N, K, lda, ldq, eps, w_tiled, rd, rp, s);

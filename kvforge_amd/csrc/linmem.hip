@@ -21,7 +21,7 @@
 //                   chunk, and the run's last state in the slot; pass 3 (the scan kernel again)
 //                   computes every chunk's outputs from that.
 //   linmem_out    : o / rms(o) * weight * silu(g) * scale per head (weight [dv] shared by the
-//                   heads, or none).
+//                   heads, or none); or with sigmoid(g) in place of silu(g).
 // Everything is fp32; the order of every sum is fixed by the shapes.
 #include "common.h"
 
@@ -215,8 +215,9 @@ __global__ __launch_bounds__(256) void linmem_carry_kernel(const int* __restrict
 }
 
 // A wave per (token, head): the head's root mean square, then weight, gate and scale.
-template <typename T>
-__global__ __launch_bounds__(KVF_WAVE) void linmem_out_kernel(const float* __restrict__ o, const T* __restrict__ g,
+// TG: the gate's type; SIG: sigmoid of the gate alone
+template <typename T, typename TG, bool SIG>
+__global__ __launch_bounds__(KVF_WAVE) void linmem_out_kernel(const float* __restrict__ o, const TG* __restrict__ g,
                                                               int g_stride, const float* __restrict__ w, float eps,
                                                               float scale, T* __restrict__ out, int H, int dv) {
   const int t = blockIdx.x, head = blockIdx.y, lane = threadIdx.x;
@@ -224,12 +225,12 @@ __global__ __launch_bounds__(KVF_WAVE) void linmem_out_kernel(const float* __res
   float ss = 0.f;
   for (int e = lane; e < dv; e += KVF_WAVE) ss = fmaf(orow[e], orow[e], ss);
   const float r = 1.f / sqrtf(wave_sum(ss) / static_cast<float>(dv) + eps);
-  const T* grow = g + static_cast<size_t>(t) * g_stride + head * dv;
+  const TG* grow = g + static_cast<size_t>(t) * g_stride + head * dv;
   T* dst = out + (static_cast<size_t>(t) * H + head) * dv;
   for (int e = lane; e < dv; e += KVF_WAVE) {
-    const float gv = Elem<T>::load(grow + e);
+    const float gv = Elem<TG>::load(grow + e);
     const float y = orow[e] * r * (w ? w[e] : 1.f);
-    Elem<T>::store(dst + e, y * (gv / (1.f + expf(-gv))) * scale);
+    Elem<T>::store(dst + e, y * ((SIG ? 1.f : gv) / (1.f + expf(-gv))) * scale);
   }
 }
 
@@ -320,16 +321,29 @@ KVF_EXPORT int kvf_linmem_chunks(LINMEM_ARGS_DECL, const int* chunks, int n_chun
   return static_cast<int>(hipErrorInvalidValue);
 }
 
-// w: null (no weight) or [dv] shared by the heads.
+// w: null (no weight) or [dv] shared by the heads.  gate_f32: the gate is fp32 whatever the output's type;
+// sigmoid: the gate is sigmoid(g), not silu(g) (with an fp32 gate).
 KVF_EXPORT int kvf_linmem_out(int dtype, const float* o, const void* g, int g_stride, const float* w, float eps,
-                              float scale, void* out, int n, int H, int dv, hipStream_t s) {
+                              float scale, void* out, int n, int H, int dv, int gate_f32, int sigmoid, hipStream_t s) {
   if (n <= 0) return 0;
-  if (H <= 0 || H > 65535 || dv <= 0) return static_cast<int>(hipErrorInvalidValue);
+  if (H <= 0 || H > 65535 || dv <= 0 || (sigmoid && !gate_f32) || (gate_f32 && !sigmoid && dtype != 0))
+    return static_cast<int>(hipErrorInvalidValue);
+  if (sigmoid) {
+    if (dtype == 0)
+      hipLaunchKernelGGL((linmem_out_kernel<float, float, true>), dim3(n, H), dim3(KVF_WAVE), 0, s, o,
+                         static_cast<const float*>(g), g_stride, w, eps, scale, static_cast<float*>(out), H, dv);
+    else if (dtype == 1)
+      hipLaunchKernelGGL((linmem_out_kernel<bf16_t, float, true>), dim3(n, H), dim3(KVF_WAVE), 0, s, o,
+                         static_cast<const float*>(g), g_stride, w, eps, scale, static_cast<bf16_t*>(out), H, dv);
+    else
+      return static_cast<int>(hipErrorInvalidValue);
+    return kvf_last_error();
+  }
   if (dtype == 0)
-    hipLaunchKernelGGL(linmem_out_kernel<float>, dim3(n, H), dim3(KVF_WAVE), 0, s, o, static_cast<const float*>(g),
+    hipLaunchKernelGGL((linmem_out_kernel<float, float, false>), dim3(n, H), dim3(KVF_WAVE), 0, s, o, static_cast<const float*>(g),
                        g_stride, w, eps, scale, static_cast<float*>(out), H, dv);
   else if (dtype == 1)
-    hipLaunchKernelGGL(linmem_out_kernel<bf16_t>, dim3(n, H), dim3(KVF_WAVE), 0, s, o, static_cast<const bf16_t*>(g),
+    hipLaunchKernelGGL((linmem_out_kernel<bf16_t, bf16_t, false>), dim3(n, H), dim3(KVF_WAVE), 0, s, o, static_cast<const bf16_t*>(g),
                        g_stride, w, eps, scale, static_cast<bf16_t*>(out), H, dv);
   else
     return static_cast<int>(hipErrorInvalidValue);

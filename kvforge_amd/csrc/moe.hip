@@ -6,14 +6,18 @@ namespace {
 constexpr int MAX_PER_LANE = 8;   // router outputs per lane: up to 512 of them
 constexpr int MAX_TOP = 16;
 
-// A wave per token.  s = softmax(z) over all R router outputs, or (`sigmoid`) s = sigmoid(z) of each by
-// itself; the `top` outputs with the largest s + correction (null: none) are chosen (the lowest index
-// among equals), and weighted by their s alone, divided (`renorm`) by the sum of the chosen s
-// (+ 1e-20).  sel [N, top], wgt [N, top].
+// A wave per token; z gets a bias per output first (null: none).  SCORE_SOFTMAX: s = softmax(z) over all R
+// router outputs; SCORE_SIGMOID: s = sigmoid(z) of each by itself; the `top` outputs with the largest
+// s + correction (null: none) are chosen (the lowest index among equals), and weighted by their s
+// alone, divided (`renorm`) by the sum of the chosen s (+ 1e-20).  SCORE_CHOSEN: the outputs with the
+// largest z are chosen, and weighted by the softmax over the chosen z.  The weights are then
+// multiplied by `scale`.  sel [N, top], wgt [N, top].
+enum { SCORE_SOFTMAX = 0, SCORE_SIGMOID = 1, SCORE_CHOSEN = 2 };
 __global__ __launch_bounds__(KVF_WAVE) void moe_topk_kernel(const float* __restrict__ z, int z_stride,
+                                                            const float* __restrict__ bias,
                                                             const float* __restrict__ correction,
                                                             int* __restrict__ sel, float* __restrict__ wgt,
-                                                            int R, int top, int sigmoid, int renorm) {
+                                                            int R, int top, int score, int renorm, float scale) {
   const int n = blockIdx.x, lane = threadIdx.x;
   const float* zr = z + static_cast<size_t>(n) * z_stride;
   float s[MAX_PER_LANE], c[MAX_PER_LANE];
@@ -21,13 +25,13 @@ __global__ __launch_bounds__(KVF_WAVE) void moe_topk_kernel(const float* __restr
 #pragma unroll
   for (int j = 0; j < MAX_PER_LANE; ++j) {
     const int e = lane + KVF_WAVE * j;
-    s[j] = e < R ? zr[e] : -INFINITY;
+    s[j] = e < R ? zr[e] + (bias ? bias[e] : 0.f) : -INFINITY;
     mx = fmaxf(mx, s[j]);
   }
-  if (sigmoid) {
+  if (score == SCORE_SIGMOID) {
 #pragma unroll
     for (int j = 0; j < MAX_PER_LANE; ++j) s[j] = 1.f / (1.f + expf(-s[j]));
-  } else {
+  } else if (score == SCORE_SOFTMAX) {
     mx = wave_max(mx);
     float sum = 0.f;
 #pragma unroll
@@ -78,23 +82,33 @@ __global__ __launch_bounds__(KVF_WAVE) void moe_topk_kernel(const float* __restr
       picked_e = cand;
     }
   }
+  if (score == SCORE_CHOSEN) {   // the first choice has the largest z
+    picked_s = lane < top ? expf(picked_s - __shfl(picked_s, 0, KVF_WAVE)) : 0.f;
+    total = wave_sum(picked_s);
+  }
   if (lane < top) {
     sel[static_cast<size_t>(n) * top + lane] = picked_e;
-    wgt[static_cast<size_t>(n) * top + lane] = renorm ? picked_s / (total + 1e-20f) : picked_s;
+    wgt[static_cast<size_t>(n) * top + lane] =
+        (score == SCORE_CHOSEN ? picked_s / total : renorm ? picked_s / (total + 1e-20f) : picked_s) * scale;
   }
 }
 
 __device__ __forceinline__ float silu(float g) { return g / (1.f + expf(-g)); }
+// an expert's (gate, up) pair joined: silu(g) u, or the limited form (GateForm)
+__device__ __forceinline__ float joined(const GateForm& f, float g, float u) {
+  return f.act == GATE_LIMITED ? limited_pair_exact(g, u, f.limit) : silu(g) * u;
+}
 
 // Every expert's gate/up pair for every token is there (one product over all experts, columns
 // 2 (e ff + j) and 2 (e ff + j) + 1): act[n, e ff + j] = weight(n, e) * silu(gate) * up where the
 // token chose expert e, and an exact zero elsewhere, so that one product with the experts' down
 // matrices side by side along K is the weighted sum over the chosen experts.  `weigh_input`: the weight
-// belongs to the expert's input, act = silu(w gate) * (w up) (gate and up are linear in it).
+// belongs to the expert's input, act = silu(w gate) * (w up) (gate and up are linear in it).  `f`: how a
+// pair is joined where it is not by silu.
 template <typename T>
 __global__ void moe_dense_act_kernel(const T* __restrict__ gu, const int* __restrict__ sel,
                                      const float* __restrict__ wgt, T* __restrict__ act, int E, int ff,
-                                     int top, int weigh_input, long total) {
+                                     int top, int weigh_input, GateForm f, long total) {
   const long i = static_cast<long>(blockIdx.x) * blockDim.x + threadIdx.x;
   if (i >= total) return;
   const long cols = static_cast<long>(E) * ff;
@@ -110,7 +124,7 @@ __global__ void moe_dense_act_kernel(const T* __restrict__ gu, const int* __rest
   float y = 0.f;
   if (chosen) {
     const float g = Elem<T>::load(gu + 2 * i), u = Elem<T>::load(gu + 2 * i + 1);
-    y = weigh_input ? silu(w * g) * (w * u) : w * (silu(g) * u);
+    y = weigh_input ? joined(f, w * g, w * u) : w * joined(f, g, u);
   }
   Elem<T>::store(act + i, y);
 }
@@ -200,7 +214,8 @@ __global__ __launch_bounds__(256) void moe_up_kernel(const bf16_t* __restrict__ 
                                                      const int* __restrict__ order,
                                                      const int* __restrict__ tiles,
                                                      const int* __restrict__ num_tiles, int top, int ff,
-                                                     const float* __restrict__ in_wgt, bf16_t* __restrict__ act) {
+                                                     const float* __restrict__ in_wgt, GateForm f,
+                                                     bf16_t* __restrict__ act) {
   const int tile = blockIdx.y;
   if (tile >= *num_tiles) return;
   const int e = tiles[3 * tile], row0 = tiles[3 * tile + 1], rows = tiles[3 * tile + 2];
@@ -263,7 +278,7 @@ __global__ __launch_bounds__(256) void moe_up_kernel(const bf16_t* __restrict__ 
     for (int g = 0; g < GW; ++g) {
       if (g_first + g >= groups) continue;
       const int col = (g_first + g) * 8 + 2 * c;
-      const float y0 = silu(w * acc[r][g][0]) * (w * acc[r][g][1]), y1 = silu(w * acc[r][g][2]) * (w * acc[r][g][3]);
+      const float y0 = joined(f, w * acc[r][g][0], w * acc[r][g][1]), y1 = joined(f, w * acc[r][g][2], w * acc[r][g][3]);
       *reinterpret_cast<uint32_t*>(out + col) =
           static_cast<uint32_t>(f32_to_bf16(y0)) | (static_cast<uint32_t>(f32_to_bf16(y1)) << 16);
     }
@@ -401,13 +416,16 @@ __global__ void moe_table_kernel(const int* __restrict__ tokens, const int* __re
 }
 }  // namespace
 
-KVF_EXPORT int kvf_moe_topk(const float* z, int z_stride, const float* correction, int* sel, float* wgt,
-                            int n, int R, int top, int sigmoid, int renorm, hipStream_t s) {
+static bool form_ok(int act, float limit) { return act == 0 || (act == GATE_LIMITED && limit > 0.f); }
+
+KVF_EXPORT int kvf_moe_topk(const float* z, int z_stride, const float* bias, const float* correction, int* sel,
+                            float* wgt, int n, int R, int top, int score, int renorm, float scale, hipStream_t s) {
   if (n <= 0) return 0;
-  if (R <= 0 || R > MAX_PER_LANE * KVF_WAVE || top <= 0 || top > MAX_TOP || top > R)
+  if (score < SCORE_SOFTMAX || score > SCORE_CHOSEN || (score == SCORE_CHOSEN && correction) ||
+      R <= 0 || R > MAX_PER_LANE * KVF_WAVE || top <= 0 || top > MAX_TOP || top > R)
     return static_cast<int>(hipErrorInvalidValue);
-  hipLaunchKernelGGL(moe_topk_kernel, dim3(n), dim3(KVF_WAVE), 0, s, z, z_stride, correction, sel, wgt, R, top,
-                     sigmoid, renorm);
+  hipLaunchKernelGGL(moe_topk_kernel, dim3(n), dim3(KVF_WAVE), 0, s, z, z_stride, bias, correction, sel, wgt, R,
+                     top, score, renorm, scale);
   return kvf_last_error();
 }
 
@@ -421,16 +439,18 @@ KVF_EXPORT int kvf_moe_table(const int* tokens, const int* table, int* sel, floa
 }
 
 KVF_EXPORT int kvf_moe_dense_act(int dtype, const void* gu, const int* sel, const float* wgt, void* act,
-                                 int n, int E, int ff, int top, int weigh_input, hipStream_t s) {
+                                 int n, int E, int ff, int top, int weigh_input, int form, float limit, hipStream_t s) {
   const long total = static_cast<long>(n) * E * ff;
   if (total <= 0) return 0;
+  if (!form_ok(form, limit)) return static_cast<int>(hipErrorInvalidValue);
+  const GateForm f{form, limit, 1.f};
   const dim3 grid(static_cast<unsigned>((total + 255) / 256));
   if (dtype == 0)
     hipLaunchKernelGGL(moe_dense_act_kernel<float>, grid, dim3(256), 0, s, static_cast<const float*>(gu), sel,
-                       wgt, static_cast<float*>(act), E, ff, top, weigh_input, total);
+                       wgt, static_cast<float*>(act), E, ff, top, weigh_input, f, total);
   else if (dtype == 1)
     hipLaunchKernelGGL(moe_dense_act_kernel<bf16_t>, grid, dim3(256), 0, s, static_cast<const bf16_t*>(gu), sel,
-                       wgt, static_cast<bf16_t*>(act), E, ff, top, weigh_input, total);
+                       wgt, static_cast<bf16_t*>(act), E, ff, top, weigh_input, f, total);
   else
     return static_cast<int>(hipErrorInvalidValue);
   return kvf_last_error();
@@ -455,17 +475,19 @@ KVF_EXPORT int kvf_moe_identity(int dtype, float* x, const void* h, const int* s
 // and [K, E ff]; sel / wgt [n, top]; scratch: where, order [n top], tiles [3 max_tiles],
 // num_tiles [1], act [n top, ff], y [n top, K].  Needs K % 8 == 0 and ff % 32 == 0.  weigh_input: the
 // weights go into the experts' inputs instead of the sum over their outputs.  fresh: residual is
-// written, not added to.
+// written, not added to.  form, limit: how an expert's pairs are joined (GateForm's act 0 or 2).
 KVF_EXPORT int kvf_moe_grouped(const void* x, int ldx, const void* h, int n, int K, int E, int ff, int top,
                                const void* w_gate_up, const void* w_down, const int* sel, const float* wgt,
                                int* where, int* order, int* tiles, int* num_tiles, int max_tiles, void* act,
-                               void* y, float* residual, int weigh_input, int fresh, hipStream_t s) {
+                               void* y, float* residual, int weigh_input, int fresh, int form, float limit,
+                               hipStream_t s) {
   if (n <= 0) return 0;
   const int pairs = n * top;
   // many rows: tiles of 64 rows (four sub-tiles share every weight fragment); few: tiles of 16
   const bool many = pairs >= 1024;
   const int tile_rows = many ? 64 : 16;
-  if (E <= 0 || E > PLAN_MAX_EXPERTS || K % 8 != 0 || ff % 32 != 0 || ldx % 8 != 0 || max_tiles > 65535 ||
+  const GateForm f{form, limit, 1.f};
+  if (!form_ok(form, limit) || E <= 0 || E > PLAN_MAX_EXPERTS || K % 8 != 0 || ff % 32 != 0 || ldx % 8 != 0 || max_tiles > 65535 ||
       max_tiles < (pairs + 15) / 16 + E)
     return static_cast<int>(hipErrorInvalidValue);
   hipLaunchKernelGGL(moe_plan_kernel, dim3(1), dim3(1024), 0, s, sel, pairs, E, where, order, tiles, num_tiles,
@@ -478,12 +500,12 @@ KVF_EXPORT int kvf_moe_grouped(const void* x, int ldx, const void* h, int n, int
   const float* in_wgt = weigh_input ? wgt : nullptr;
   if (many) {
     hipLaunchKernelGGL((moe_up_kernel<4, 4>), up_grid, dim3(256), 0, s, xb, ldx, K, static_cast<const uint4*>(w_gate_up), S,
-                       order, tiles, num_tiles, top, ff, in_wgt, static_cast<bf16_t*>(act));
+                       order, tiles, num_tiles, top, ff, in_wgt, f, static_cast<bf16_t*>(act));
     hipLaunchKernelGGL((moe_down_kernel<4, 4>), down_grid, dim3(256), 0, s, static_cast<const bf16_t*>(act), ff,
                        static_cast<const uint4*>(w_down), E * (ff / 32), tiles, num_tiles, static_cast<bf16_t*>(y), K);
   } else {
     hipLaunchKernelGGL((moe_up_kernel<1, 1>), up_grid, dim3(256), 0, s, xb, ldx, K, static_cast<const uint4*>(w_gate_up), S,
-                       order, tiles, num_tiles, top, ff, in_wgt, static_cast<bf16_t*>(act));
+                       order, tiles, num_tiles, top, ff, in_wgt, f, static_cast<bf16_t*>(act));
     hipLaunchKernelGGL((moe_down_kernel<1, 1>), down_grid, dim3(256), 0, s, static_cast<const bf16_t*>(act), ff,
                        static_cast<const uint4*>(w_down), E * (ff / 32), tiles, num_tiles, static_cast<bf16_t*>(y), K);
   }

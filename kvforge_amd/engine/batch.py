@@ -197,6 +197,9 @@ class Step:
         # library product over many rows leaves it here instead of running an add kernel; the
         # next norm adds it on its way (``take_owed``), anything else calls ``settle`` first.
         self.owed: tuple[torch.Tensor, torch.Tensor] | None = None
+        # A vector still owed to every row of the stream: (stream, fp32 vector), the bias of a
+        # feed-forward's last product; a norm that adds biases takes it (``take_owed_bias``).
+        self.owed_bias: tuple[torch.Tensor, torch.Tensor] | None = None
         # Rows that a block has handed to a sublayer in place of the stream and that hold
         # nothing yet: the sublayer's last product is written there instead of added
         # (``parts.base.add_product``), which then forgets the mark.
@@ -228,8 +231,31 @@ class Step:
         self.settle()
         self.owed = (residual, product)
 
+    def owe_bias(self, residual: torch.Tensor, bias: torch.Tensor) -> None:
+        self._settle_bias()
+        self.owed_bias = (residual, bias)
+
+    def take_owed_bias(self, residual: torch.Tensor) -> torch.Tensor | None:
+        """The vector owed to every row of ``residual``, for a norm kernel that adds it itself (to be
+        asked for before ``take_owed``, which otherwise brings the stream up to date)."""
+        if self.owed_bias is None:
+            return None
+        if self.owed_bias[0] is not residual:
+            self.settle()
+            return None
+        bias = self.owed_bias[1]
+        self.owed_bias = None
+        return bias
+
+    def _settle_bias(self) -> None:
+        if self.owed_bias is not None:
+            from kvforge_amd.kernels import ops
+            ops.add_bias(*self.owed_bias)
+            self.owed_bias = None
+
     def take_owed(self, residual: torch.Tensor) -> torch.Tensor | None:
         """The product owed to ``residual``, for a norm kernel that adds it itself."""
+        self._settle_bias()
         if self.owed is None:
             return None
         if self.owed[0] is not residual or len(self.owed) != 2:
@@ -243,6 +269,7 @@ class Step:
         """``(rows, weight, eps)`` if what is owed to ``residual`` is the RMS norm of fp32 rows (a
         sublayer's output that joins the stream through a norm of its own), for a kernel that
         adds it itself; ``None`` otherwise (whatever else is owed stays owed)."""
+        self._settle_bias()
         if self.owed is None or self.owed[0] is not residual or len(self.owed) != 4:
             return None
         owed = self.owed[1:]
@@ -251,7 +278,8 @@ class Step:
 
     def settle(self) -> None:
         """Add what is owed to the residual stream now: ``(stream, rows)``, or ``(stream, rows,
-        weight, eps)`` for rows that join through their RMS norm."""
+        weight, eps)`` for rows that join through their RMS norm; and a bias owed to every row."""
+        self._settle_bias()
         if self.owed is not None:
             from kvforge_amd.kernels import ops
             if len(self.owed) == 4:

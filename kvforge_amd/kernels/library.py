@@ -50,6 +50,8 @@ MODULES: dict[str, list[str]] = {
     "wkv": ["wkv.hip"],
     "linmem": ["linmem.hip"],
     "ssm": ["ssm.hip"],
+    "convkv": ["convkv.hip"],
+    "chdelta": ["chdelta.hip"],
 }
 
 

@@ -124,11 +124,13 @@ def softcap(x: torch.Tensor, cap: float | None, scale: float = 1.0) -> None:
 
 # ------------------------------------------------------------------------------ RMS norm
 def rmsnorm(x: torch.Tensor, weight: torch.Tensor | None, eps: float, out: torch.Tensor,
-            rows: torch.Tensor | None = None, add: torch.Tensor | None = None) -> None:
+            rows: torch.Tensor | None = None, add: torch.Tensor | None = None,
+            bias: torch.Tensor | None = None) -> None:
     """``out[m] = y * rsqrt(mean(y^2) + eps) * weight`` with ``y = x[rows[m] or m]`` in fp32
     (``weight=None``: no weight, for a norm whose weight is folded into the next matrix).
     ``add`` (``[rows of x, h]``, dtype of ``out`` or fp32) is a sum still owed to ``x``: the norm
-    is taken of ``x + add``, and without ``rows`` the sum is written back to ``x`` as well."""
+    is taken of ``x + add``, and without ``rows`` the sum is written back to ``x`` as well.  ``bias``
+    (fp32 ``[h]``): a vector still owed to every row of ``x``, likewise."""
     _check(x, "x", F32, (None, None))
     xr, h = x.shape
     m = out.shape[0]
@@ -145,12 +147,15 @@ def rmsnorm(x: torch.Tensor, weight: torch.Tensor | None, eps: float, out: torch
         _check(add, "add", None, (xr, h))
         if add.dtype not in (F32, out.dtype):
             raise KernelError(f"rmsnorm: add must be float32 or {out.dtype}, got {add.dtype}")
+    if bias is not None:
+        _check(bias, "bias", F32, (h,))
     f = _fn("elementwise", f"kvf_rmsnorm_{_suffix(out.dtype)}",
-            [c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_int, c_float, c_void_p, c_int, c_int,
+            [c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_int, c_float, c_void_p, c_int, c_int,
              c_int, c_void_p])
     _ok(f(x.data_ptr(), rows.data_ptr() if rows is not None else None,
           add.data_ptr() if add is not None else None,
           1 if add is not None and add.dtype == F32 else 0,
+          bias.data_ptr() if bias is not None else None,
           weight.data_ptr() if weight is not None else None,
           1 if weight is not None and weight.dtype == F32 else 0, float(eps), out.data_ptr(),
           m, h, xr, _stream()), "rmsnorm")
@@ -231,28 +236,41 @@ def norm_shift(x: torch.Tensor, weight: torch.Tensor, mu: torch.Tensor, state: t
 
 
 ACTIVATIONS = {"silu": 0, "gelu_tanh": 1}
+# ... and one that joins the pair in a way of its own: g = min(gate, limit), u = clamp(up, -limit, limit),
+# g sigmoid(1.702 g) (u + 1)
+GATE_FORMS = dict(ACTIVATIONS, limited=2)
+
+
+def _gate_form(activation: str, limit: float | None, who: str) -> tuple[int, float]:
+    """(code, limit) of a gated pair's form as the kernels take it."""
+    if activation not in GATE_FORMS:
+        raise KernelError(f"{who}: unknown activation {activation!r}; known: {sorted(GATE_FORMS)}")
+    if (activation == "limited") != (limit is not None) or (limit is not None and not limit > 0.0):
+        raise KernelError(f"{who}: a positive limit goes with the limited form, got {activation!r} and {limit}")
+    return GATE_FORMS[activation], float(limit or 0.0)
 
 
 def gated_act(gate_up: torch.Tensor, out: torch.Tensor, activation: str, paired: bool = False,
-              gate_bias: torch.Tensor | None = None, up_bias: torch.Tensor | None = None) -> None:
-    """``out[:, i] = act(gate_i + gate_bias[i]) * (up_i + up_bias[i])``; the input row holds gate
-    at ``i`` and up at ``I + i``, or with ``paired`` at ``2i`` and ``2i + 1``.  ``activation``:
-    ``"silu"`` or ``"gelu_tanh"``; the biases are fp32 ``[I]`` or ``None``."""
+              gate_bias: torch.Tensor | None = None, up_bias: torch.Tensor | None = None,
+              limit: float | None = None, scale: float = 1.0) -> None:
+    """``out[:, i] = act(gate_i + gate_bias[i]) * (up_i + up_bias[i]) * scale``; the input row holds
+    gate at ``i`` and up at ``I + i``, or with ``paired`` at ``2i`` and ``2i + 1``.  ``activation``:
+    ``"silu"``, ``"gelu_tanh"`` or ``"limited"`` (with ``limit``; see ``GATE_FORMS``); the biases are fp32
+    ``[I]`` or ``None``."""
     m, two_i = gate_up.shape
     if two_i % 2:
         raise KernelError("gated_act: input width must be even")
-    if activation not in ACTIVATIONS:
-        raise KernelError(f"gated_act: unknown activation {activation!r}; known: {sorted(ACTIVATIONS)}")
+    act, lim = _gate_form(activation, limit, "gated_act")
     _check(gate_up, "gate_up", None, (m, two_i))
     _check(out, "out", gate_up.dtype, (m, two_i // 2))
     for b, name in ((gate_bias, "gate_bias"), (up_bias, "up_bias")):
         if b is not None:
             _check(b, name, F32, (two_i // 2,))
     f = _fn("elementwise", f"kvf_gated_act_{_suffix(out.dtype)}",
-            [c_void_p] * 4 + [c_int] * 4 + [c_void_p])
+            [c_void_p] * 4 + [c_int] * 4 + [c_float, c_float, c_void_p])
     _ok(f(gate_up.data_ptr(), gate_bias.data_ptr() if gate_bias is not None else None,
           up_bias.data_ptr() if up_bias is not None else None, out.data_ptr(), m, two_i // 2,
-          1 if paired else 0, ACTIVATIONS[activation], _stream()), "gated_act")
+          1 if paired else 0, act, lim, float(scale), _stream()), "gated_act")
 
 
 def sigmoid_gate(y: torch.Tensor, gate: torch.Tensor) -> None:
@@ -369,6 +387,21 @@ def rms_add(x: torch.Tensor, y: torch.Tensor, weight: torch.Tensor, eps: float) 
         "rms_add")
 
 
+def rms_add_two(x: torch.Tensor, ya: torch.Tensor, wa: torch.Tensor, yb: torch.Tensor, wb: torch.Tensor,
+                eps: float) -> None:
+    """``x[m] += ya[m] * rsqrt(mean(ya[m]^2) + eps) * wa + yb[m] * rsqrt(mean(yb[m]^2) + eps) * wb``, all fp32."""
+    _check(x, "x", F32, (None, None))
+    for t, name in ((ya, "ya"), (yb, "yb")):
+        _check(t, name, F32, tuple(x.shape))
+        if _overlap(x, t):
+            raise KernelError(f"rms_add_two: x must not share memory with {name}")
+    _check(wa, "wa", F32, (x.shape[1],))
+    _check(wb, "wb", F32, (x.shape[1],))
+    f = _fn("elementwise", "kvf_rms_add_two", [c_void_p] * 5 + [c_float, c_int, c_int, c_void_p])
+    _ok(f(x.data_ptr(), ya.data_ptr(), wa.data_ptr(), yb.data_ptr(), wb.data_ptr(), float(eps), x.shape[0], x.shape[1],
+          _stream()), "rms_add_two")
+
+
 def rms_add_cast(x: torch.Tensor, y: torch.Tensor, weight: torch.Tensor, eps: float, out: torch.Tensor) -> None:
     """``rms_add`` and a copy of the sum in one pass: ``x[m] += y[m] * rsqrt(mean(y[m]^2) + eps) * weight``,
     then ``out[m] = x[m]`` in ``out``'s type."""
@@ -464,6 +497,68 @@ def rope_kvwrite(qkv: torch.Tensor, positions: torch.Tensor, seq_of_token: torch
           n, H, KV, d, rot, table_len, bs, stride, nb, 1 if write_kv else 0, n_seqs,
           qkv.shape[1], _stream()),
         "rope_kvwrite")
+
+
+CONVKV_MAX_TAPS = 8
+
+
+def convkv_state_floats(heads: int, kv_heads: int, head_dim: int, taps: int) -> int:
+    """fp32 numbers of a request's slot: the last ``taps - 1`` projected rows of q, k and v."""
+    return (int(taps) - 1) * (int(heads) + 2 * int(kv_heads)) * int(head_dim)
+
+
+def conv_norm_kvwrite(rows: torch.Tensor, weight: torch.Tensor, cu_q: torch.Tensor, positions: torch.Tensor,
+                      slot_ids: torch.Tensor, state: torch.Tensor | None, block_table: torch.Tensor, q_out: torch.Tensor,
+                      k_pages: torch.Tensor, v_pages: torch.Tensor, num_heads: int, num_kv_heads: int, head_dim: int,
+                      n_seqs: int, longest: int, norm_dim: int | None = None, eps: float = 0.0,
+                      q_weight: torch.Tensor | None = None, k_weight: torch.Tensor | None = None) -> None:
+    """A short causal convolution over time on every channel of the projected q, k and v heads
+    (``rows [n, >= (H + 2 KV) d]``; ``weight`` fp32 ``[(H + 2 KV) d, taps]``, whose last tap meets the token itself), then with
+    ``norm_dim`` an RMS norm of every q and k head over its first ``norm_dim`` elements (the others are zero; optional
+    weights ``[norm_dim]`` that the heads share), then q to ``q_out [n, H d]`` and k and v to the pages; fp32 with one
+    rounding.  What lies before a run is read from the sequence's slot (``taps - 1`` rows of all channels, the
+    oldest first; zeros at position 0), where the run leaves its own last rows; ``state`` may be a block of columns of
+    wider slots (``None`` with one tap).  ``longest``: tokens of the longest run."""
+    n = rows.shape[0]
+    H, KV, d = int(num_heads), int(num_kv_heads), int(head_dim)
+    C, taps = weight.shape
+    _check(rows, "rows", None, (n, None), contiguous=False)
+    if rows.stride(1) != 1 or rows.shape[1] < (H + 2 * KV) * d or (n > 1 and rows.stride(0) % 4) or rows.data_ptr() % 16:
+        raise KernelError("conv_norm_kvwrite: dense rows that hold q, k and v and start on 16 bytes")
+    _check(weight, "weight", F32, ((H + 2 * KV) * d, taps))
+    if not 1 <= taps <= CONVKV_MAX_TAPS or d % 16 or not 0 < d <= 256:
+        raise KernelError(f"conv_norm_kvwrite: 1 to {CONVKV_MAX_TAPS} taps and heads in steps of 16 up to 256, got {taps} and {d}")
+    if norm_dim is not None and not 0 < norm_dim <= d:
+        raise KernelError(f"conv_norm_kvwrite: a norm over {norm_dim} of {d} elements")
+    for t, name in ((q_weight, "q_weight"), (k_weight, "k_weight")):
+        if t is not None:
+            _check(t, name, F32, (norm_dim,))
+    if (q_weight is None) != (k_weight is None):
+        raise KernelError("conv_norm_kvwrite: the norms of q and k both have weights or neither has")
+    for t, name in ((cu_q, "cu_q"), (positions, "positions"), (slot_ids, "slot_ids")):
+        _check(t, name, I32, (None,))
+    _check(block_table, "block_table", I32, (None, None))
+    if (cu_q.shape[0] < n_seqs + 1 or slot_ids.shape[0] < n_seqs or positions.shape[0] < n or block_table.shape[0] < n_seqs
+            or not 0 < longest <= n):
+        raise KernelError("conv_norm_kvwrite: batch arrays shorter than the batch")
+    slots = (0, 0)
+    if taps > 1:
+        slots = _slots(state, "conv_norm_kvwrite")
+        if state.shape[1] < (taps - 1) * C or slots[1] % 4 or state.data_ptr() % 16:
+            raise KernelError(f"conv_norm_kvwrite: slots of {state.shape[1]} floats do not hold {taps - 1} x {C} inputs on 16 bytes")
+    _check(q_out, "q_out", rows.dtype, (n, H * d))
+    _check(k_pages, "k_pages", rows.dtype, (None, KV, None, d))
+    nb, _, bs, _ = k_pages.shape
+    _check(v_pages, "v_pages", rows.dtype, (nb, KV, d, bs))
+    f = _fn("convkv", "kvf_conv_norm_kvwrite",
+            [c_int, c_void_p, c_int, c_int, c_void_p, c_int, c_int, c_float] + [c_void_p] * 6 + [c_int, c_void_p]
+            + [c_int] * 2 + [c_void_p, c_int] + [c_void_p] * 2 + [c_int] * 7 + [c_void_p])
+    _ok(f(_tcode(rows.dtype), rows.data_ptr(), rows.stride(0) if n > 1 else rows.shape[1], taps, weight.data_ptr(),
+          1 if norm_dim is not None else 0, int(norm_dim or d), float(eps),
+          q_weight.data_ptr() if q_weight is not None else None, k_weight.data_ptr() if k_weight is not None else None,
+          cu_q.data_ptr(), positions.data_ptr(), slot_ids.data_ptr(), block_table.data_ptr(), block_table.shape[1],
+          state.data_ptr() if taps > 1 else None, *slots, q_out.data_ptr(), q_out.shape[1], k_pages.data_ptr(),
+          v_pages.data_ptr(), H, KV, d, bs, nb, int(n_seqs), int(longest), _stream()), "conv_norm_kvwrite")
 
 
 def qknorm_rope_kvwrite(qkv: torch.Tensor, positions: torch.Tensor, seq_of_token: torch.Tensor,
@@ -867,10 +962,10 @@ def gemm_generic_vector_alus_only(on: bool) -> bool:
 
 def gemm_gated(a: torch.Tensor, w, out: torch.Tensor, activation: str = "silu",
                gate_bias: torch.Tensor | None = None, up_bias: torch.Tensor | None = None,
-               rms_eps: float | None = None) -> None:
+               rms_eps: float | None = None, limit: float | None = None, scale: float = 1.0) -> None:
     """The MFMA weight-streaming product over (gate, up) row pairs of ``w`` with the gate folded
-    into its store: ``out[:, j] = act(c[2j] + gate_bias[j]) * (c[2j+1] + up_bias[j])``,
-    ``out: [M, N/2]`` bf16.  ``activation``: ``"silu"`` or ``"gelu_tanh"``; biases fp32 ``[N/2]`` or
+    into its store: ``out[:, j] = act(c[2j] + gate_bias[j]) * (c[2j+1] + up_bias[j]) * scale``,
+    ``out: [M, N/2]`` bf16.  ``activation``, ``limit``: as in ``gated_act``; biases fp32 ``[N/2]`` or
     ``None``; ``rms_eps`` as in ``gemm_fused``.  Callers check ``bf16_kernel_takes`` first."""
     rms = rms_eps is not None
     m, n, k, lda, ldc = _gemm_operands(a, w, out, lambda n: n // 2)
@@ -878,19 +973,18 @@ def gemm_gated(a: torch.Tensor, w, out: torch.Tensor, activation: str = "silu",
         raise KernelError("gemm_gated: operands do not fit the MFMA kernel")
     if n % 4 or out.dtype != BF16:
         raise KernelError("gemm_gated: pairs need N in steps of 4 and a bf16 output")
-    if activation not in ACTIVATIONS:
-        raise KernelError(f"gemm_gated: unknown activation {activation!r}; known: {sorted(ACTIVATIONS)}")
+    act, lim = _gate_form(activation, limit, "gemm_gated")
     for b, name in ((gate_bias, "gate_bias"), (up_bias, "up_bias")):
         if b is not None:
             _check(b, name, F32, (n // 2,))
     if m == 0:
         return
     f = _fn("gemm_bf16", "kvf_gemm_bf16_gated",
-            [c_void_p, c_int, c_void_p, c_int, c_void_p] + [c_int] * 5 + [c_float, c_int, c_void_p, c_void_p,
-                                                                        c_void_p])
+            [c_void_p, c_int, c_void_p, c_int, c_void_p] + [c_int] * 5 + [c_float, c_int, c_float, c_float]
+            + [c_void_p] * 3)
     wp, tiled = _w_args(w)
     _ok(f(a.data_ptr(), 1 if rms else 0, wp, tiled, out.data_ptr(), m, n, k, lda, ldc, float(rms_eps or 0.0),
-          ACTIVATIONS[activation], gate_bias.data_ptr() if gate_bias is not None else None,
+          act, lim, float(scale), gate_bias.data_ptr() if gate_bias is not None else None,
           up_bias.data_ptr() if up_bias is not None else None, _stream()), "gemm_gated")
 
 
@@ -1103,6 +1197,19 @@ def _sinks_ptr(sinks, H: int, like: torch.Tensor):
     return sinks.data_ptr()
 
 
+def _dist_args(dist, H: int, like: torch.Tensor, slopes, sinks, cap: float, window: int, on_matrix_cores: bool):
+    """(pointer, distances) of a table of biases by distance (fp32 ``[H, distances]``), or (None, 0)."""
+    if dist is None:
+        return None, 0
+    _check(dist, "dist", F32, (H, None))
+    if dist.device != like.device or dist.shape[1] < 1 or dist.numel() >= 2**31:
+        raise KernelError("attention: biases by distance are a table of at least one column on the device of q")
+    if on_matrix_cores and (slopes is not None or sinks is not None or cap > 0.0 or window < 0):
+        raise KernelError("attention: the matrix-core kernels take biases by distance without slopes, sinks, a "
+                          "score cap and chunks")
+    return dist.data_ptr(), dist.shape[1]
+
+
 def _no_sinks_with_slopes(sinks, slopes, on_matrix_cores: bool) -> None:
     if sinks is not None and slopes is not None and on_matrix_cores:
         raise KernelError("attention: the matrix-core kernels take sinks or slopes, not both")
@@ -1184,7 +1291,7 @@ def attn_prefill(q: torch.Tensor, k_pages: torch.Tensor, v_pages: torch.Tensor,
                  slopes: torch.Tensor | None = None, rows_per_item: int | None = None,
                  keep_first: int = 0, gate: torch.Tensor | None = None,
                  sinks: torch.Tensor | None = None, score_cap: float | None = None,
-                 chunk: int = 0) -> None:
+                 chunk: int = 0, dist: torch.Tensor | None = None) -> None:
     """Causal attention of query runs over the paged cache.  ``work``: ``[num_work, 3]`` rows
     (sequence row, item, item or -1) where a sequence has ``query_len * H/KV`` rows per kv head,
     an item covers ``rows_per_item`` of them (what ``prefill_rows_per_item`` gave when the rows
@@ -1201,7 +1308,10 @@ def attn_prefill(q: torch.Tensor, k_pages: torch.Tensor, v_pages: torch.Tensor,
     ``score_cap``: the scaled score ``s`` becomes ``score_cap * tanh(s / score_cap)`` (the
     matrix-core kernels have it without sinks and slopes only).
     ``chunk``: positions are cut into chunks of so many, counted from position 0 of the sequence,
-    and a query sees only the keys of its own chunk (instead of a window, not beside one)."""
+    and a query sees only the keys of its own chunk (instead of a window, not beside one).
+    ``dist``: fp32 ``[H, distances]``; the scaled score of key ``j`` for a query at position ``p`` of head
+    ``h`` gets ``dist[h, min(p - j, distances - 1)]`` added (in the matrix-core kernels without slopes,
+    sinks, score cap and chunks beside it)."""
     H, KV, d = num_heads, num_kv_heads, head_dim
     window = _mask_arg(window, chunk)
     n_seqs = _attn_common(q, k_pages, v_pages, block_table, cu_q, ctx_lens, out, H, KV, d)
@@ -1215,16 +1325,18 @@ def attn_prefill(q: torch.Tensor, k_pages: torch.Tensor, v_pages: torch.Tensor,
     if rows_per_item is None:
         rows_per_item = prefill_rows_per_item(q.dtype, d, bs)
     _no_sinks_with_slopes(sinks, slopes, attention_on_matrix_cores(q.dtype, bs, d))
+    dp, nd = _dist_args(dist, H, q, slopes, sinks, cap, window, attention_on_matrix_cores(q.dtype, bs, d))
     if attention_on_matrix_cores(q.dtype, bs, d):
         if window < 0 and (sinks is not None or slopes is not None or cap > 0.0):
             raise KernelError("attn_prefill: the matrix-core kernel has chunks of positions with plain scores "
                               "only (no sinks, slopes or score cap beside them)")
         f = _fn("attn_mfma", "kvf_attn_mfma_prefill",
-                [c_void_p] * 7 + [c_int, c_int] + [c_void_p] + [c_int] * 11 + [c_float, c_void_p, c_void_p, c_int, c_void_p, c_float, c_void_p])
+                [c_void_p] * 7 + [c_int, c_int] + [c_void_p] + [c_int] * 11
+                + [c_float, c_void_p, c_void_p, c_int, c_void_p, c_float, c_void_p, c_int, c_void_p])
         _ok(f(q.data_ptr(), k_pages.data_ptr(), v_pages.data_ptr(), block_table.data_ptr(),
               cu_q.data_ptr(), ctx_lens.data_ptr(), work.data_ptr(), work.shape[0], int(rows_per_item), out.data_ptr(),
               H, KV, d, bs, nb, block_table.shape[1], q.stride(0), out.stride(0), int(window), keep,
-              n_seqs, float(scale), sl, gp, gs, sk, cap, _stream()), "attn_mfma_prefill")
+              n_seqs, float(scale), sl, gp, gs, sk, cap, dp, nd, _stream()), "attn_mfma_prefill")
         return
     if gate is not None:
         raise KernelError("attn_prefill: the 32-bit kernel takes no gate; gate its rows afterwards")
@@ -1235,11 +1347,11 @@ def attn_prefill(q: torch.Tensor, k_pages: torch.Tensor, v_pages: torch.Tensor,
         raise KernelError("attn_prefill: rows of q and out must start on 16 bytes")
     f = _fn("attn_generic", "kvf_attn_generic",
             [c_int] + [c_void_p] * 7 + [c_int] + [c_void_p] + [c_int] * 11
-            + [c_float, c_void_p, c_void_p, c_float, c_void_p])
+            + [c_float, c_void_p, c_void_p, c_float, c_void_p, c_int, c_void_p])
     _ok(f(_tcode(q.dtype), q.data_ptr(), k_pages.data_ptr(), v_pages.data_ptr(),
           block_table.data_ptr(), cu_q.data_ptr(), ctx_lens.data_ptr(), work.data_ptr(),
           work.shape[0], out.data_ptr(), H, KV, d, bs, nb, block_table.shape[1], q.stride(0),
-          out.stride(0), int(window), keep, n_seqs, float(scale), sl, sk, cap, _stream()), "attn_generic")
+          out.stride(0), int(window), keep, n_seqs, float(scale), sl, sk, cap, dp, nd, _stream()), "attn_generic")
 
 
 def attn_decode(q: torch.Tensor, k_pages: torch.Tensor, v_pages: torch.Tensor,
@@ -1250,7 +1362,7 @@ def attn_decode(q: torch.Tensor, k_pages: torch.Tensor, v_pages: torch.Tensor,
                 token_is_seq: bool = False, slopes: torch.Tensor | None = None,
                 keep_first: int = 0, gate: torch.Tensor | None = None,
                 sinks: torch.Tensor | None = None, score_cap: float | None = None,
-                chunk: int = 0) -> None:
+                chunk: int = 0, dist: torch.Tensor | None = None) -> None:
     """Attention of one-token queries: sequence rows ``seq_ids[:num_seqs]`` (or ``0..num_seqs-1``)
     each attend from their token ``cu_q[seq]`` over ``ctx_lens[seq]`` cached keys.  The key
     range may be cut into ``splits`` runs; ``workspace`` then holds fp32 partial accumulators
@@ -1259,8 +1371,8 @@ def attn_decode(q: torch.Tensor, k_pages: torch.Tensor, v_pages: torch.Tensor,
     single tokens), which spares the matrix-core kernel a dependent load.  ``slopes``: as in
     ``attn_prefill``; ``keep_first`` and ``gate`` likewise (the matrix-core kernels only: the
     32-bit path is given no gate, its caller gates the rows afterwards); ``sinks`` likewise (all
-    kernels; with cuts the term joins the sum where the cuts are merged); ``score_cap`` and
-    ``chunk`` likewise."""
+    kernels; with cuts the term joins the sum where the cuts are merged); ``score_cap``,
+    ``chunk`` and ``dist`` likewise."""
     H, KV, d = num_heads, num_kv_heads, head_dim
     window = _mask_arg(window, chunk)
     n_seqs = _attn_common(q, k_pages, v_pages, block_table, cu_q, ctx_lens, out, H, KV, d)
@@ -1290,27 +1402,29 @@ def attn_decode(q: torch.Tensor, k_pages: torch.Tensor, v_pages: torch.Tensor,
         if pa.numel() < num_seqs * H * splits * d or pm.numel() < num_seqs * H * splits * 2:
             raise KernelError("attn_decode: workspace too small")
     _no_sinks_with_slopes(sinks, slopes, attention_on_matrix_cores(q.dtype, bs, d))
+    dp, nd = _dist_args(dist, H, q, slopes, sinks, cap, window, attention_on_matrix_cores(q.dtype, bs, d))
     if not attention_on_matrix_cores(q.dtype, bs, d):
         if gate is not None:
             raise KernelError("attn_decode: the 32-bit kernel takes no gate; gate its rows afterwards")
         f = _fn("attn_generic", "kvf_attn_generic_decode",
-                [c_int] + [c_void_p] * 10 + [c_int] * 13 + [c_float, c_void_p, c_void_p, c_float, c_void_p])
+                [c_int] + [c_void_p] * 10 + [c_int] * 13 + [c_float, c_void_p, c_void_p, c_float, c_void_p, c_int, c_void_p])
         _ok(f(_tcode(q.dtype), q.data_ptr(), k_pages.data_ptr(), v_pages.data_ptr(),
               block_table.data_ptr(), seq_ids.data_ptr() if seq_ids is not None else None,
               None if token_is_seq else cu_q.data_ptr(), ctx_lens.data_ptr(), out.data_ptr(),
               pa.data_ptr() if pa is not None else None, pm.data_ptr() if pm is not None else None,
               num_seqs, H, KV, d, bs, nb, block_table.shape[1], q.stride(0), out.stride(0),
-              int(window), keep, n_seqs, int(splits), float(scale), sl, sk, cap, _stream()), "attn_generic_decode")
+              int(window), keep, n_seqs, int(splits), float(scale), sl, sk, cap, dp, nd, _stream()), "attn_generic_decode")
         return
     f = _fn("attn_mfma", "kvf_attn_mfma_decode",
-            [c_void_p] * 10 + [c_int] * 13 + [c_float, c_void_p, c_void_p, c_int, c_void_p, c_float, c_void_p])
+            [c_void_p] * 10 + [c_int] * 13
+            + [c_float, c_void_p, c_void_p, c_int, c_void_p, c_float, c_void_p, c_int, c_void_p])
     _ok(f(q.data_ptr(), k_pages.data_ptr(), v_pages.data_ptr(), block_table.data_ptr(),
           seq_ids.data_ptr() if seq_ids is not None else None,
           None if token_is_seq else cu_q.data_ptr(),
           ctx_lens.data_ptr(), out.data_ptr(), pa.data_ptr() if pa is not None else None,
           pm.data_ptr() if pm is not None else None, num_seqs, H, KV, d, bs, nb,
           block_table.shape[1], q.stride(0), out.stride(0), int(window), keep, n_seqs, int(splits),
-          float(scale), sl, gp, gs, sk, cap, _stream()), "attn_mfma_decode")
+          float(scale), sl, gp, gs, sk, cap, dp, nd, _stream()), "attn_mfma_decode")
 
 
 # ------------------------------------------------------------------------------ matrix-memory recurrence
@@ -1444,39 +1558,44 @@ def mlstm_out(heads_raw: torch.Tensor, gate: torch.Tensor, weight: torch.Tensor,
 
 
 # ------------------------------------------------------------------------------ latent attention
-def latent_split(proj: torch.Tensor, qkv: torch.Tensor, norm_weight: torch.Tensor | None, eps: float,
-                 heads: int, dim: int, rot: int, rank: int, head_dim: int) -> None:
-    """A projected row ``[heads x (dim | rot) | latent (rank) | shared key part (rot)]`` becomes
-    the attention kernels' row ``[heads + 2, head_dim]``: q head ``h`` gets its ``rot`` part in
+def latent_split(q: torch.Tensor, qkv: torch.Tensor, norm_weight: torch.Tensor | None, eps: float, heads: int, dim: int,
+                 rot: int, rank: int, head_dim: int, down: torch.Tensor | None = None) -> None:
+    """A token's projected rows ``q [heads x (dim | rot)]`` and ``down [latent (rank) | shared key part (rot)]`` (blocks
+    of columns of wider rows are fine; ``None``: the columns behind the q heads in ``q``'s own rows) become the attention kernels' row ``[heads + 2, head_dim]``: q head ``h`` gets its ``rot`` part in
     front (columns ``rot..rot+rank-1`` are left for ``head_product`` to fill, the rest is
     zero), the one k head is ``[key part | norm(latent) | 0]`` and the one v head
     ``[0 | norm(latent) | 0]``, the norm being ``x / sqrt(mean(x^2) + eps) * norm_weight`` in
-    fp32 with one rounding.  ``norm_weight=None``: the projected row holds q heads alone, and so
-    does the attention row, ``[heads, head_dim]`` (attention over another layer's keys)."""
-    n = proj.shape[0]
+    fp32 with one rounding.  ``norm_weight=None``: ``down`` is not read and the attention row holds q heads
+    alone, ``[heads, head_dim]`` (attention over another layer's keys)."""
+    n = q.shape[0]
     H, d = int(heads), int(head_dim)
     own = norm_weight is not None
-    _check(proj, "proj", None, (n, None), contiguous=False)
-    _check(qkv, "qkv", proj.dtype, (n, (H + (2 if own else 0)) * d))
+    if own and down is None:
+        down = q[:, H * (dim + rot):]
+    _check(q, "q", None, (n, None), contiguous=False)
+    _check(qkv, "qkv", q.dtype, (n, (H + (2 if own else 0)) * d))
     if own:
         _check(norm_weight, "norm_weight", F32, (rank,))
-    if proj.stride(1) != 1 or proj.shape[1] < H * (dim + rot) + (rank + rot if own else 0) or d < rot + rank:
-        raise KernelError(f"latent_split: rows of {proj.shape[1]} elements / heads of {d} do not hold "
-                          f"{H} x ({dim} + {rot}) + {rank} + {rot}")
-    f = _fn("latent", "kvf_latent_split", [c_int, c_void_p, c_int, c_void_p, c_int, c_void_p, c_float]
+        _check(down, "down", q.dtype, (n, None), contiguous=False)
+    if (q.stride(1) != 1 or q.shape[1] < H * (dim + rot) or d < rot + rank
+            or (own and (down.stride(1) != 1 or down.shape[1] < rank + rot))):
+        raise KernelError(f"latent_split: rows of {q.shape[1]} and {down.shape[1] if own else 0} elements / heads of {d} "
+                          f"do not hold {H} x ({dim} + {rot}) and {rank} + {rot}")
+    f = _fn("latent", "kvf_latent_split", [c_int, c_void_p, c_int, c_void_p, c_int, c_void_p, c_int, c_void_p, c_float]
             + [c_int] * 6 + [c_void_p])
-    _ok(f(_tcode(proj.dtype), proj.data_ptr(), proj.stride(0) if n > 1 else proj.shape[1], qkv.data_ptr(),
-          qkv.shape[1], norm_weight.data_ptr() if own else None, float(eps), n, H, int(dim), int(rot), int(rank), d,
+    _ok(f(_tcode(q.dtype), q.data_ptr(), q.stride(0) if n > 1 else q.shape[1], down.data_ptr() if own else None,
+          (down.stride(0) if n > 1 else down.shape[1]) if own else 0, qkv.data_ptr(), qkv.shape[1], norm_weight.data_ptr() if own else None, float(eps), n, H, int(dim), int(rot), int(rank), d,
           _stream()), "latent_split")
 
 
 def head_product(x: torch.Tensor, in_head: int, w: torch.Tensor, out: torch.Tensor, out_head: int,
-                 gate: torch.Tensor | None = None) -> None:
+                 gate: torch.Tensor | None = None, gate_outputs: bool = False, scale: float = 1.0) -> None:
     """``out[n, h * out_head + o] = sum_i w[h, o, i] * x[n, h * in_head + i]`` for per-head
     matrices ``w [H, O, I]``: ``x`` and ``out`` are rows (views of wider rows are fine) in which
     head ``h`` starts ``h * in_head`` / ``h * out_head`` elements in.  fp32 multiply and add.
     ``gate`` (``[n, >= H]``, dense rows of ``x``'s type): what is stored is the product times
-    ``sigmoid(gate[n, h])``."""
+    ``sigmoid(gate[n, h])``, or with ``gate_outputs`` (``[n, >= H * O]``) times ``sigmoid(gate[n, h * O + o])``;
+    and times ``scale``."""
     n = x.shape[0]
     _check(w, "w", None, (None, None, None))
     H, O, I = w.shape
@@ -1491,14 +1610,31 @@ def head_product(x: torch.Tensor, in_head: int, w: torch.Tensor, out: torch.Tens
         raise KernelError("head_product: out must not share memory with x")
     if gate is not None:
         _check(gate, "gate", x.dtype, (n, None), contiguous=False)
-        if gate.stride(1) != 1 or gate.shape[1] < H:
-            raise KernelError("head_product: a gate needs a number per head in dense rows")
+        if gate.stride(1) != 1 or gate.shape[1] < (H * O if gate_outputs else H):
+            raise KernelError("head_product: a gate needs a number per head (or output) in dense rows")
+    elif gate_outputs:
+        raise KernelError("head_product: gate_outputs without a gate")
     f = _fn("latent", "kvf_head_product", [c_int, c_int, c_void_p, c_int, c_int, c_void_p, c_void_p]
-            + [c_int] * 6 + [c_void_p, c_int, c_void_p])
+            + [c_int] * 6 + [c_void_p, c_int, c_int, c_float, c_void_p])
     _ok(f(_tcode(x.dtype), _tcode(w.dtype), x.data_ptr(), x.stride(0) if n > 1 else x.shape[1], int(in_head),
           w.data_ptr(), out.data_ptr(), out.stride(0) if n > 1 else out.shape[1], int(out_head), n, H, O, I,
           gate.data_ptr() if gate is not None else None,
-          (gate.stride(0) if n > 1 else gate.shape[1]) if gate is not None else 0, _stream()), "head_product")
+          (gate.stride(0) if n > 1 else gate.shape[1]) if gate is not None else 0, 1 if gate_outputs else 0,
+          float(scale), _stream()), "head_product")
+
+
+def latent_norm(x: torch.Tensor, weight: torch.Tensor, eps: float, out: torch.Tensor) -> None:
+    """``out[n] = x[n] / sqrt(mean(x[n]^2) + eps) * weight`` in fp32 with one rounding, for dense rows ``x`` that may be
+    a block of columns of wider ones; ``out`` contiguous, of ``x``'s type."""
+    n, rank = out.shape
+    _check(x, "x", out.dtype, (n, rank), contiguous=False)
+    _check(out, "out")
+    _check(weight, "weight", F32, (rank,))
+    if x.stride(1) != 1 or _overlap(x, out):
+        raise KernelError("latent_norm: dense rows, and an output of its own")
+    f = _fn("latent", "kvf_latent_norm", [c_int, c_void_p, c_int, c_void_p, c_float, c_void_p, c_int, c_int, c_void_p])
+    _ok(f(_tcode(out.dtype), x.data_ptr(), x.stride(0) if n > 1 else rank, weight.data_ptr(), float(eps), out.data_ptr(),
+          n, rank, _stream()), "latent_norm")
 
 
 # ------------------------------------------------------------------------------ decaying matrix memory
@@ -1646,16 +1782,26 @@ MOE_MAX_ROUTER_OUTPUTS = 512
 MOE_MAX_TOP = 16
 
 
-MOE_SCORES = {"softmax": 0, "sigmoid": 1}
+MOE_SCORES = {"softmax": 0, "sigmoid": 1, "chosen": 2}
+MOE_FORMS = ("silu", "limited")      # how an expert joins its (gate, up) pairs (see ``GATE_FORMS``)
+
+
+def _moe_form(form: str, limit: float | None, who: str) -> tuple[int, float]:
+    if form not in MOE_FORMS:
+        raise KernelError(f"{who}: experts join their pairs by one of {MOE_FORMS}, got {form!r}")
+    return _gate_form(form, limit, who)
 
 
 def moe_topk(logits: torch.Tensor, correction: torch.Tensor | None, chosen: torch.Tensor,
-             weights: torch.Tensor, scores: str = "softmax", renormalize: bool = True) -> None:
+             weights: torch.Tensor, scores: str = "softmax", renormalize: bool = True,
+             bias: torch.Tensor | None = None, scale: float = 1.0) -> None:
     """The router's choice per token from its fp32 ``logits [N, R]``: ``s = softmax(logits)`` or, with
     ``scores="sigmoid"``, ``s = sigmoid(logits)`` of every output by itself; the ``top`` outputs with
     the largest ``s + correction`` (``None``: ``s`` alone; the lowest index among equals) go to
     ``chosen [N, top]`` (int32) and their ``s``, with ``renormalize`` divided by the sum of the chosen
-    ``s`` (+ 1e-20), to ``weights [N, top]`` (fp32)."""
+    ``s`` (+ 1e-20), to ``weights [N, top]`` (fp32).  ``scores="chosen"``: the outputs with the largest
+    logits are chosen and weighted by the softmax over the chosen logits alone (no correction).
+    ``bias`` (fp32 ``[R]``) is added to the logits first; the weights are multiplied by ``scale`` last."""
     if scores not in MOE_SCORES:
         raise KernelError(f"moe_topk: unknown scores {scores!r}; known: {sorted(MOE_SCORES)}")
     n, R = logits.shape
@@ -1664,32 +1810,38 @@ def moe_topk(logits: torch.Tensor, correction: torch.Tensor | None, chosen: torc
         raise KernelError("moe_topk: logits rows must be dense")
     if correction is not None:
         _check(correction, "correction", F32, (R,))
+        if scores == "chosen":
+            raise KernelError("moe_topk: no correction beside weights that are a softmax over the chosen logits")
+    if bias is not None:
+        _check(bias, "bias", F32, (R,))
     top = chosen.shape[1]
     _check(chosen, "chosen", I32, (n, top))
     _check(weights, "weights", F32, (n, top))
     if R > MOE_MAX_ROUTER_OUTPUTS or not 0 < top <= min(MOE_MAX_TOP, R):
         raise KernelError(f"moe_topk: up to {MOE_MAX_ROUTER_OUTPUTS} router outputs and {MOE_MAX_TOP} choices, got {R} / {top}")
-    f = _fn("moe", "kvf_moe_topk", [c_void_p, c_int, c_void_p, c_void_p, c_void_p] + [c_int] * 5 + [c_void_p])
-    _ok(f(logits.data_ptr(), logits.stride(0) if n > 1 else R,
+    f = _fn("moe", "kvf_moe_topk", [c_void_p, c_int] + [c_void_p] * 4 + [c_int] * 5 + [c_float, c_void_p])
+    _ok(f(logits.data_ptr(), logits.stride(0) if n > 1 else R, bias.data_ptr() if bias is not None else None,
           correction.data_ptr() if correction is not None else None, chosen.data_ptr(), weights.data_ptr(), n, R, top,
-          MOE_SCORES[scores], 1 if renormalize else 0, _stream()), "moe_topk")
+          MOE_SCORES[scores], 1 if renormalize else 0, float(scale), _stream()), "moe_topk")
 
 
 def moe_dense_act(gate_up: torch.Tensor, chosen: torch.Tensor, weights: torch.Tensor, out: torch.Tensor,
-                  experts: int, ff: int, weigh_input: bool = False) -> None:
+                  experts: int, ff: int, weigh_input: bool = False, form: str = "silu",
+                  limit: float | None = None) -> None:
     """``gate_up [N, 2 experts ff]`` holds every expert's (gate, up) pairs as neighbouring columns;
     ``out[n, e ff + j] = weight(n, e) * silu(gate) * up`` where token ``n`` chose expert ``e`` and an
     exact zero elsewhere.  ``weigh_input``: ``silu(w gate) * (w up)`` with ``w = weight(n, e)`` instead
-    (the weight belongs to the expert's input)."""
+    (the weight belongs to the expert's input).  ``form``, ``limit``: how a pair is joined (``MOE_FORMS``)."""
+    code, lim = _moe_form(form, limit, "moe_dense_act")
     n = gate_up.shape[0]
     E, top = int(experts), chosen.shape[1]
     _check(gate_up, "gate_up", None, (n, 2 * E * ff))
     _check(out, "out", gate_up.dtype, (n, E * ff))
     _check(chosen, "chosen", I32, (n, top))
     _check(weights, "weights", F32, (n, top))
-    f = _fn("moe", "kvf_moe_dense_act", [c_int] + [c_void_p] * 4 + [c_int] * 5 + [c_void_p])
+    f = _fn("moe", "kvf_moe_dense_act", [c_int] + [c_void_p] * 4 + [c_int] * 6 + [c_float, c_void_p])
     _ok(f(_tcode(gate_up.dtype), gate_up.data_ptr(), chosen.data_ptr(), weights.data_ptr(), out.data_ptr(),
-          n, E, int(ff), top, 1 if weigh_input else 0, _stream()), "moe_dense_act")
+          n, E, int(ff), top, 1 if weigh_input else 0, code, lim, _stream()), "moe_dense_act")
 
 
 def moe_identity(x: torch.Tensor, h: torch.Tensor, chosen: torch.Tensor, weights: torch.Tensor,
@@ -1723,7 +1875,8 @@ def moe_grouped_tiles(rows: int, top: int, experts: int) -> int:
 
 def moe_grouped(x: torch.Tensor, w_gate_up: "StreamedWeight", w_down: "StreamedWeight", chosen: torch.Tensor,
                 weights: torch.Tensor, residual: torch.Tensor, experts: int, ff: int,
-                scratch: dict[str, torch.Tensor], weigh_input: bool = False, fresh: bool = False) -> None:
+                scratch: dict[str, torch.Tensor], weigh_input: bool = False, fresh: bool = False,
+                form: str = "silu", limit: float | None = None) -> None:
     """``residual[n] += sum_k weights[n, k] * expert_{chosen[n, k]}(x[n])`` (a choice ``>= experts``
     stands for ``x[n]`` itself) with every expert's products taken over only the rows that chose
     it: the pairs are grouped by expert on the device, tiles of 16 rows go through the
@@ -1733,7 +1886,9 @@ def moe_grouped(x: torch.Tensor, w_gate_up: "StreamedWeight", w_down: "StreamedW
     ``scratch``: ``where order [n top]``, ``tiles [3 moe_grouped_tiles]``, ``num_tiles [1]`` (int32),
     ``act [n top, ff]``, ``y [n top, K]`` (bf16).  ``weigh_input``: every chosen expert reads its
     weight times the row, ``expert(weights[n, k] * x[n])``, and the outputs are summed as they are.
-    ``fresh``: ``residual`` is written instead of added to."""
+    ``fresh``: ``residual`` is written instead of added to.  ``form``, ``limit``: how an expert joins its
+    pairs (``MOE_FORMS``)."""
+    code, lim = _moe_form(form, limit, "moe_grouped")
     n, k = x.shape
     top = chosen.shape[1]
     if not moe_grouped_takes(x, w_gate_up, w_down, experts, ff):
@@ -1749,12 +1904,12 @@ def moe_grouped(x: torch.Tensor, w_gate_up: "StreamedWeight", w_down: "StreamedW
                                ("num_tiles", I32, (1,)), ("act", BF16, (pairs, ff)), ("y", BF16, (pairs, k))):
         _check(scratch[name], name, dtype, shape)
     f = _fn("moe", "kvf_moe_grouped", [c_void_p, c_int, c_void_p] + [c_int] * 5 + [c_void_p] * 8 + [c_int]
-            + [c_void_p] * 3 + [c_int, c_int, c_void_p])
+            + [c_void_p] * 3 + [c_int, c_int, c_int, c_float, c_void_p])
     _ok(f(x.data_ptr(), x.stride(0) if n > 1 else k, x.data_ptr(), n, k, int(experts), int(ff), top,
           w_gate_up.tiles.data_ptr(), w_down.tiles.data_ptr(), chosen.data_ptr(), weights.data_ptr(),
           scratch["where"].data_ptr(), scratch["order"].data_ptr(), scratch["tiles"].data_ptr(),
           scratch["num_tiles"].data_ptr(), max_tiles, scratch["act"].data_ptr(), scratch["y"].data_ptr(),
-          residual.data_ptr(), 1 if weigh_input else 0, 1 if fresh else 0, _stream()), "moe_grouped")
+          residual.data_ptr(), 1 if weigh_input else 0, 1 if fresh else 0, code, lim, _stream()), "moe_grouped")
 
 
 
@@ -1884,25 +2039,26 @@ def linmem_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, decay: torch.
 
 
 def linmem_out(heads_raw: torch.Tensor, gate: torch.Tensor, weight: torch.Tensor | None, eps: float,
-               out: torch.Tensor, heads: int, value_dim: int, scale: float = 1.0) -> None:
+               out: torch.Tensor, heads: int, value_dim: int, scale: float = 1.0, sigmoid: bool = False) -> None:
     """``out[n, h, :] = o / rms(o) * weight * silu(gate[n, h, :]) * scale`` for the raw heads
     ``o = heads_raw[n, h, :]`` (fp32), the root mean square per head with ``eps`` inside the
     root; ``weight`` fp32 ``[value_dim]`` shared by the heads, or ``None`` for none.  ``gate``:
-    dense rows of ``out``'s type (a view of wider rows is fine)."""
+    dense rows of ``out``'s type (a view of wider rows is fine).  ``sigmoid``: the gate is ``sigmoid(gate)``,
+    from fp32 rows."""
     n = heads_raw.shape[0]
     H, dv = int(heads), int(value_dim)
     _check(heads_raw, "heads_raw", F32, (n, H * dv))
     if weight is not None:
         _check(weight, "weight", F32, (dv,))
     _check(out, "out", None, (n, H * dv))
-    _check(gate, "gate", out.dtype, (n, H * dv), contiguous=False)
+    _check(gate, "gate", F32 if sigmoid else out.dtype, (n, H * dv), contiguous=False)
     if gate.stride(1) != 1:
         raise KernelError("linmem_out: gate rows must be dense")
     f = _fn("linmem", "kvf_linmem_out", [c_int, c_void_p, c_void_p, c_int, c_void_p, c_float, c_float, c_void_p]
-            + [c_int] * 3 + [c_void_p])
+            + [c_int] * 5 + [c_void_p])
     _ok(f(_tcode(out.dtype), heads_raw.data_ptr(), gate.data_ptr(), gate.stride(0) if n > 1 else H * dv,
           weight.data_ptr() if weight is not None else None, float(eps), float(scale), out.data_ptr(), n, H, dv,
-          _stream()), "linmem_out")
+          1 if gate.dtype == F32 else 0, 1 if sigmoid else 0, _stream()), "linmem_out")
 
 
 # ------------------------------------------------------------------------------ state-space memories
@@ -1952,6 +2108,14 @@ def ssm_scratch(n_tokens: int, n_chunks: int, heads: int, key_dim: int, value_di
     return out
 
 
+def _slots(state: torch.Tensor, who: str) -> tuple[int, int]:
+    """(slots, floats from one slot to the next) of state slots, which may be a block of columns of wider ones."""
+    _check(state, "state", F32, (None, None), contiguous=False)
+    if state.stride(1) != 1 or (state.shape[0] > 1 and state.stride(0) < state.shape[1]):
+        raise KernelError(f"{who}: slots are dense rows")
+    return state.shape[0], state.stride(0) if state.shape[0] > 1 else state.shape[1]
+
+
 def ssm_conv(rows: torch.Tensor, col0: int, weight: torch.Tensor, bias: torch.Tensor | None, cu_q: torch.Tensor,
              positions: torch.Tensor, slot_ids: torch.Tensor, state: torch.Tensor, state_off: int, out: torch.Tensor,
              n_seqs: int, longest: int, unit: int = 0, key_dim: int = 0, q_scale: float = 1.0) -> None:
@@ -1974,7 +2138,7 @@ def ssm_conv(rows: torch.Tensor, col0: int, weight: torch.Tensor, bias: torch.Te
         _check(bias, "bias", F32, (C,))
     if unit and (not 0 < key_dim <= 256 or unit % (2 * key_dim) or unit > C):
         raise KernelError(f"ssm_conv: {unit} channels are not q and k heads of {key_dim} elements (at most 256)")
-    _check(state, "state", F32, (None, None))
+    slots = _slots(state, "ssm_conv")
     if state_off < 0 or state_off + (taps - 1) * C > state.shape[1]:
         raise KernelError(f"ssm_conv: slots of {state.shape[1]} floats do not hold {taps - 1} x {C} inputs from {state_off} on")
     for t, name in ((cu_q, "cu_q"), (positions, "positions"), (slot_ids, "slot_ids")):
@@ -1986,7 +2150,7 @@ def ssm_conv(rows: torch.Tensor, col0: int, weight: torch.Tensor, bias: torch.Te
             + [c_void_p] * 4 + [c_int] * 3 + [c_void_p] + [c_int] * 2 + [c_void_p])
     _ok(f(_tcode(rows.dtype), rows.data_ptr(), rows.stride(0) if n > 1 else rows.shape[1], int(col0), C, taps,
           weight.data_ptr(), bias.data_ptr() if bias is not None else None, int(unit), int(key_dim), float(q_scale),
-          cu_q.data_ptr(), positions.data_ptr(), slot_ids.data_ptr(), state.data_ptr(), state.shape[0], state.shape[1],
+          cu_q.data_ptr(), positions.data_ptr(), slot_ids.data_ptr(), state.data_ptr(), *slots,
           int(state_off), out.data_ptr(), int(n_seqs), int(longest), _stream()), "ssm_conv")
 
 
@@ -2053,6 +2217,55 @@ def ssm_scan(rows: torch.Tensor, q_off: int, k_off: int, v_off: int, gates: torc
     f = _fn("ssm", "kvf_ssm_chunks", types + [c_void_p, c_int, c_void_p, c_int] + [c_void_p] * 6)
     _ok(f(*common, chunks.data_ptr(), nc, runs.data_ptr(), runs.shape[0],
           *(multi[k].data_ptr() if k in multi else None for k in ("T", "B", "W", "U", "E")), _stream()), "ssm_chunks")
+
+
+# ------------------------------------------------------------------------------ delta rule, a decay per key channel
+CHDELTA_CHUNK_FROM = 24
+
+
+def chdelta_scan(rows: torch.Tensor, q_off: int, k_off: int, v_off: int, decay: torch.Tensor, a_off: int,
+                 steps: torch.Tensor, b_off: int, neg_a: torch.Tensor, dt_bias: torch.Tensor, cu_q: torch.Tensor,
+                 positions: torch.Tensor, slot_ids: torch.Tensor, state: torch.Tensor, out: torch.Tensor, n_seqs: int,
+                 heads: int, key_heads: int, key_dim: int, value_dim: int, multi: dict | None = None,
+                 short_runs: bool = True) -> None:
+    """A matrix memory per head under the delta rule with a decay per head and key channel, over every
+    query run, in fp32, from and to the sequences' state slots (as ``ssm_scan`` keeps them; ``state`` may be
+    a block of columns of wider slots).  ``rows`` as in ``ssm_scan``.  ``decay`` fp32 ``[n, >= a_off + heads *
+    key_dim]``: ``a = exp(neg_a[h] * softplus(decay[a_off + h * key_dim + i] + dt_bias[h * key_dim + i]))`` multiplies key row
+    ``i``; ``steps`` fp32: ``beta = sigmoid(steps[b_off + h])``.  ``S <- diag(a) S``, ``S <- S + k (beta (v - S^T k))^T``,
+    ``o = S^T q``."""
+    n = rows.shape[0]
+    H, G, dk, dv = int(heads), int(key_heads), int(key_dim), int(value_dim)
+    _check(rows, "rows", F32, (n, None), contiguous=False)
+    if rows.stride(1) != 1 or G <= 0 or H % G or not 0 < dk <= 256 or dv <= 0:
+        raise KernelError(f"chdelta_scan: dense rows, {H} heads over {G} key heads of {dk} (at most 256) x {dv}")
+    for off, size, name in ((q_off, G * dk, "q"), (k_off, G * dk, "k"), (v_off, H * dv, "v")):
+        if off < 0 or off + size > rows.shape[1]:
+            raise KernelError(f"chdelta_scan: {name} at columns {off}..{off + size} lies outside rows of {rows.shape[1]}")
+    for t, off, size, name in ((decay, a_off, H * dk, "decay"), (steps, b_off, H, "steps")):
+        _check(t, name, F32, (n, None), contiguous=False)
+        if t.stride(1) != 1 or not 0 <= off <= t.shape[1] - size:
+            raise KernelError(f"chdelta_scan: {name} rows too short or not dense")
+    _check(neg_a, "neg_a", F32, (H,))
+    _check(dt_bias, "dt_bias", F32, (H * dk,))
+    _check(out, "out", F32, (n, H * dv))
+    slots = _slots(state, "chdelta_scan")
+    if state.shape[1] < H * dk * dv:
+        raise KernelError(f"chdelta_scan: heads of {dk} x {dv} need slots of {H * dk * dv} floats")
+    for t, name in ((cu_q, "cu_q"), (positions, "positions"), (slot_ids, "slot_ids")):
+        _check(t, name, I32, (None,))
+    if cu_q.shape[0] < n_seqs + 1 or slot_ids.shape[0] < n_seqs or positions.shape[0] < n:
+        raise KernelError("chdelta_scan: batch arrays shorter than the batch")
+    ld = lambda t: t.stride(0) if n > 1 else t.shape[1]  # noqa: E731
+    common = (rows.data_ptr(), ld(rows), int(q_off), int(k_off), int(v_off), decay.data_ptr(), ld(decay), int(a_off),
+              steps.data_ptr(), ld(steps), int(b_off), neg_a.data_ptr(), dt_bias.data_ptr(), positions.data_ptr(),
+              slot_ids.data_ptr(), state.data_ptr(), *slots, out.data_ptr(), H, G, dk, dv)
+    types = ([c_void_p] + [c_int] * 4 + [c_void_p] + [c_int] * 2 + [c_void_p] + [c_int] * 2 + [c_void_p] * 5
+             + [c_int] * 2 + [c_void_p] + [c_int] * 4)
+    if short_runs or multi is None:
+        f = _fn("chdelta", "kvf_chdelta_scan", types + [c_void_p, c_int, c_int, c_void_p])
+        _ok(f(*common, cu_q.data_ptr(), int(n_seqs), CHDELTA_CHUNK_FROM if multi is not None else 0, _stream()),
+            "chdelta_scan")
 
 
 def ssm_gate_norm(y: torch.Tensor, gate: torch.Tensor, weight: torch.Tensor, eps: float, parts: int,

@@ -9,6 +9,7 @@ import torch
 from kvforge_amd import registry
 from kvforge_amd.cache.manager import CacheGroup
 from kvforge_amd.kernels import library
+from kvforge_amd.parts.block import norm_rows
 from kvforge_amd.parts.base import Block, CacheSpec, LayerState, ModelSpec, StateSpec
 from kvforge_amd.weights.loader import load_model_weights
 
@@ -186,11 +187,11 @@ class Transformer:
             raise ValueError("the greedy tail is for steps of single tokens that all want their "
                              "logits, on a model that can_pick")
         if r == 0:
-            step.owed = None
+            step.owed = step.owed_bias = None
             return torch.empty((0, cfg.vocab_size), dtype=torch.float32, device=residual.device)
         x = step.ws.buf("final_normed", (r, hidden), step.act_dtype)
         # only the wanted rows matter now: what is still owed to the stream is added to them alone
-        spec.final_norm.forward(residual, x, step.logits_rows, add=step.take_owed(residual))
+        norm_rows(spec.final_norm, residual, x, step, step.logits_rows)
         if tail is not None:
             spec.head.pick(x, residual, step, tail)
             return None

@@ -12,7 +12,7 @@ from kvforge_amd.parts.latent import LatentAttention
 from kvforge_amd.parts.wkv import DecayMemory
 from kvforge_amd.parts.linmem import LinearMemory
 from kvforge_amd.parts.pair import MixerPair
-from kvforge_amd.parts.ssm import ConvMemory, GatedDelta, Mamba2
+from kvforge_amd.parts.ssm import ChannelDelta, ConvMemory, GatedDelta, Mamba2
 from kvforge_amd.parts.embedding import LMHead, TokenEmbedding
 from kvforge_amd.parts.block import ParallelBlock, PostNormBlock, PreNormBlock, SandwichBlock
 
@@ -22,4 +22,4 @@ __all__ = ["BLOCK", "PageTensor", "attention_pages", "Block", "CacheSpec", "Embe
            "PreNormBlock", "ParallelBlock", "ScalarRMSNorm", "LearnedPositions", "GatedFeedForward",
            "TokenSideInput", "OnePlusRMSNorm", "YarnStretch", "MatrixLSTM", "RoutedExperts",
            "NamedRMSNorm", "LatentAttention", "DecayMemory", "SandwichBlock", "LinearMemory", "MixerPair",
-           "PlainFeedForward", "ConvMemory", "GatedDelta", "Mamba2", "PostNormBlock"]
+           "PlainFeedForward", "ConvMemory", "GatedDelta", "ChannelDelta", "Mamba2", "PostNormBlock"]

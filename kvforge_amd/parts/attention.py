@@ -13,7 +13,7 @@ import math
 import torch
 
 from kvforge_amd.kernels import ops
-from kvforge_amd.parts.base import (CacheSpec, LayerState, Mixer, WeightSpec, add_product,
+from kvforge_amd.parts.base import (CacheSpec, LayerState, Mixer, StateSpec, WeightSpec, add_product,
                                     attention_pages)
 from kvforge_amd.parts.positions import RotaryPositions
 from kvforge_amd.registry import register_mixer
@@ -71,6 +71,28 @@ def prefill_work_rows(q_lens, prefill_seqs, group_size: int, rows_per_item: int,
     return [(b, i, -1) for _, b, i in rows]
 
 
+def distance_bucket(n: int, buckets: int, far: float) -> int:
+    """The bucket of a distance ``n >= 0``: with ``half = buckets // 2``, ``n`` itself below ``half``, then ``half +
+    floor(ln(n / half) / ln(far / half) * (buckets - half))``, at most ``buckets - 1``."""
+    half = buckets // 2
+    if n < half or buckets == 1:
+        return min(n, buckets - 1)
+    return min(buckets - 1, half + math.floor(math.log(n / half) / math.log(far / half) * (buckets - half)))
+
+
+def distance_table(table: torch.Tensor, far: float) -> torch.Tensor:
+    """``table [buckets, heads]`` by distance instead of by bucket: fp32 ``[heads, distances]``, whose last column
+    stands for every distance from there on (the first that falls into the last bucket)."""
+    buckets = int(table.shape[0])
+    if not far > max(buckets // 2, 1) or buckets < 2:
+        raise ValueError(f"a bias over {buckets} distance buckets (at least 2) needs a far distance beyond "
+                         f"{buckets // 2}, got {far}")
+    rows = [0]
+    while rows[-1] != buckets - 1:
+        rows.append(distance_bucket(len(rows), buckets, far))
+    return table.float()[torch.tensor(rows, device=table.device)].t().contiguous()
+
+
 @register_mixer("attention")
 class PagedAttention(Mixer):
     """``window``: ``None`` attends to every earlier position, ``w`` to the last ``w``.
@@ -119,7 +141,17 @@ class PagedAttention(Mixer):
     multiplied by ``sigmoid(W x)_h``, one number per head, from the same input as the
     projections; a product of its own with fp32 sums stored in fp32.
     ``out_scale``: a constant on the heads' outputs, applied in fp32 ahead of the (linear) output
-    projection."""
+    projection.
+    ``conv``: ``(taps, name)``; every channel of q, k and v passes a causal convolution over the last
+    ``taps`` tokens as it leaves the projection, ``y_t = sum_j w[:, j] x_(t - taps + 1 + j)`` with zeros before the
+    sequence's start; ``name`` is a format with ``{of}``, the name of the projection, of a tensor ``[channels,
+    taps]``.  The last ``taps - 1`` projected rows of a request are its state.  Convolution, norm of q and k
+    and cache write are one kernel (so there is no rotation, gate in the product or ``row_norm`` beside it).
+    Then ``qk_norm`` may be ``(None, None, eps)``, a norm without weights.
+    ``distance_bias``: ``(name, far)``; the scaled score of key ``j`` for a query at position ``p`` of head ``h`` gets
+    ``table[bucket(p - j), h]`` added, ``table`` being the tensor ``name`` of ``B`` rows (the checkpoint's number, or
+    ``distance_buckets``): with ``half = B / 2``, distances below ``half`` have buckets of their own, the others share
+    the rest by their logarithm up to the distance ``far`` (``distance_bucket``)."""
 
     NAMES = {"q": "q_proj.weight", "k": "k_proj.weight", "v": "v_proj.weight", "o": "o_proj.weight",
              "g": "g_proj.weight"}
@@ -136,7 +168,8 @@ class PagedAttention(Mixer):
                  score_cap: float | None = None, q_temp: tuple[float, int] | None = None,
                  row_norm: tuple[str, str, float] | None = None, bias: tuple[str, str] | None = None,
                  values_are_keys: bool = False, chunk: int | None = None, head_gate: str | None = None,
-                 out_scale: float = 1.0) -> None:
+                 out_scale: float = 1.0, conv: tuple[int, str] | None = None,
+                 distance_bias: tuple[str, float] | None = None, distance_buckets: int | None = None) -> None:
         if num_heads % num_kv_heads:
             raise ValueError("num_heads must be a multiple of num_kv_heads")
         self.dk = int(head_dim)
@@ -186,6 +219,23 @@ class PagedAttention(Mixer):
                              "neighbouring pairs, or none)")
         self.head_gate, self.out_scale = head_gate, float(out_scale)
         self.q_bias = self.k_bias = self.w_head_gate = None
+        self.conv = (int(conv[0]), conv[1]) if conv is not None else None
+        self.conv_w: torch.Tensor | None = None
+        if self.conv is not None:
+            taps = self.conv[0]
+            if not 1 <= taps <= ops.CONVKV_MAX_TAPS:
+                raise ValueError(f"convolutions of 1 to {ops.CONVKV_MAX_TAPS} taps, got {taps}")
+            if rotary is not None or gated or row_norm is not None or not own_kv or self.q_temp is not None:
+                raise ValueError("a convolution of q, k and v goes without rotation, element-wise gate, row_norm and "
+                                 "q_temp, with key and value projections of the mixer's own")
+            if taps > 1:
+                self.state_spec = StateSpec((ops.convkv_state_floats(self.H, self.KV, self.d, taps),), torch.float32)
+        elif qk_norm is not None and (qk_norm[0] is None or qk_norm[1] is None):
+            raise ValueError("a norm of q and k without weights goes with a convolution")
+        self.distance_bias, self.distance_buckets = distance_bias, distance_buckets
+        self.dist: torch.Tensor | None = None
+        if distance_bias is not None and (score_slopes is not None or sink is not None or self.score_cap or self.chunk):
+            raise ValueError("biases by distance go without slopes, sink, score cap and chunks")
         # a chunk's keys all lie within the last `chunk` positions
         self.cache_spec = CacheSpec(attention_pages(self.KV, self.d), self.window or self.chunk, self.keep_first)
         self.w_qkv: torch.Tensor | None = None
@@ -201,7 +251,12 @@ class PagedAttention(Mixer):
                   "g": (H * self.dv, h)}
         out = {self._name(self.names[n]): WeightSpec(shapes[n]) for n in self._matrices()}
         out[self._name(self.names["o"])] = WeightSpec((h, H * self.dv))
-        if self.qk_norm is not None:
+        if self.conv is not None:
+            for key, rows in (("q", H * self.dk), ("k", KV * self.dk), ("v", KV * self.dv)):
+                out[self._conv_name(key)] = WeightSpec((rows, self.conv[0]), std=0.3)
+        if self.distance_bias is not None:
+            out[self._name(self.distance_bias[0])] = WeightSpec((self.distance_buckets, H), std=0.5)
+        if self.qk_norm is not None and self.qk_norm[0] is not None:
             out[self._name(self.qk_norm[0])] = WeightSpec((self.dk,), init="norm", std=0.1)
             out[self._name(self.qk_norm[1])] = WeightSpec((self.dk,), init="norm", std=0.1)
         if self.sink is not None:
@@ -215,6 +270,9 @@ class PagedAttention(Mixer):
         if self.head_gate is not None:
             out[self._name(self.head_gate)] = WeightSpec((H, h))
         return out
+
+    def _conv_name(self, key: str) -> str:
+        return self._name(self.conv[1].format(of=self.names[key]))
 
     def _padded_heads(self, w: torch.Tensor, heads: int, size: int, perm=None) -> torch.Tensor:
         """Rows of ``heads`` heads of ``size`` rows each, every head padded with zero rows up to
@@ -252,7 +310,15 @@ class PagedAttention(Mixer):
             w_o = w_o.reshape(self.hidden, self.H * self.d).contiguous()
         self.w_o = w_o
         self.norm_eps = None
-        if self.qk_norm is not None:
+        if self.conv is not None:
+            self.conv_w = torch.cat([
+                self._padded_heads(tensors[self._conv_name(key)].float(), heads, size)
+                for key, heads, size in (("q", self.H, self.dk), ("k", self.KV, self.dk), ("v", self.KV, self.dv))],
+                dim=0).contiguous()
+        if self.distance_bias is not None:
+            name, far = self._name(self.distance_bias[0]), self.distance_bias[1]
+            self.dist = distance_table(tensors[name], float(far))
+        if self.qk_norm is not None and self.qk_norm[0] is not None:
             self.q_norm_w = tensors[self._name(self.qk_norm[0])].float().contiguous()
             self.k_norm_w = tensors[self._name(self.qk_norm[1])].float().contiguous()
         if self.sink is not None:
@@ -298,7 +364,8 @@ class PagedAttention(Mixer):
     def _plain(self) -> bool:
         """Whether the product holds q, k and v and nothing else, and nothing but the rotation
         lies between it and the cache."""
-        return self.own_kv and not self.gated and self.qk_norm is None and self.row_norm is None
+        return (self.own_kv and not self.gated and self.qk_norm is None and self.row_norm is None
+                and self.conv is None)
 
     def absorb_norm(self, norm) -> bool:
         if self._hooked() or not self._plain() or self.head_gate is not None:
@@ -311,6 +378,8 @@ class PagedAttention(Mixer):
 
     def kernel_modules(self, dtype: torch.dtype) -> set[str]:
         mods = {"elementwise", "gemm_generic", "attn_generic"}
+        if self.conv is not None:
+            mods.add("convkv")
         if dtype == torch.bfloat16:
             mods |= {"gemm_bf16", "attn_mfma"}
         return mods
@@ -321,13 +390,13 @@ class PagedAttention(Mixer):
 
     def _small(self) -> list[torch.Tensor]:
         gate = ops.plain_of(self.w_head_gate) if self.w_head_gate is not None else None
-        return [t for t in (self.q_norm_w, self.k_norm_w, self.sinks, self.q_bias, self.k_bias, gate)
+        return [t for t in (self.q_norm_w, self.k_norm_w, self.sinks, self.q_bias, self.k_bias, gate, self.dist)
                 if t is not None]
 
     def held_tensors(self) -> list[torch.Tensor]:
         gate = ops.copies_of(self.w_head_gate) if self.w_head_gate is not None else []
         return (ops.copies_of(self.w_qkv) + ops.copies_of(self.w_o) + gate
-                + [t for t in self._small() if t.dim() == 1])
+                + [t for t in self._small() if t.dim() == 1] + [t for t in (self.conv_w, self.dist) if t is not None])
 
     def seal(self) -> None:
         self.w_qkv, self.w_o = ops.streamed(ops.plain_of(self.w_qkv)), ops.streamed(ops.plain_of(self.w_o))
@@ -405,7 +474,7 @@ class PagedAttention(Mixer):
             normed = ws.buf("normed", (n, self.hidden), act)
             ops.rmsnorm(x, None, rms, normed, add=step.take_owed(residual))
             x, rms = normed, None
-        fused = (not self._hooked() and self.qk_norm is None and self.row_norm is None
+        fused = (not self._hooked() and self.qk_norm is None and self.row_norm is None and self.conv is None
                  and ops.bf16_kernel_takes(x, self.w_qkv, rms is not None, True)
                  and layer.k_pages.dtype == torch.bfloat16)
         if fused and rms is not None:
@@ -426,6 +495,17 @@ class PagedAttention(Mixer):
                               layer.k_pages, layer.v_pages, H, KV if self.own_kv else 0, d,
                               write_kv=layer.owns_cache and self.own_kv, rms_eps=rms, a_owed=owed,
                               extra_cols=extra)
+        elif self.conv is not None:
+            if layer.state is None and self.conv[0] > 1:
+                raise RuntimeError("attention behind a convolution needs a state slot per request")
+            rows = ws.buf("conv_rows", (n, self.w_qkv.shape[0]), act)
+            ops.gemm(x, self.w_qkv, rows)
+            qkv = ws.buf("conv_q", (n, H * d), act)
+            ops.conv_norm_kvwrite(rows, self.conv_w, step.cu_q, step.positions, step.slot_ids, layer.state, table, qkv,
+                                  layer.k_pages, layer.v_pages, H, KV, d, step.n_seqs, max(step.q_lens),
+                                  norm_dim=self.dk if self.qk_norm is not None else None,
+                                  eps=self.qk_norm[2] if self.qk_norm is not None else 0.0,
+                                  q_weight=self.q_norm_w, k_weight=self.k_norm_w)
         elif self.row_norm is not None:
             # the projection's 32-bit sums are kept up to the norm: biases, the values (which may
             # be the keys as they stand), the norm over whole rows, rotation and cache write are
@@ -466,7 +546,7 @@ class PagedAttention(Mixer):
             ops.attn_prefill(qkv, layer.k_pages, layer.v_pages, table, step.cu_q, step.ctx_lens,
                              work, out, H, KV, d, self.scale, window, self.slopes, rows_per_item,
                              keep_first=self.keep_first, gate=gate_in_kernel, sinks=self.sinks,
-                             score_cap=self.score_cap, chunk=chunk)
+                             score_cap=self.score_cap, chunk=chunk, dist=self.dist)
         if step.n_decode:
             splits = self._decode_cuts(step, ops.attention_on_matrix_cores(act, bs, d))
             workspace = None
@@ -478,7 +558,7 @@ class PagedAttention(Mixer):
                             window, splits, workspace,
                             token_is_seq=step.decode_seq_ids is None and work is None,
                             slopes=self.slopes, keep_first=self.keep_first, gate=gate_in_kernel,
-                            sinks=self.sinks, score_cap=self.score_cap, chunk=chunk)
+                            sinks=self.sinks, score_cap=self.score_cap, chunk=chunk, dist=self.dist)
         if gate is not None and gate_in_kernel is None:
             ops.sigmoid_gate(out, gate)
         if head_gates is not None or self.out_scale != 1.0:

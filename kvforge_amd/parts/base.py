@@ -170,6 +170,9 @@ class Part:
 
 
 class Norm(Part):
+    # whether ``forward`` takes ``bias=``, a vector still owed to every row of ``x`` (``Step.owe_bias``)
+    adds_bias = False
+
     def forward(self, x: torch.Tensor, out: torch.Tensor, rows: torch.Tensor | None = None,
                 add: torch.Tensor | None = None) -> None:
         """``out[m] = norm(x[rows[m] or m])``; ``x`` is the fp32 residual stream.  ``add`` is a

@@ -12,6 +12,15 @@ from kvforge_amd.parts.base import (Block, FeedForward, LayerState, Mixer, Norm,
 from kvforge_amd.registry import register_block
 
 
+def norm_rows(norm: Norm, stream: torch.Tensor, out: torch.Tensor, step, rows: torch.Tensor | None = None) -> None:
+    """``out = norm(stream)`` (of the rows ``rows``), with what the step still owes the stream added on the way."""
+    if norm.adds_bias and step.owed_bias is not None:
+        bias = step.take_owed_bias(stream)
+        norm.forward(stream, out, rows, add=step.take_owed(stream), bias=bias)
+    else:
+        norm.forward(stream, out, rows, add=step.take_owed(stream))
+
+
 @register_block("pre_norm")
 class PreNormBlock(Block):
     """``ffn`` (and its norm) may be ``None``: a layer of the mixer alone."""
@@ -39,7 +48,7 @@ class PreNormBlock(Block):
             self.mixer.forward(residual, step, layer, residual)
         else:
             x = step.ws.buf("normed", tuple(residual.shape), step.act_dtype)
-            self.mixer_norm.forward(residual, x, add=step.take_owed(residual))
+            norm_rows(self.mixer_norm, residual, x, step)
             self.mixer.forward(x, step, layer, residual)
         if self.ffn is None:
             return
@@ -49,7 +58,7 @@ class PreNormBlock(Block):
             self.ffn.forward(residual, step, residual)
         else:
             x = step.ws.buf("normed", tuple(residual.shape), step.act_dtype)
-            self.ffn_norm.forward(residual, x, add=step.take_owed(residual))
+            norm_rows(self.ffn_norm, residual, x, step)
             self.ffn.forward(x, step, residual)
 
 
@@ -138,7 +147,7 @@ class ParallelBlock(Block):
             ops.rmsnorm_pair(residual, self.norm.weight, self.ffn_norm.weight, self.norm.eps, hs, h,
                              add=step.take_owed(residual))
         else:
-            self.norm.forward(residual, h, add=step.take_owed(residual))
+            norm_rows(self.norm, residual, h, step)
             hs = h
         if self.ffn_norm is not None and not (self.mu is None and self._norms_pair()):
             # of the same stream as the mixer's norm: taken before the mixer adds to it
@@ -265,4 +274,4 @@ class SandwichBlock(Block):
             return
         if owed is not None:
             ops.rms_add(residual, *owed)
-        norm.forward(residual, x, add=step.take_owed(residual))
+        norm_rows(norm, residual, x, step)

@@ -90,22 +90,28 @@ class SwiGLU(FeedForward):
 class GatedFeedForward(SwiGLU):
     """``down(act(gate x + b_gate) * (up x + b_up)) + b_down``.
 
-    ``activation``: ``"silu"`` or ``"gelu_tanh"`` (``0.5 z (1 + tanh(sqrt(2/pi) (z + 0.044715 z^3)))``).
+    ``activation``: ``"silu"``, ``"gelu_tanh"`` (``0.5 z (1 + tanh(sqrt(2/pi) (z + 0.044715 z^3)))``), or
+    ``"limited"``, which joins the pair otherwise: with ``g = min(gate, limit)`` and ``u = clamp(up, -limit,
+    limit)`` it is ``g sigmoid(1.702 g) (u + 1)``.  ``out_scale``: a constant on the output, applied in fp32
+    ahead of the (linear) down projection and to its bias.
     ``bias``: whether the three projections have biases; they are held in fp32 and added in
     fp32, the first two inside the activation kernel.  The bias of the down projection belongs
-    to the stream: ``forward`` adds it with a kernel of its own unless the block asks to add it
-    itself (``defer_down_bias``), in which case it is found in ``down_bias``.
+    to the stream, to which ``forward`` leaves it owed (``Step.owe_bias``: the next norm adds it on its way)
+    unless the block asks to add it itself (``defer_down_bias``), in which case it is found in ``down_bias``.
     ``names``: checkpoint names under the prefix, by ``gate up down``; a bias is ``<name><bias_suffix>``."""
 
     NAMES = {"gate": "gate_proj.weight", "up": "up_proj.weight", "down": "down_proj.weight"}
 
     def __init__(self, prefix: str, hidden: int, intermediate: int, activation: str = "silu",
                  bias: bool = False, names: dict[str, str] | None = None,
-                 bias_suffix: str = ".bias") -> None:
+                 bias_suffix: str = ".bias", limit: float | None = None, out_scale: float = 1.0) -> None:
         super().__init__(prefix, hidden, intermediate)
-        if activation not in ops.ACTIVATIONS:
-            raise ValueError(f"unknown activation {activation!r}; known: {sorted(ops.ACTIVATIONS)}")
+        if activation not in ops.GATE_FORMS:
+            raise ValueError(f"unknown activation {activation!r}; known: {sorted(ops.GATE_FORMS)}")
+        if (activation == "limited") != (limit is not None) or (limit is not None and not limit > 0):
+            raise ValueError(f"a positive limit goes with 'limited' pairs, got {activation!r} and {limit}")
         self.activation, self.bias = activation, bool(bias)
+        self.limit, self.out_scale = limit, float(out_scale)
         self.names = dict(self.NAMES, **(names or {}))
         self.bias_suffix = bias_suffix
         self.gate_bias = self.up_bias = self.down_bias = None
@@ -131,6 +137,8 @@ class GatedFeedForward(SwiGLU):
             self.gate_bias, self.up_bias, self.down_bias = (
                 tensors[self._name(self.names[n] + self.bias_suffix)].float().contiguous()
                 for n in ("gate", "up", "down"))
+            if self.out_scale != 1.0:
+                self.down_bias = self.down_bias * self.out_scale
 
     def absorb_norm(self, norm) -> bool:
         return False
@@ -151,16 +159,16 @@ class GatedFeedForward(SwiGLU):
         act = ws.buf("ffn_act", (n, self.inter), dt)
         if ops.bf16_kernel_takes(x, self.w_gate_up, False, True) and self.inter % 2 == 0:
             # one kernel: gate/up projection, biases, activation, gate
-            ops.gemm_gated(x, self.w_gate_up, act, self.activation, self.gate_bias, self.up_bias)
+            ops.gemm_gated(x, self.w_gate_up, act, self.activation, self.gate_bias, self.up_bias, limit=self.limit,
+                           scale=self.out_scale)
         else:
             gu = ws.buf("gate_up", (n, 2 * self.inter), dt)
             ops.gemm(x, self.w_gate_up, gu)
             ops.gated_act(gu, act, self.activation, paired=True, gate_bias=self.gate_bias,
-                          up_bias=self.up_bias)
+                          up_bias=self.up_bias, limit=self.limit, scale=self.out_scale)
         add_product(step, act, self.w_down, residual)
         if self.down_bias is not None and not self.defer_down_bias:
-            step.settle()
-            ops.add_bias(residual, self.down_bias)
+            step.owe_bias(residual, self.down_bias)
 
 
 @register_feed_forward("plain")

@@ -14,7 +14,8 @@ expert's output may be multiplied by ``sigmoid(w . x)``, one number per token.
 
 Variants of the router: ``s = sigmoid(W_r x)`` of every output by itself, weights that are the chosen
 ``s`` as they are, no correction, and weights that belong to the chosen experts' inputs,
-``sum expert(w x)``, instead of their outputs.
+``sum expert(w x)``, instead of their outputs; or outputs chosen by their logits (``W_r x`` plus a bias)
+and weighted by the softmax over the chosen logits alone.
 """
 
 from __future__ import annotations
@@ -40,17 +41,22 @@ class RoutedExperts(FeedForward):
     whether the weights are divided by their sum; ``correct``: whether there is a ``correction``;
     ``weigh_input``: the weights go into the experts' inputs (gate and up are linear in it, so they
     are multiplied into those two products' fp32 sums, or into the stored products, ahead of the
-    activation)."""
+    activation).  ``scores="chosen"``: chosen by the logits, weighted by the softmax over the chosen
+    ones.  ``router_bias``: the logits get a bias (fp32, named ``router_bias``).  ``form``, ``limit``: how an
+    expert joins its pairs (``ops.MOE_FORMS``).  ``out_scale``: a constant on the experts' sum, taken into
+    their weights (it goes without weights on the inputs, identity outputs and a shared expert)."""
 
     NAMES = {"expert": "e{e}", "gate": "gate", "up": "up", "down": "down", "router": "router",
-             "correction": "correction", "shared": "shared", "table": "table", "shared_gate": "sg"}
+             "correction": "correction", "shared": "shared", "table": "table", "shared_gate": "sg",
+             "router_bias": "router.b"}
 
     replayable = True
 
     def __init__(self, prefix: str, hidden: int, ff: int, experts: int, top: int, identity: int = 0,
                  shared_ff: int = 0, names: dict[str, str] | None = None, table_vocab: int | None = None,
                  shared_gate: bool = False, scores: str = "softmax", renormalize: bool = True,
-                 correct: bool = True, weigh_input: bool = False) -> None:
+                 correct: bool = True, weigh_input: bool = False, router_bias: bool = False,
+                 form: str = "silu", limit: float | None = None, out_scale: float = 1.0) -> None:
         self.prefix, self.hidden, self.ff = prefix, int(hidden), int(ff)
         self.E, self.top, self.identity = int(experts), int(top), int(identity)
         self.R = self.E + self.identity
@@ -65,6 +71,15 @@ class RoutedExperts(FeedForward):
             raise ValueError(f"unknown router scores {scores!r}; known: {sorted(ops.MOE_SCORES)}")
         self.scores, self.renormalize = scores, bool(renormalize)
         self.correct, self.weigh_input = bool(correct), bool(weigh_input)
+        self.router_bias, self.form, self.limit = bool(router_bias), form, limit
+        self.out_scale = float(out_scale)
+        if form not in ops.MOE_FORMS or (form == "limited") != (limit is not None) or (limit is not None and not limit > 0):
+            raise ValueError(f"experts join their pairs by one of {ops.MOE_FORMS}, 'limited' with a positive limit; "
+                             f"got {form!r} and {limit}")
+        if self.scores == "chosen" and (self.correct or self.identity):
+            raise ValueError("weights that are a softmax over the chosen logits go without correction and identity outputs")
+        if self.out_scale != 1.0 and (self.weigh_input or self.identity or shared_ff or self.table_vocab):
+            raise ValueError("a constant on the experts' sum goes with weights on their outputs and nothing beside them")
         if self.weigh_input and self.identity:
             raise ValueError("weights on the experts' inputs go without identity outputs")
         if not 0 < self.top <= min(self.R, ops.MOE_MAX_TOP) or self.R > ops.MOE_MAX_ROUTER_OUTPUTS:
@@ -76,7 +91,7 @@ class RoutedExperts(FeedForward):
             self.shared = GatedFeedForward(
                 self._name(self.names["shared"]), hidden, shared_ff, activation="silu",
                 names={k: self.names[k] for k in ("gate", "up", "down")})
-        self.w_router = self.correction = self.w_gate_up = self.w_down = None
+        self.w_router = self.correction = self.r_bias = self.w_gate_up = self.w_down = None
 
     def _expert(self, e: int, which: str) -> str:
         return self._name(f"{self.names['expert'].format(e=e)}.{self.names[which]}")
@@ -90,6 +105,8 @@ class RoutedExperts(FeedForward):
             out = {self._name(self.names["router"]): WeightSpec((self.R, h))}
             if self.correct:
                 out[self._name(self.names["correction"])] = WeightSpec((self.R,))
+            if self.router_bias:
+                out[self._name(self.names["router_bias"])] = WeightSpec((self.R,), std=0.5)
         for e in range(self.E):
             out[self._expert(e, "gate")] = WeightSpec((ff, h))
             out[self._expert(e, "up")] = WeightSpec((ff, h))
@@ -112,6 +129,8 @@ class RoutedExperts(FeedForward):
             self.w_router = torch.cat([r, r.new_zeros(self.R_pad - self.R, self.hidden)], dim=0).contiguous()
             if self.correct:
                 self.correction = tensors[self._name(self.names["correction"])].float().contiguous()
+            if self.router_bias:
+                self.r_bias = tensors[self._name(self.names["router_bias"])].float().contiguous()
         if self.shared_gate:
             # one row, padded with zero rows to 16 (which every product kernel takes)
             g = tensors[self.shared._name(self.names["shared_gate"])]
@@ -152,7 +171,7 @@ class RoutedExperts(FeedForward):
         experts = sum(t.numel() * t.element_size() for t in map(ops.plain_of, (self.w_gate_up, self.w_down))
                       if t is not None)
         small = sum(t.numel() * t.element_size()
-                    for t in (ops.plain_of(self.w_router) if self.w_router is not None else None, self.correction,
+                    for t in (ops.plain_of(self.w_router) if self.w_router is not None else None, self.correction, self.r_bias,
                               ops.plain_of(self.w_shared_gate) if self.w_shared_gate is not None else None)
                     if t is not None)
         return (small + experts * min(self.top, self.E) // max(self.E, 1)
@@ -162,7 +181,7 @@ class RoutedExperts(FeedForward):
         return (ops.copies_of(self.w_gate_up) + ops.copies_of(self.w_down)
                 + (ops.copies_of(self.w_router) if self.w_router is not None else [])
                 + (ops.copies_of(self.w_shared_gate) if self.w_shared_gate is not None else [])
-                + [t for t in (self.correction, self.table) if t is not None]
+                + [t for t in (self.correction, self.r_bias, self.table) if t is not None]
                 + (self.shared.held_tensors() if self.shared is not None else []))
 
     def forward(self, x, step, residual) -> None:
@@ -177,7 +196,8 @@ class RoutedExperts(FeedForward):
         else:
             logits = ws.buf("moe_logits", (n, self.R_pad), torch.float32)[:, :self.R]
             ops.gemm(x, self.w_router, ws.buf("moe_logits", (n, self.R_pad), torch.float32))   # 32-bit sums, stored so
-            ops.moe_topk(logits, self.correction, chosen, weights, self.scores, self.renormalize)
+            ops.moe_topk(logits, self.correction, chosen, weights, self.scores, self.renormalize, bias=self.r_bias,
+                         scale=self.out_scale)
         if ops.moe_grouped_takes(x, self.w_gate_up, self.w_down, self.E, self.ff) and x.is_contiguous():
             # bf16: every expert over only the rows that chose it, grouped on the device
             pairs, tiles = n * self.top, ops.moe_grouped_tiles(n, self.top, self.E)
@@ -191,7 +211,7 @@ class RoutedExperts(FeedForward):
             if fresh:
                 step.fresh = None      # written here instead of added to
             ops.moe_grouped(x, self.w_gate_up, self.w_down, chosen, weights, residual, self.E, self.ff, scratch,
-                            weigh_input=self.weigh_input, fresh=fresh)
+                            weigh_input=self.weigh_input, fresh=fresh, form=self.form, limit=self.limit)
             self._shared_forward(x, step, residual)
             return
         # otherwise (32-bit, or sizes the grouped kernels do not take): every expert over every
@@ -202,7 +222,7 @@ class RoutedExperts(FeedForward):
         gu = ws.buf("moe_gate_up", (n, 2 * self.E * self.ff), dt)
         ops.gemm(x, self.w_gate_up, gu)
         act = ws.buf("moe_act", (n, self.E * self.ff), dt)
-        ops.moe_dense_act(gu, chosen, weights, act, self.E, self.ff, self.weigh_input)
+        ops.moe_dense_act(gu, chosen, weights, act, self.E, self.ff, self.weigh_input, self.form, self.limit)
         add_product(step, act, self.w_down, residual)
         if self.identity and not first:     # fresh rows are written by the product before they are added to
             ops.moe_identity(residual, x, chosen, weights, self.E)

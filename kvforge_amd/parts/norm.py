@@ -14,6 +14,7 @@ class RMSNorm(Norm):
     """``y = x * rsqrt(mean(x^2) + eps) * weight`` in fp32, rounded once to the output type."""
 
     replayable = True
+    adds_bias = True
 
     def __init__(self, prefix: str, width: int, eps: float) -> None:
         self.prefix, self.width, self.eps = prefix, int(width), float(eps)
@@ -35,8 +36,8 @@ class RMSNorm(Norm):
         return [] if self.weight is None else [self.weight]
 
     def forward(self, x: torch.Tensor, out: torch.Tensor, rows: torch.Tensor | None = None,
-                add: torch.Tensor | None = None) -> None:
-        ops.rmsnorm(x, self.weight, self.eps, out, rows, add)
+                add: torch.Tensor | None = None, bias: torch.Tensor | None = None) -> None:
+        ops.rmsnorm(x, self.weight, self.eps, out, rows, add, bias)
 
     def add_to(self, stream: torch.Tensor, y: torch.Tensor) -> None:
         if self.weight.dtype != torch.float32:

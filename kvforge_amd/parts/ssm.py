@@ -5,8 +5,9 @@ Per head a memory ``S [dk, dv]`` that starts at zero; for a token with rows ``q,
 several memories may share) and ``v``, a step ``dt = softplus(z_a + dt_bias)`` and the decay
 ``a = exp(-exp(A_log) dt)``::
 
-    Mamba2      S <- a S + dt k v^T;                              y = S^T q + D v
-    GatedDelta  S <- a S;   S <- S + k (beta (v - S^T k))^T;      o = S^T q       (beta = sigmoid(z_b))
+    Mamba2        S <- a S + dt k v^T;                              y = S^T q + D v
+    GatedDelta    S <- a S;   S <- S + k (beta (v - S^T k))^T;      o = S^T q       (beta = sigmoid(z_b))
+    ChannelDelta  the same with one decay per key channel, S <- diag(a) S
 
 q, k and v pass a convolution over the last few tokens, channel by channel, and silu.  A request's
 state slot holds every head's ``S`` and the convolution's last inputs in fp32, so that a prompt may
@@ -122,18 +123,25 @@ class ConvMemory(Mixer):
                      layer.state, self.state_off, mixed, step.n_seqs, max(step.q_lens), unit=self.unit,
                      key_dim=self.dk, q_scale=self.q_scale)
         raw = ws.buf("ssm_raw", (n, self.H * self.dv), torch.float32)
+        gate_rows = self.scan(mixed, rows, gates, raw, step, layer)
+        heads = ws.buf("ssm_heads", (n, self.H * self.dv), act)
+        self.finish(raw, gate_rows, heads)
+        add_product(step, heads, self.w_o, residual)
+
+    def scan(self, mixed, rows, gates, raw, step, layer: LayerState) -> torch.Tensor:
+        """``raw``: the memories' read-out (fp32), from the convolved rows ``mixed`` and what the two projections
+        gave (``rows``, ``gates``).  Returns the rows that hold the output gate, for ``finish``."""
         # which kernels have work is known from the runs' lengths (all ones in a captured step of
         # single tokens, so a replay launches what the capture launched)
         ops.ssm_scan(mixed, self.q_off, self.k_off, self.v_off, gates, self.a_off, self.b_off, self.neg_a, self.dt_bias,
                      self.skip, step.cu_q, step.positions, step.slot_ids, layer.state, raw, step.n_seqs, self.H, self.G,
                      self.dk, self.dv, multi=self._long_runs(step),
                      short_runs=any(q < ops.SSM_CHUNK_FROM for q in step.q_lens))
-        heads = ws.buf("ssm_heads", (n, self.H * self.dv), act)
-        self.finish(raw, rows, heads)
-        add_product(step, heads, self.w_o, residual)
+        return rows
 
     def finish(self, raw: torch.Tensor, rows: torch.Tensor, heads: torch.Tensor) -> None:
-        """``heads``: what the output projection reads, from the memories' read-out ``raw`` (fp32)."""
+        """``heads``: what the output projection reads, from the memories' read-out ``raw`` (fp32) and the rows that
+        ``scan`` returned."""
         raise NotImplementedError
 
 
@@ -228,3 +236,87 @@ class GatedDelta(ConvMemory):
     def finish(self, raw, rows, heads) -> None:
         V = self.H * self.dv
         ops.linmem_out(raw, rows[:, self.channels:self.channels + V], self.norm_w, self.norm_eps, heads, self.H, self.dv)
+
+
+@register_mixer("channel_delta")
+class ChannelDelta(GatedDelta):
+    """The gated delta rule with a decay per head and key channel and gates of low rank.  Channel ``i`` of
+    head ``h`` decays by ``exp(-exp(A_log[h]) softplus((W_a2 W_a1 x)[h, i] + dt_bias[h, i]))``.  Every memory's read-out
+    is divided by its root mean square, multiplied by a weight ``[value_dim]`` that the heads share and by
+    ``sigmoid(W_g2 W_g1 x)``, element by element.  ``a_rank``, ``g_rank``: the ranks (``None``: the checkpoint's).
+    ``names``: checkpoint names under the prefix, by ``q k v b a1 a2 g1 g2 A_log dt_bias norm o`` and ``conv``.
+
+    One product holds q, k, v and the two low-rank rows, a second (over ``[W_a1 x | W_g1 x]``, the two second
+    matrices as diagonal blocks) the pre-activations of decays and output gate, with fp32 sums stored in fp32."""
+
+    NAMES = {"q": "q", "k": "k", "v": "v", "b": "b", "a1": "a1", "a2": "a2", "g1": "g1", "g2": "g2", "A_log": "A_log",
+             "dt_bias": "dt_bias", "norm": "norm", "o": "o", "conv": "{of}.conv"}
+
+    def __init__(self, prefix: str, hidden: int, heads: int, key_heads: int, key_dim: int, value_dim: int, taps: int,
+                 norm_eps: float, names: dict[str, str] | None = None, a_rank: int | None = None,
+                 g_rank: int | None = None) -> None:
+        super().__init__(prefix, hidden, heads, key_heads, key_dim, value_dim, taps, norm_eps, names)
+        self.a_rank, self.g_rank = a_rank, g_rank
+        self.b_off = 0
+        self.w_low2 = None
+        self.low = self.low2 = None      # columns of the low-rank rows in the first product, width of the second's input
+
+    def weight_specs(self) -> dict[str, WeightSpec]:
+        h, H, Q, V, K = self.hidden, self.H, self.G * self.dk, self.H * self.dv, self.H * self.dk
+        n = lambda key: self._name(self.names[key])  # noqa: E731
+        out = {n("o"): WeightSpec((h, V)), n("b"): WeightSpec((H, h)), n("A_log"): WeightSpec((H,), std=0.5),
+               n("dt_bias"): WeightSpec((K,), std=1.0), n("norm"): WeightSpec((self.dv,), init="norm", std=0.1),
+               n("a1"): WeightSpec((self.a_rank, h)), n("a2"): WeightSpec((K, self.a_rank)),
+               n("g1"): WeightSpec((self.g_rank, h)), n("g2"): WeightSpec((V, self.g_rank))}
+        for key, rows in (("q", Q), ("k", Q), ("v", V)):
+            out[n(key)] = WeightSpec((rows, h))
+            out[self._conv(key)] = WeightSpec((rows, self.taps), std=0.3)
+        return out
+
+    def load(self, tensors: dict[str, torch.Tensor]) -> None:
+        t = lambda key: tensors[self._name(self.names[key])]  # noqa: E731
+        a1, a2, g1, g2 = _one_type([t(k) for k in ("a1", "a2", "g1", "g2")])
+        ra, rg = int(a1.shape[0]), int(g1.shape[0])
+        for first, second, rank, want in (("a1", a2, ra, self.a_rank), ("g1", g2, rg, self.g_rank)):
+            if second.shape[1] != rank or rank <= 0 or (want is not None and rank != want):
+                raise ValueError(f"{self._name(self.names[first])} and the matrix behind it do not agree on their rank")
+        pa, pg = -(-ra // 16) * 16, -(-rg // 16) * 16     # ranks as every product kernel takes them
+        rows = _one_type([t(k) for k in ("q", "k", "v")] + [a1, g1])
+        lead = rows[0].new_zeros(-self.channels % 16, self.hidden)      # the low-rank rows start on 16 bytes
+        self.low = self.channels + lead.shape[0]
+        self.low2 = pa + pg
+        pad = lambda w, n: torch.cat([w, w.new_zeros(n - w.shape[0], w.shape[1])], dim=0)  # noqa: E731
+        self.w_rows = torch.cat([*rows[:3], lead, pad(rows[3], pa), pad(rows[4], pg)], dim=0).contiguous()
+        K, V = self.H * self.dk, self.H * self.dv
+        second = a2.new_zeros(-(-(K + V) // 16) * 16, pa + pg)
+        second[:K, :ra], second[K:K + V, pa:pa + rg] = a2, g2
+        self.w_low2 = second
+        self.w_gates = _padded_rows(t("b"))
+        self.conv_w = torch.cat([tensors[self._conv(k)].float() for k in ("q", "k", "v")], dim=0).contiguous()
+        self._take_gates(tensors)
+
+    def seal(self) -> None:
+        super().seal()
+        self.w_low2 = ops.streamed(ops.plain_of(self.w_low2))
+
+    def kernel_modules(self, dtype: torch.dtype) -> set[str]:
+        return super().kernel_modules(dtype) | {"chdelta"}
+
+    def _matrices(self) -> list:
+        return super()._matrices() + ([self.w_low2] if self.w_low2 is not None else [])
+
+    def _long_runs(self, step) -> dict | None:
+        return None
+
+    def scan(self, mixed, rows, gates, raw, step, layer: LayerState) -> torch.Tensor:
+        n = rows.shape[0]
+        low = step.ws.buf("chdelta_gates", (n, self.w_low2.shape[0]), torch.float32)
+        ops.gemm(rows[:, self.low:self.low + self.low2], self.w_low2, low)     # 32-bit sums, stored so
+        ops.chdelta_scan(mixed, self.q_off, self.k_off, self.v_off, low, 0, gates, self.b_off, self.neg_a, self.dt_bias,
+                         step.cu_q, step.positions, step.slot_ids, layer.state, raw, step.n_seqs, self.H, self.G,
+                         self.dk, self.dv, multi=self._long_runs(step),
+                         short_runs=any(q < ops.CHDELTA_CHUNK_FROM for q in step.q_lens))
+        return low[:, self.H * self.dk:self.H * (self.dk + self.dv)]
+
+    def finish(self, raw, rows, heads) -> None:
+        ops.linmem_out(raw, rows, self.norm_w, self.norm_eps, heads, self.H, self.dv, sigmoid=True)
