@@ -377,6 +377,78 @@ PRESETS["balalorn-1b"] = balalorn_stack(
     top=4)
 
 
+def depolix(vocab: int, width: int, layers: list, eps: float = 1e-6, embed_scale: float = 1.0,
+            residual_mult: float = 1.0, logit_scale: float = 1.0, max_positions: int | None = None) -> dict[str, Any]:
+    """A Depolix config.json.  ``layers``: one ``(type, mixer, mlp)`` per layer.  For ``"latent_attention"`` the mixer
+    holds ``heads dim rot_dim vdim q_rank kv_rank scale`` and optionally ``base`` and ``scaling`` (``(factor, original, fast,
+    slow)``); for ``"parallel"`` ``left`` (``heads kv_heads dim vdim scale conv bias_max buckets`` and optionally ``window``,
+    ``keep_first``) and ``right`` (``heads kv_heads dim vdim conv a_rank g_rank``).  ``mlp``: ``None``, ``(ff, limit)`` for a dense
+    feed-forward or ``(ff, limit, experts, top)``."""
+    out = []
+    for kind, m, mlp in layers:
+        mixer = dict(m)
+        if kind == "latent_attention":
+            base, sc = mixer.pop("base", 10000.0), mixer.pop("scaling", None)
+            rot: dict[str, Any] = {"base": float(base), "dims": m["rot_dim"]}
+            if sc is not None:
+                rot["scaling"] = dict(zip(("factor", "original", "fast", "slow"), sc))
+            mixer["rot"] = rot if m["rot_dim"] else None
+        else:
+            left = dict(m["left"])
+            window, keep = left.pop("window", None), left.pop("keep_first", 0)
+            if window:
+                left["mask"] = {"keep_first": keep, "size": window}
+            mixer = {"left": left, "right": dict(m["right"])}
+        if mlp is None:
+            ff: dict[str, Any] | None = None
+        elif len(mlp) == 2:
+            ff = {"ff": mlp[0], "kind": "dense", "limit": mlp[1]}
+        else:
+            ff = {"expert": {"ff": mlp[0], "limit": mlp[1]}, "kind": "moe", "router": {"experts": mlp[2], "top": mlp[3]}}
+        out.append({"mixer": mixer, "mlp": ff, "type": kind})
+    cfg: dict[str, Any] = {"architecture": "Depolix", "embedding": {"scale": embed_scale}, "layers": out,
+                           "logit_scale": logit_scale, "norm": {"eps": eps}, "residual_mult": residual_mult,
+                           "vocab": vocab, "width": width}
+    if max_positions is not None:
+        cfg["max_positions"] = max_positions
+    return cfg
+
+
+def depolix_stack(vocab: int, width: int, groups: int, heads: int, latent_dim: int, rot_dim: int, q_rank: int,
+                  kv_rank: int, att_heads: int, att_kv_heads: int, att_dim: int, window: int, mem_heads: int,
+                  mem_kv_heads: int, mem_dim: int, mem_vdim: int, gate_rank: int, ff: int, moe_ff: int, experts: int,
+                  top: int, max_positions: int = 131072) -> dict[str, Any]:
+    """``groups`` times (latent attention with a dense feed-forward, two mixers side by side with experts, latent
+    attention with experts, two mixers side by side with a dense feed-forward)."""
+    lat = dict(heads=heads, dim=latent_dim, rot_dim=rot_dim, vdim=latent_dim, q_rank=q_rank, kv_rank=kv_rank,
+               scale=float(latent_dim + rot_dim) ** -0.5, base=1000000.0, scaling=(4.0, 8192, 32.0, 1.0))
+    par = dict(left=dict(heads=att_heads, kv_heads=att_kv_heads, dim=att_dim, vdim=att_dim, scale=float(att_dim) ** -0.5,
+                         conv=4, bias_max=128, buckets=32, window=window, keep_first=16),
+               right=dict(heads=mem_heads, kv_heads=mem_kv_heads, dim=mem_dim, vdim=mem_vdim, conv=4, a_rank=gate_rank,
+                          g_rank=gate_rank))
+    dense, moe = (ff, 7.0), (moe_ff, 7.0, experts, top)
+    layers = [("latent_attention", lat, dense), ("parallel", par, moe), ("latent_attention", lat, moe),
+              ("parallel", par, dense)] * groups
+    return depolix(vocab, width, layers, max_positions=max_positions)
+
+
+PRESETS["depolix-tiny"] = depolix(
+    vocab=288, width=80,
+    layers=[("latent_attention", dict(heads=3, dim=16, rot_dim=8, vdim=24, q_rank=40, kv_rank=24, scale=0.2,
+                                      scaling=(4.0, 64, 16.0, 1.0)), (112, 3.0)),
+            ("parallel", dict(left=dict(heads=4, kv_heads=2, dim=16, vdim=24, scale=0.25, conv=3, bias_max=40, buckets=8,
+                                        window=24, keep_first=4),
+                              right=dict(heads=4, kv_heads=2, dim=24, vdim=16, conv=4, a_rank=8, g_rank=12)),
+             (32, 3.0, 6, 2)),
+            ("latent_attention", dict(heads=2, dim=24, rot_dim=4, vdim=16, q_rank=24, kv_rank=40, scale=0.25), None)],
+    embed_scale=9.0, residual_mult=0.8, logit_scale=1.5, max_positions=1024)
+# layers of the width of llama-1b: what this design's kernels are measured at
+PRESETS["depolix-1b"] = depolix_stack(
+    vocab=128256, width=2048, groups=4, heads=32, latent_dim=64, rot_dim=32, q_rank=768, kv_rank=192, att_heads=32,
+    att_kv_heads=8, att_dim=64, window=1024, mem_heads=16, mem_kv_heads=8, mem_dim=128, mem_vdim=128, gate_rank=128, ff=8192,
+    moe_ff=1024, experts=32, top=4)
+
+
 def preset_dict(name: str) -> dict[str, Any]:
     try:
         return dict(PRESETS[name])

@@ -2223,6 +2223,15 @@ def ssm_scan(rows: torch.Tensor, q_off: int, k_off: int, v_off: int, gates: torc
 CHDELTA_CHUNK_FROM = 24
 
 
+def chdelta_scratch(n_tokens: int, n_chunks: int, heads: int, key_dim: int, value_dim: int) -> dict[str, tuple]:
+    """(shape, dtype) of the scratch tensors the passes over the chunks (of ``ssm_plan``) need, by name."""
+    H, dk, dv, cl = int(heads), int(key_dim), int(value_dim), ssm_chunk_len(key_dim)
+    out = {name: ((n_chunks, H, cl, cl), F32) for name in ("T", "A")}
+    out.update({name: ((n_tokens, H, dk), F32) for name in ("Kd", "Kw", "Qd")})
+    out.update({"E": ((n_chunks, H, dk), F32), "W": ((n_chunks, H, dk, dv), F32), "U": ((n_tokens, H, dv), F32)})
+    return out
+
+
 def chdelta_scan(rows: torch.Tensor, q_off: int, k_off: int, v_off: int, decay: torch.Tensor, a_off: int,
                  steps: torch.Tensor, b_off: int, neg_a: torch.Tensor, dt_bias: torch.Tensor, cu_q: torch.Tensor,
                  positions: torch.Tensor, slot_ids: torch.Tensor, state: torch.Tensor, out: torch.Tensor, n_seqs: int,
@@ -2233,7 +2242,9 @@ def chdelta_scan(rows: torch.Tensor, q_off: int, k_off: int, v_off: int, decay: 
     a block of columns of wider slots).  ``rows`` as in ``ssm_scan``.  ``decay`` fp32 ``[n, >= a_off + heads *
     key_dim]``: ``a = exp(neg_a[h] * softplus(decay[a_off + h * key_dim + i] + dt_bias[h * key_dim + i]))`` multiplies key row
     ``i``; ``steps`` fp32: ``beta = sigmoid(steps[b_off + h])``.  ``S <- diag(a) S``, ``S <- S + k (beta (v - S^T k))^T``,
-    ``o = S^T q``."""
+    ``o = S^T q``.  ``multi``: ``chunks`` and ``runs`` (int32 device tensors of ``ssm_plan``'s rows, made with
+    ``CHDELTA_CHUNK_FROM``) and the tensors of ``chdelta_scratch``: those runs go chunk by chunk and the
+    token-by-token kernel leaves them alone; it is not launched with ``short_runs=False``."""
     n = rows.shape[0]
     H, G, dk, dv = int(heads), int(key_heads), int(key_dim), int(value_dim)
     _check(rows, "rows", F32, (n, None), contiguous=False)
@@ -2266,6 +2277,19 @@ def chdelta_scan(rows: torch.Tensor, q_off: int, k_off: int, v_off: int, decay: 
         f = _fn("chdelta", "kvf_chdelta_scan", types + [c_void_p, c_int, c_int, c_void_p])
         _ok(f(*common, cu_q.data_ptr(), int(n_seqs), CHDELTA_CHUNK_FROM if multi is not None else 0, _stream()),
             "chdelta_scan")
+    if multi is None:
+        return
+    chunks, runs = multi["chunks"], multi["runs"]
+    _check(chunks, "chunks", I32, (None, 4))
+    _check(runs, "runs", I32, (None, 3))
+    nc = chunks.shape[0]
+    for name, (shape, dtype) in chdelta_scratch(n, nc, H, dk, dv).items():
+        _check(multi[name], name, dtype, shape)
+        if multi[name].data_ptr() % 16:
+            raise KernelError(f"chdelta_scan: scratch {name} must start on 16 bytes")
+    f = _fn("chdelta", "kvf_chdelta_chunks", types + [c_void_p, c_int, c_void_p, c_int] + [c_void_p] * 9)
+    _ok(f(*common, chunks.data_ptr(), nc, runs.data_ptr(), runs.shape[0],
+          *(multi[k].data_ptr() for k in ("T", "A", "E", "Kd", "Kw", "Qd", "W", "U")), _stream()), "chdelta_chunks")
 
 
 def ssm_gate_norm(y: torch.Tensor, gate: torch.Tensor, weight: torch.Tensor, eps: float, parts: int,

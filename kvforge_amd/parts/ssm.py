@@ -47,6 +47,7 @@ class ConvMemory(Mixer):
     b_off: int | None = None     # column of the delta rule's gates, ``None`` for plain writes
     unit = 0                     # how many of the first channels are q and k heads made unit vectors
     q_scale = 1.0
+    chunk_from = ops.SSM_CHUNK_FROM   # runs of at least so many tokens go chunk by chunk
 
     def _sizes(self, prefix: str, hidden: int, heads: int, key_heads: int, key_dim: int, value_dim: int, taps: int,
                channels: int, norm_eps: float) -> None:
@@ -93,19 +94,21 @@ class ConvMemory(Mixer):
         """Chunk and run tables of this step's long runs (made once per step, shared by the layers
         whose chunks are equally long) and scratch from the step's workspace.  ``None`` when no run
         is that long."""
-        key = ("ssm.long_runs", ops.ssm_chunk_len(self.dk))
+        key = ("ssm.long_runs", ops.ssm_chunk_len(self.dk), self.chunk_from)
         plan = step.scratch.get(key)
         if plan is None:
-            chunks, runs = ops.ssm_plan(step.q_lens, self.dk)
+            chunks, runs = ops.ssm_plan(step.q_lens, self.dk, self.chunk_from)
             plan = (step.upload_ints(chunks).view(-1, 4), step.upload_ints(runs).view(-1, 3)) if chunks else ()
             step.scratch[key] = plan
         if not plan:
             return None
         out = {"chunks": plan[0], "runs": plan[1]}
-        for name, (shape, dtype) in ops.ssm_scratch(step.n_tokens, plan[0].shape[0], self.H, self.dk, self.dv,
-                                                    self.b_off is not None).items():
+        for name, (shape, dtype) in self._chunk_scratch(step.n_tokens, plan[0].shape[0]).items():
             out[name] = step.ws.buf("ssm_" + name, shape, dtype)
         return out
+
+    def _chunk_scratch(self, n_tokens: int, n_chunks: int) -> dict[str, tuple]:
+        return ops.ssm_scratch(n_tokens, n_chunks, self.H, self.dk, self.dv, self.b_off is not None)
 
     def forward(self, x, step, layer: LayerState, residual) -> None:
         """``x``: the mixer's input rows in the step's activation type."""
@@ -305,8 +308,10 @@ class ChannelDelta(GatedDelta):
     def _matrices(self) -> list:
         return super()._matrices() + ([self.w_low2] if self.w_low2 is not None else [])
 
-    def _long_runs(self, step) -> dict | None:
-        return None
+    chunk_from = ops.CHDELTA_CHUNK_FROM
+
+    def _chunk_scratch(self, n_tokens: int, n_chunks: int) -> dict[str, tuple]:
+        return ops.chdelta_scratch(n_tokens, n_chunks, self.H, self.dk, self.dv)
 
     def scan(self, mixed, rows, gates, raw, step, layer: LayerState) -> torch.Tensor:
         n = rows.shape[0]
