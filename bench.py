@@ -736,6 +736,75 @@ def balalorn_points(dtype, batch, prompt_len, steps, warmup, use_graphs=True, on
     return out
 
 
+# (name, width, latent heads, their plain / rotated / value size, query latent, key latent, attention heads beside the
+#  memories, their kv heads and size, delta memories, q/k heads they share, their key and value size, rank of their
+#  gates, feed-forward, expert width, experts, chosen, groups of four layers, vocabulary): every size that Balalorn has
+#  as in BALALORN_SIZES
+DEPOLIX_SIZES = [("w1024", 1024, 16, 64, 32, 64, 384, 192, 16, 4, 64, 8, 4, 128, 128, 128, 4096, 1024, 16, 4, 2, 32000),
+                 ("w2048", 2048, 32, 64, 32, 64, 768, 192, 32, 8, 64, 16, 8, 128, 128, 128, 8192, 2048, 32, 4, 2, 128256),
+                 ("w4096", 4096, 32, 128, 64, 128, 1536, 192, 32, 8, 128, 32, 16, 128, 128, 128, 14336, 3584, 32, 4, 1, 128256)]
+DEPOLIX_FIELDS = ("width", "latent_heads", "latent_dim", "latent_rot_dim", "latent_vdim", "q_rank", "kv_rank", "heads",
+                  "kv_heads", "head_dim", "delta_heads", "delta_kv_heads", "delta_dim", "delta_vdim", "gate_rank", "ff",
+                  "expert_ff", "experts", "top", "groups", "vocab")
+DEPOLIX_WINDOW, DEPOLIX_KEEP = 1024, 16
+
+
+def depolix_points(dtype, batch, prompt_len, steps, warmup, use_graphs=True, only=None, models=None):
+    """Depolix at a few sizes that resemble a real model's layers (groups of latent attention with a dense
+    feed-forward, attention with a bias by distance beside a delta-rule memory with experts, latent attention with
+    experts, the two side by side with a dense feed-forward), beside the engine's closest existing model, Balalorn, of
+    the same width, latents, memories, feed-forwards and number of layers (``balalorn_points``); random weights drawn
+    on the device.  Per size and model: ms per decode step, its share of the HBM roofline, tokens a second of a
+    2,048-token prefill and its share of the matrix-core peak, with the bytes and products of the work itself, as
+    for Balalorn."""
+    import torch
+    from kvforge_amd.config.presets import depolix_stack
+
+    elem = 2 if dtype == "bfloat16" else 4
+    out = {}
+    for (name, w, H, ld, lr, lv, qr, rank, Ha, KV, d, Hd, Gd, dk, dv, gr, ff, eff, E, top, groups, vocab) in DEPOLIX_SIZES:
+        if only and name not in only:
+            continue
+        if not models or "depolix" in models:
+            cfg = depolix_stack(vocab=vocab, width=w, groups=groups, heads=H, latent_dim=ld, rot_dim=lr, q_rank=qr,
+                                kv_rank=rank, att_heads=Ha, att_kv_heads=KV, att_dim=d, window=DEPOLIX_WINDOW, mem_heads=Hd,
+                                mem_kv_heads=Gd, mem_dim=dk, mem_vdim=dv, gate_rank=gr, ff=ff, moe_ff=eff, experts=E, top=top,
+                                max_positions=CONTEXT_CAP)
+            for layer in cfg["layers"]:
+                if layer["type"] == "latent_attention":
+                    layer["mixer"]["vdim"] = lv
+            latent = w * (qr + rank + lr + 2 * H * lv) + qr * H * (ld + lr) + H * (ld + lv) * rank
+            left = w * (2 * Ha * d + 2 * KV * d + Ha)
+            right = w * (2 * Gd * dk + 2 * Hd * dv + 2 * gr + Hd) + gr * Hd * (dk + dv)
+            routed = 3 * w * eff
+            touched = E * (1.0 - (1.0 - top / E) ** batch)
+            fixed = groups * (2 * (latent + left + right) + 2 * 3 * w * ff + 2 * w * E)
+            state_bytes = 2 * groups * (Hd * dk * dv + 3 * (2 * Gd * dk + Hd * dv) + 3 * (Ha + 2 * KV) * d) * 4 * 2
+            n = PREFILL_TOKENS
+            full, seen = n * n / 2.0, min(n, DEPOLIX_WINDOW)
+            windowed = n * seen - seen * seen / 2.0
+            mixing = 2 * groups * (full * 2.0 * H * (lr + 2 * rank) + windowed * 4.0 * Ha * d + n * 6.0 * Hd * dk * dv)
+            need = batch * (prompt_len + steps + warmup + early_tokens(batch, prompt_len) + 32)
+            engine = build_engine(cfg, dtype, batch, max(need, PREFILL_TOKENS + 64), use_graphs=use_graphs)
+            r = decode_run(engine, vocab, batch, prompt_len, steps, warmup)
+            s = prefill_run(engine, vocab, PREFILL_TOKENS, repeats=2)
+            ctx = r["mean_ctx"]
+            kept = min(ctx, DEPOLIX_WINDOW + DEPOLIX_KEEP) * 2 * KV * d
+            read = ((fixed + 2 * groups * touched * routed + vocab * w) * elem
+                    + batch * (2 * groups * (ctx * (lr + rank) + kept) * elem + state_bytes))
+            flops = 2.0 * n * (fixed + 2 * groups * top * routed) + 2.0 * vocab * w + mixing
+            out[f"{name}_depolix"] = {
+                "decode_ms": round(r["ms_per_step"], 4), "decode_tok_s": round(r["tok_s"], 1),
+                "decode_hbm_frac": round(read / (r["seconds"] / steps) / 1e9 / HBM_PEAK_GBS, 4),
+                "prefill_tok_s": round(PREFILL_TOKENS / s, 1), "prefill_ms": round(s * 1e3, 3),
+                "prefill_frac": round(flops / s / MFMA_PEAK[dtype], 4)}
+            del engine
+            torch.cuda.empty_cache()
+        if not models or "balalorn" in models:
+            out.update(balalorn_points(dtype, batch, prompt_len, steps, warmup, use_graphs, [name], ["balalorn"]))
+    return out
+
+
 def model_numbers(cfg, layers_run):
     h, H, KV, d, I, V = (cfg["hidden_size"], cfg["num_attention_heads"], cfg["num_key_value_heads"],
                          cfg["head_dim"], cfg["intermediate_size"], cfg["vocab_size"])
@@ -764,7 +833,7 @@ def main() -> int:
     ap.add_argument("--no-graphs", action="store_true")
     ap.add_argument("--decode-run-steps", type=int, default=None,
                     help="decode steps the device takes between two looks of the host (engine default: 8)")
-    ap.add_argument("--phase", choices=["all", "decode", "prefill", "mixed", "burst", "products", "fogorax", "rudorax", "buzinex", "ludelix", "balalorn"],
+    ap.add_argument("--phase", choices=["all", "decode", "prefill", "mixed", "burst", "products", "fogorax", "rudorax", "buzinex", "ludelix", "balalorn", "depolix"],
                     default="all",
                     help="for profiles: only the decode steps at --batch, or only the prefill; "
                          "mixed: --batch requests with prompts of 128 to 4,096 tokens, chunked "
@@ -776,8 +845,8 @@ def main() -> int:
                          "Fogorax design at a few layer sizes beside a Llama model of equal sizes; "
                          "rudorax: the Rudorax design likewise (--sizes names some of them); "
                          "buzinex: the Buzinex design likewise; ludelix: the Ludelix design beside Rudorax; "
-                         "balalorn: the Balalorn design beside Buzinex")
-    ap.add_argument("--sizes", default="", help="with --phase rudorax, buzinex, ludelix or balalorn: the sizes to run, with commas")
+                         "balalorn: the Balalorn design beside Buzinex; depolix: the Depolix design beside Balalorn")
+    ap.add_argument("--sizes", default="", help="with --phase rudorax, buzinex, ludelix, balalorn or depolix: the sizes to run, with commas")
     args = ap.parse_args()
     if args.gpus != 1:
         print(f"bench.py measures one GPU; --gpus {args.gpus} is not supported by this engine")
@@ -845,6 +914,16 @@ def main() -> int:
                           **balalorn_points(args.dtype, args.batch, args.prompt_len, steps,
                                             min(args.warmup, 8), not args.no_graphs,
                                             [x for x in args.sizes.split(",") if x] or None)}))
+        return 0
+    if args.phase == "depolix":
+        steps = min(args.steps, 64)
+        print(json.dumps({"phase": "depolix", "dtype": args.dtype, "batch": args.batch,
+                          "prompt_len": args.prompt_len, "steps": steps, "window": DEPOLIX_WINDOW,
+                          "keep_first": DEPOLIX_KEEP, "prefill_tokens": PREFILL_TOKENS,
+                          "sizes": {r[0]: dict(zip(DEPOLIX_FIELDS, r[1:])) for r in DEPOLIX_SIZES},
+                          **depolix_points(args.dtype, args.batch, args.prompt_len, steps,
+                                           min(args.warmup, 8), not args.no_graphs,
+                                           [x for x in args.sizes.split(",") if x] or None)}))
         return 0
     if args.preset == "small" and args.phase != "burst":
         print("--preset small goes with --phase burst")

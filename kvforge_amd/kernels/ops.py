@@ -84,6 +84,14 @@ def _ok(code: int, what: str) -> None:
 _fn_cache: dict[tuple[str, str], object] = {}
 
 
+def _slots(state: torch.Tensor, who: str) -> tuple[int, int]:
+    """(slots, floats from one slot to the next) of state slots, which may be a block of columns of wider ones."""
+    _check(state, "state", F32, (None, None), contiguous=False)
+    if state.stride(1) != 1 or (state.shape[0] > 1 and state.stride(0) < state.shape[1]):
+        raise KernelError(f"{who}: slots are dense rows")
+    return state.shape[0], state.stride(0) if state.shape[0] > 1 else state.shape[1]
+
+
 def _fn(module: str, name: str, argtypes: list):
     key = (module, name)
     f = _fn_cache.get(key)
@@ -2003,7 +2011,7 @@ def linmem_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, decay: torch.
         if gate_bias is not None:
             raise KernelError("linmem_scan: a gate bias goes with gates (tau)")
     _check(out, "out", F32, (n, H * dv))
-    _check(state, "state", F32, (None, None))
+    slots = _slots(state, "linmem_scan")
     if state.shape[1] < H * dk * dv or not 0 < dk <= 256 or dv <= 0:
         raise KernelError(f"linmem_scan: heads of {dk} x {dv} (key size at most 256) need slots of {H * dk * dv} floats")
     for t, name in ((cu_q, "cu_q"), (positions, "positions"), (slot_ids, "slot_ids")):
@@ -2015,8 +2023,8 @@ def linmem_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, decay: torch.
     common = (_tcode(q.dtype), q.data_ptr(), k.data_ptr(), v.data_ptr(), decay.data_ptr(),
               gate_bias.data_ptr() if gate_bias is not None else None, cos_p, sin_p, rot, table_len,
               cu_q.data_ptr(), positions.data_ptr(),
-              slot_ids.data_ptr(), state.data_ptr(), out.data_ptr(), int(n_seqs), H, dk, dv, state.shape[0],
-              state.shape[1], stride(q, H * dk), stride(k, H * dk), stride(v, H * dv), 1 if gated else 0,
+              slot_ids.data_ptr(), state.data_ptr(), out.data_ptr(), int(n_seqs), H, dk, dv, *slots,
+              stride(q, H * dk), stride(k, H * dk), stride(v, H * dv), 1 if gated else 0,
               (decay.stride(0) if n > 1 else decay.shape[1]) if gated else 0,
               1.0 / float(tau) if gated else 1.0, float(q_scale), float(k_scale))
     types = [c_int] + [c_void_p] * 7 + [c_int] * 2 + [c_void_p] * 5 + [c_int] * 11 + [c_float] * 3
@@ -2108,14 +2116,6 @@ def ssm_scratch(n_tokens: int, n_chunks: int, heads: int, key_dim: int, value_di
     return out
 
 
-def _slots(state: torch.Tensor, who: str) -> tuple[int, int]:
-    """(slots, floats from one slot to the next) of state slots, which may be a block of columns of wider ones."""
-    _check(state, "state", F32, (None, None), contiguous=False)
-    if state.stride(1) != 1 or (state.shape[0] > 1 and state.stride(0) < state.shape[1]):
-        raise KernelError(f"{who}: slots are dense rows")
-    return state.shape[0], state.stride(0) if state.shape[0] > 1 else state.shape[1]
-
-
 def ssm_conv(rows: torch.Tensor, col0: int, weight: torch.Tensor, bias: torch.Tensor | None, cu_q: torch.Tensor,
              positions: torch.Tensor, slot_ids: torch.Tensor, state: torch.Tensor, state_off: int, out: torch.Tensor,
              n_seqs: int, longest: int, unit: int = 0, key_dim: int = 0, q_scale: float = 1.0) -> None:
@@ -2189,7 +2189,7 @@ def ssm_scan(rows: torch.Tensor, q_off: int, k_off: int, v_off: int, gates: torc
         if delta:
             raise KernelError("ssm_scan: no skip beside the delta rule")
     _check(out, "out", F32, (n, H * dv))
-    _check(state, "state", F32, (None, None))
+    slots = _slots(state, "ssm_scan")
     if state.shape[1] < H * dk * dv:
         raise KernelError(f"ssm_scan: heads of {dk} x {dv} need slots of {H * dk * dv} floats")
     for t, name in ((cu_q, "cu_q"), (positions, "positions"), (slot_ids, "slot_ids")):
@@ -2200,7 +2200,7 @@ def ssm_scan(rows: torch.Tensor, q_off: int, k_off: int, v_off: int, gates: torc
               int(v_off), gates.data_ptr(), gates.stride(0) if n > 1 else gates.shape[1], int(a_off),
               int(b_off) if delta else 0, neg_a.data_ptr(), dt_bias.data_ptr(),
               skip.data_ptr() if skip is not None else None, positions.data_ptr(), slot_ids.data_ptr(),
-              state.data_ptr(), state.shape[0], state.shape[1], out.data_ptr(), H, G, dk, dv)
+              state.data_ptr(), *slots, out.data_ptr(), H, G, dk, dv)
     types = ([c_int, c_void_p] + [c_int] * 4 + [c_void_p] + [c_int] * 3 + [c_void_p] * 6 + [c_int] * 2 + [c_void_p]
              + [c_int] * 4)
     if short_runs or multi is None:

@@ -157,6 +157,7 @@ class PagedAttention(Mixer):
              "g": "g_proj.weight"}
 
     replayable = True
+    shares_slot = True
     settles_residual = True  # its norm kernel adds what is owed to the stream
 
     def __init__(self, prefix: str, hidden: int, num_heads: int, num_kv_heads: int, head_dim: int,

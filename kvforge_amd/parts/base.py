@@ -208,6 +208,8 @@ class Mixer(Part):
 
     cache_spec: CacheSpec | None = None
     state_spec: StateSpec | None = None
+    # whether ``LayerState.state`` may be a block of columns of wider slots (``[slots, floats]``, dense rows)
+    shares_slot = False
 
     def forward(self, x: torch.Tensor, step: "Step", layer: LayerState,
                 residual: torch.Tensor) -> None:

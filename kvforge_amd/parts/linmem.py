@@ -42,6 +42,7 @@ class LinearMemory(Mixer):
              "norm": "norm"}
 
     replayable = True
+    shares_slot = True
     cache_spec = None
 
     def __init__(self, prefix: str, hidden: int, heads: int, dim: int, vdim: int, norm_eps: float,

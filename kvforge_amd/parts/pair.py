@@ -41,6 +41,8 @@ class MixerPair(Mixer):
         # where the right one's numbers begin in a slot that both use (on 16 bytes)
         self.right_off = 0
         if left.state_spec is not None and right.state_spec is not None:
+            if not (left.shares_slot and right.shares_slot):
+                raise ValueError("two mixers side by side that both keep a state must take a block of columns of a slot")
             self.right_off = -(-_floats(left.state_spec) // 4) * 4
 
     @property

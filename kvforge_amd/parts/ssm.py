@@ -42,6 +42,7 @@ class ConvMemory(Mixer):
     the gates' columns (``a_off``, ``b_off``) and what becomes of the read-out (``finish``)."""
 
     replayable = True
+    shares_slot = True
     cache_spec = None
 
     b_off: int | None = None     # column of the delta rule's gates, ``None`` for plain writes

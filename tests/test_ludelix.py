@@ -13,7 +13,7 @@ from kvforge_amd import registry
 from kvforge_amd.config import ConfigError, LudelixConfig
 from kvforge_amd.config.presets import PRESETS, ludelix as make_config
 from kvforge_amd.models.transformer import Transformer
-from kvforge_amd.parts import (LinearMemory, MixerPair, NamedRMSNorm, PagedAttention, PlainFeedForward,
+from kvforge_amd.parts import (LinearMemory, MatrixLSTM, MixerPair, NamedRMSNorm, PagedAttention, PlainFeedForward,
                                PreNormBlock, RoutedExperts)
 from kvforge_amd.weights.random_init import random_tensors
 from tests.plain import ludelix as plain
@@ -117,8 +117,11 @@ def test_parts_refuse_what_their_kernels_do_not_compute():
     with pytest.raises(ValueError, match="only one of them may keep pages"):
         MixerPair(att, PagedAttention("b", 32, 2, 1, 16, None))
     mem = LinearMemory("m", 32, 2, 16, 16, 1e-5, head_decays=[0.9, 0.8])
-    with pytest.raises(ValueError, match="only one of them may keep a state"):
-        MixerPair(mem, LinearMemory("n", 32, 2, 16, 16, 1e-5, head_decays=[0.9, 0.8]))
+    # two states lie in one slot, one behind the other
+    pair = MixerPair(mem, LinearMemory("n", 32, 2, 16, 16, 1e-5, head_decays=[0.9, 0.8]))
+    assert pair.state_spec.shape == (mem.state_spec.shape[0] + 2 * 16 * 16,)
+    with pytest.raises(ValueError, match="must take a block of columns"):
+        MixerPair(mem, MatrixLSTM("n", 32, 2, 16, 16, 15.0, 1e-5))
     with pytest.raises(ValueError, match="no identity outputs"):
         RoutedExperts("f", 32, 16, 4, 2, identity=1, table_vocab=10)
 
