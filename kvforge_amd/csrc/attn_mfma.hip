@@ -256,6 +256,7 @@ template <int RT> struct Rows {
   int pos[RT];         // the row's own position; with slope2, only for kernels with BIAS
   float slope2[RT];    // the head's slope in log2 units
   int drow[RT];        // the head's row in the table of biases by distance (BIAS 4 alone)
+  float far[RT];       // its last entry in log2 units, the bias of every distance beyond the table
 };
 
 // One key block for the row tiles of a wave: scores, lazy softmax update, P * V.
@@ -269,7 +270,8 @@ __device__ __forceinline__ void block_update(const bf16x8 (&kf)[2][(DT + 1) / 2]
                                              const bf16x8 (&qf)[RT][(DT + 1) / 2], const Rows<RT>& rows,
                                              int kb, int kg, bool edge, float scale_log2, float (&m_ref)[RT], float (&l_run)[RT],
                                              f32x4 (&acc)[RT][DT], float cap = 0.f,
-                                             const DistTable& dist = DistTable{nullptr, nullptr, 0}) {
+                                             const DistTable& dist = DistTable{nullptr, nullptr, 0},
+                                             int pos_min = 0) {
   constexpr int DC = (DT + 1) / 2;
   const float scale2 = BIAS != 0 ? 1.f : scale_log2;
   f32x4 s[RT][2];
@@ -319,7 +321,12 @@ __device__ __forceinline__ void block_update(const bf16x8 (&kf)[2][(DT + 1) / 2]
 #pragma unroll
     for (int rt = 0; rt < RT; ++rt) {
       float b[8];
-      dist_eight(dist, rows.drow[rt], rows.pos[rt] - (kb + 8 * kg), b);
+      if (pos_min - (kb + 31) >= dist.n - 1) {      // the whole block lies beyond the table, for all rows of the wave
+#pragma unroll
+        for (int j = 0; j < 8; ++j) b[j] = rows.far[rt];
+      } else {
+        dist_eight(dist, rows.drow[rt], rows.pos[rt] - (kb + 8 * kg), b);
+      }
 #pragma unroll
       for (int t = 0; t < 2; ++t)
 #pragma unroll
@@ -477,7 +484,10 @@ __global__ __launch_bounds__(256) KVF_VGPR_FORM(DT <= 8) void attn_mfma_runs_ker
   if constexpr (SCORE == 4) {
 #pragma unroll
     for (int rt = 0; rt < RT; ++rt)
+    {
       rows.drow[rt] = a.dist_lds ? (rows.head[rt] - kvh * G) * dist_row(a.n_dist) : rows.head[rt] * a.n_dist;
+      rows.far[rt] = a.dist[static_cast<size_t>(rows.head[rt]) * a.n_dist + a.n_dist - 1] * LOG2E;
+    }
   }
   // key range of this wave, and of the workgroup (tiles wg_tile .. wg_tile + 4*RT - 1)
   int lo_w = 0, hi_w = -1;
@@ -588,7 +598,7 @@ __global__ __launch_bounds__(256) KVF_VGPR_FORM(DT <= 8) void attn_mfma_runs_ker
 #pragma unroll
         for (int t = 0; t < DT; ++t) vf[t] = as_frag(frag_lds[(buf * N_FRAG + N_K + t) * KVF_WAVE + lane]);
         const bool edge = kb + 31 > pos_min || kb + 32 > ctx || a.window > 0 || CHUNK;
-        block_update<DT, RT, SCORE>(kf, vf, qf, rows, kb, kg, edge, scale2, m_ref, l_run, acc, a.cap, dist);
+        block_update<DT, RT, SCORE>(kf, vf, qf, rows, kb, kg, edge, scale2, m_ref, l_run, acc, a.cap, dist, pos_min);
       }
     };
     const int kb_first = wk.first;
@@ -672,7 +682,7 @@ __global__ __launch_bounds__(256) KVF_VGPR_FORM(DT <= 8) void attn_mfma_runs_ker
 #pragma unroll
       for (int t = 0; t < DT; ++t) vf[t] = as_frag(keep_first(vr[t], vl));
       const bool edge = kb + 31 > pos_min || kb + 32 > ctx || a.window > 0 || CHUNK;
-      block_update<DT, RT, SCORE>(kf, vf, qf, rows, kb, kg, edge, scale2, m_ref, l_run, acc, a.cap, dist);
+      block_update<DT, RT, SCORE>(kf, vf, qf, rows, kb, kg, edge, scale2, m_ref, l_run, acc, a.cap, dist, pos_min);
     }
   }
 
@@ -738,6 +748,7 @@ __global__ __launch_bounds__(NW * KVF_WAVE) KVF_VGPR_FORM(DT <= 6) void attn_mfm
   if constexpr (BIAS == 4) {
     rows.drow[0] = !rows.ok[0] ? 0 : a.dist_lds ? (rows.head[0] - kvh * G - tile * 16) * dist_row(a.n_dist)
                                                 : rows.head[0] * a.n_dist;
+    rows.far[0] = a.dist[static_cast<size_t>(rows.ok[0] ? rows.head[0] : 0) * a.n_dist + a.n_dist - 1] * LOG2E;
     if (a.dist_lds) __syncthreads();
   }
   if (a.window < 0 && rows.ok[0]) {   // chunks of positions: the rows see from their chunk's first key
@@ -799,7 +810,7 @@ __global__ __launch_bounds__(NW * KVF_WAVE) KVF_VGPR_FORM(DT <= 6) void attn_mfm
 #pragma unroll
     for (int t = 0; t < DT; ++t) vf[t] = as_frag(keep_first(r.v[t], r.vl));
     const bool edge = kb + 31 > pos_min || kb + 32 > ctx || a.window != 0;
-    block_update<DT, 1, BIAS>(kf, vf, qf, rows, kb, kg, edge, scale2, m_ref, l_run, acc, a.cap, dist);
+    block_update<DT, 1, BIAS>(kf, vf, qf, rows, kb, kg, edge, scale2, m_ref, l_run, acc, a.cap, dist, pos_min);
   };
   // Without a window the page lookups of the first blocks are asked for together with the
   // query and the context length, not after them: one round trip to memory less.

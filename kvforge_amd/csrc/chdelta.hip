@@ -40,6 +40,15 @@ struct ChArgs {
   int chunk_from;                   // runs of at least so many tokens go chunk by chunk
 };
 
+// A key channel's decay exp(-A softplus(z)), neg_a = -A.  With x = e^-|z| and u = 1 + x rounded, log1p(x) =
+// log(u) x / (u - 1), which keeps small x whole: a channel that hardly fades has softplus(z) ~ x far below the
+// rounding of 1 + x.  (The hardware's exponential and logarithm: within an ulp or so.)
+__device__ __forceinline__ float decay_of(float z, float neg_a) {
+  const float x = __expf(-fabsf(z)), u = 1.f + x, d = u - 1.f;
+  const float l = d == 0.f ? x : __logf(u) * __fdividef(x, d);
+  return __expf(neg_a * (fmaxf(z, 0.f) + l));
+}
+
 constexpr int SCAN_STAGE = 8;      // tokens staged in LDS at a time
 
 // Workgroup (64 value columns, head, sequence) of ceil(dk / ROWS) waves.  Lane l of a wave keeps row l's
@@ -88,7 +97,7 @@ __global__ __launch_bounds__(256) void chdelta_scan_kernel(const float* __restri
       const float* row = rows + static_cast<size_t>(tb + t) * a.ld + kh * dk + e;
       qs[i] = row[a.q_off];
       ks[i] = row[a.k_off];
-      as[i] = expf(na * softplus(z[static_cast<size_t>(tb + t) * a.z_ld + a.a_off + head * dk + e] + db[e]));
+      as[i] = decay_of(z[static_cast<size_t>(tb + t) * a.z_ld + a.a_off + head * dk + e] + db[e], na);
     }
     for (int i = threadIdx.x; i < cnt * KVF_WAVE; i += blockDim.x) {
       const int t = i / KVF_WAVE, c = blockIdx.x * KVF_WAVE + i % KVF_WAVE;
@@ -200,7 +209,7 @@ __global__ __launch_bounds__(DKP * (CL / 16)) void chdelta_solve_kernel(
       const bool in = 16 * sub + j < cnt;
       q[j] = in && ch_ok ? q[j] : 0.f;
       k[j] = in && ch_ok ? k[j] : 0.f;
-      pre[j] = in ? expf(na * softplus(pre[j] + db)) : 1.f;
+      pre[j] = in ? decay_of(pre[j] + db, na) : 1.f;
       suf[j] = 1.f;
     }
   }
@@ -363,7 +372,9 @@ struct RowArgs {
   int ld, dk;
 };
 
-// runs: rows (sequence, first chunk, chunks).  Workgroup (16 value columns, head, run).  A chunk's Kd, Kw, T, V
+// runs: rows (sequence, first chunk, chunks).  Workgroup (head, 16 value columns, run): the heads are the grid's
+// fastest index, so with eight heads or a multiple the slices of a head, which read the same Kd, Kw and T, lie on
+// one XCD and find them in its L2.  A chunk's Kd, Kw, T, V
 // and P(0, L) are asked for while the chunk before is worked on.  W [chunks, H, dk, dv] receives the state
 // before every chunk, U [tokens, H, dv] the chunks' u.
 constexpr int DCOLS = 16;
@@ -386,7 +397,7 @@ __global__ __launch_bounds__(256) void chdelta_delta_kernel(
   float* Rt = Vt + DCOLS * TLD;                  // [DCOLS][TLD]
   float* Ut = Rt + DCOLS * TLD;                  // [DCOLS][TLD]
   float* St = Ut + DCOLS * TLD;                  // [DCOLS][QLD]
-  const int head = blockIdx.y, col0 = blockIdx.x * DCOLS;
+  const int head = blockIdx.x, col0 = blockIdx.y * DCOLS;
   const int seq = runs[3 * blockIdx.z], c0 = runs[3 * blockIdx.z + 1], nc = runs[3 * blockIdx.z + 2];
   const int tid = threadIdx.x, lane = tid % KVF_WAVE, wave = tid / KVF_WAVE, l16 = lane % 16, lq = lane / 16;
   const int dk = a.dk, dv = a.dv;
@@ -498,7 +509,7 @@ __global__ __launch_bounds__(256) void chdelta_delta_kernel(
   }
 }
 
-// Workgroup of eight waves (64 value columns, head, chunk): O = A U + Qd S0.  Wave w has the chunk's rows
+// Workgroup of eight waves (head, 64 value columns, chunk): O = A U + Qd S0.  Wave w has the chunk's rows
 // 16 (w % RT) .. + 15, whose Qd it keeps in registers.
 constexpr int VCOLS = 64;
 template <int DKP, int CL> constexpr size_t read_lds() {
@@ -513,7 +524,7 @@ __global__ __launch_bounds__(512, DKP <= 128 ? 4 : 2) void chdelta_read_kernel(
   float* Sc = lds;                               // [VCOLS][QLD] the state's columns
   float* As = Sc + VCOLS * QLD;                  // [CL][TLD]
   float* Ut = As + CL * TLD;                     // [VCOLS][TLD]
-  const int chunk = blockIdx.z, head = blockIdx.y, col0 = blockIdx.x * VCOLS;
+  const int chunk = blockIdx.z, head = blockIdx.x, col0 = blockIdx.y * VCOLS;
   const int tb = chunks[4 * chunk + 1], cnt = chunks[4 * chunk + 2];
   const int tid = threadIdx.x, lane = tid % KVF_WAVE, wave = tid / KVF_WAVE, l16 = lane % 16, lq = lane / 16;
   const int dk = a.dk, dv = a.dv, rt = wave % RT, share = wave / RT;
@@ -582,10 +593,10 @@ template <int DKP, int CL, bool VEC> int chunks_go(const ChunkPtrs& p, ChArgs a,
   }
   hipLaunchKernelGGL((chdelta_solve_kernel<DKP, CL>), dim3(a.H, p.n_chunks), dim3(solve_threads<DKP, CL>()), lds_solve, s,
                      p.rows, p.z, p.zb, p.neg_a, p.dt_bias, p.chunks, p.T, p.A, p.E, p.Kd, p.Kw, p.Qd, a);
-  hipLaunchKernelGGL((chdelta_delta_kernel<DKP, CL, VEC>), dim3((a.dv + DCOLS - 1) / DCOLS, a.H, p.n_runs), dim3(256),
+  hipLaunchKernelGGL((chdelta_delta_kernel<DKP, CL, VEC>), dim3(a.H, (a.dv + DCOLS - 1) / DCOLS, p.n_runs), dim3(256),
                      lds_delta, s, p.rows, p.chunks, p.runs, p.positions, p.slot_ids, p.state, p.T, p.E, p.Kd, p.Kw, p.W,
                      p.U, a);
-  hipLaunchKernelGGL((chdelta_read_kernel<DKP, CL, VEC>), dim3((a.dv + VCOLS - 1) / VCOLS, a.H, p.n_chunks), dim3(512),
+  hipLaunchKernelGGL((chdelta_read_kernel<DKP, CL, VEC>), dim3(a.H, (a.dv + VCOLS - 1) / VCOLS, p.n_chunks), dim3(512),
                      lds_read, s, p.chunks, p.Qd, p.A, p.W, p.U, p.out, a);
   return kvf_last_error();
 }
@@ -594,7 +605,7 @@ bool args_ok(const ChArgs& a) {
   return a.H > 0 && a.G > 0 && a.H % a.G == 0 && a.H <= 65535 && a.dk > 0 && a.dk <= 256 && a.dv > 0 &&
          a.q_off >= 0 && a.k_off >= 0 && a.v_off >= 0 && a.q_off + a.G * a.dk <= a.ld && a.k_off + a.G * a.dk <= a.ld &&
          a.v_off + a.H * a.dv <= a.ld && a.a_off >= 0 && a.a_off + a.H * a.dk <= a.z_ld && a.b_off >= 0 &&
-         a.b_off + a.H <= a.b_ld && static_cast<long>(a.slot_stride) >= static_cast<long>(a.H) * a.dk * a.dv;
+         a.b_off + a.H <= a.b_ld && a.dv <= 65535 && static_cast<long>(a.slot_stride) >= static_cast<long>(a.H) * a.dk * a.dv;
 }
 }  // namespace
 

@@ -11,9 +11,9 @@
 // zero): H q heads, KV k heads, KV v heads.  P = 4 .. 64 lanes share a head, four neighbouring
 // elements each.  A run is cut into tiles of TT tokens at multiples of TT *positions*, so that a
 // tile's values lie side by side in one (transposed) V page where a page's size is a multiple of
-// TT; only the first two tiles of a run can reach back into the slot (taps - 1 < TT), so one
-// workgroup takes both, and each of its threads alone reads and rewrites the slot's numbers of its
-// channels.
+// TT; a workgroup takes two tiles.  Only the first two tiles of a run can reach back into the slot
+// (taps - 1 < TT), so they are one workgroup's, and each of its threads alone reads and rewrites the
+// slot's numbers of its channels.  The weights lie [taps][C].
 #include "common.h"
 
 namespace {
@@ -56,7 +56,7 @@ template <int TT> __device__ __forceinline__ void store_run(bf16_t* p, const flo
                                                   two(y[i + 4][e], y[i + 5][e]), two(y[i + 6][e], y[i + 7][e]));
 }
 
-// Grid (shares of the heads, tiles, sequences).  TT = 1: every run of the launch is one token.
+// Grid (shares of the heads, pairs of tiles, sequences).  TT = 1: every run of the launch is one token.
 template <typename T, int TAPS, int TT>
 __global__ __launch_bounds__(256) void conv_norm_kvwrite_kernel(
     const T* __restrict__ rows, const float* __restrict__ w, const float* __restrict__ qw, const float* __restrict__ kw,
@@ -69,7 +69,7 @@ __global__ __launch_bounds__(256) void conv_norm_kvwrite_kernel(
   if (len <= 0) return;
   const int p0 = positions[run0];
   const int lead = TT > 1 && p0 > 0 ? p0 % TT : 0;          // positions of the first tile that lie before the run
-  const int first_tile = blockIdx.y == 0 ? 0 : blockIdx.y + 1, last_tile = blockIdx.y + 1;
+  const int first_tile = 2 * blockIdx.y, last_tile = first_tile + 1;
   if (first_tile * TT - lead >= len) return;
   const int group = threadIdx.x / P, lane = threadIdx.x % P;
   const int head = blockIdx.x * (256 / P) + group;          // of H + 2 KV
@@ -79,9 +79,7 @@ __global__ __launch_bounds__(256) void conv_norm_kvwrite_kernel(
   const T* src = rows + c;
   float wt[TAPS][4];
 #pragma unroll
-  for (int e = 0; e < 4; ++e)
-#pragma unroll
-    for (int j = 0; j < TAPS; ++j) wt[j][e] = w[static_cast<size_t>(c + e) * TAPS + j];
+  for (int j = 0; j < TAPS; ++j) load4(w + static_cast<size_t>(j) * C + c, wt[j]);
   float old[K > 0 ? K : 1][4] = {};
   float* st = nullptr;
   if (K > 0 && blockIdx.y == 0) {
@@ -218,7 +216,7 @@ int go(const void* rows, const float* w, const float* qw, const float* kw, const
   const int shares = (a.H + 2 * a.KV + 256 / P - 1) / (256 / P);
   const int tiles = longest == 1 ? 1 : (longest + TILE - 1 + TILE - 1) / TILE;
 #define GO(TT)                                                                                                        \
-  hipLaunchKernelGGL((conv_norm_kvwrite_kernel<T, TAPS, TT>), dim3(shares, tiles > 1 ? tiles - 1 : 1, a.n_seqs),     \
+  hipLaunchKernelGGL((conv_norm_kvwrite_kernel<T, TAPS, TT>), dim3(shares, (tiles + 1) / 2, a.n_seqs),               \
                      dim3(256), 0, s, static_cast<const T*>(rows), w, qw, kw, cu_q, positions, slot_ids, block_table, \
                      state, static_cast<T*>(q_out), static_cast<T*>(k_pages), static_cast<T*>(v_pages), P, a)
   if (longest == 1) GO(1);
@@ -228,7 +226,7 @@ int go(const void* rows, const float* w, const float* qw, const float* kw, const
 }
 }  // namespace
 
-// dtype: 0 = fp32, 1 = bf16 (rows, q_out and pages).  rows [n, ld]: (H + 2 KV) heads of d; w [(H + 2 KV) d, taps]
+// dtype: 0 = fp32, 1 = bf16 (rows, q_out and pages).  rows [n, ld]: (H + 2 KV) heads of d; w [taps, (H + 2 KV) d]
 // fp32; qw, kw: null, or [dk] fp32 (with norm).  longest: tokens of the longest run.  ld, ldq, slot_stride and d are
 // multiples of 4, and rows, q_out, pages and state start on 16 bytes (what the host checks).
 KVF_EXPORT int kvf_conv_norm_kvwrite(int dtype, const void* rows, int ld, int taps, const float* w, int norm, int dk,

@@ -521,7 +521,7 @@ def conv_norm_kvwrite(rows: torch.Tensor, weight: torch.Tensor, cu_q: torch.Tens
                       n_seqs: int, longest: int, norm_dim: int | None = None, eps: float = 0.0,
                       q_weight: torch.Tensor | None = None, k_weight: torch.Tensor | None = None) -> None:
     """A short causal convolution over time on every channel of the projected q, k and v heads
-    (``rows [n, >= (H + 2 KV) d]``; ``weight`` fp32 ``[(H + 2 KV) d, taps]``, whose last tap meets the token itself), then with
+    (``rows [n, >= (H + 2 KV) d]``; ``weight`` fp32 ``[taps, (H + 2 KV) d]``, whose last row meets the token itself), then with
     ``norm_dim`` an RMS norm of every q and k head over its first ``norm_dim`` elements (the others are zero; optional
     weights ``[norm_dim]`` that the heads share), then q to ``q_out [n, H d]`` and k and v to the pages; fp32 with one
     rounding.  What lies before a run is read from the sequence's slot (``taps - 1`` rows of all channels, the
@@ -529,11 +529,11 @@ def conv_norm_kvwrite(rows: torch.Tensor, weight: torch.Tensor, cu_q: torch.Tens
     wider slots (``None`` with one tap).  ``longest``: tokens of the longest run."""
     n = rows.shape[0]
     H, KV, d = int(num_heads), int(num_kv_heads), int(head_dim)
-    C, taps = weight.shape
+    taps, C = weight.shape
     _check(rows, "rows", None, (n, None), contiguous=False)
     if rows.stride(1) != 1 or rows.shape[1] < (H + 2 * KV) * d or (n > 1 and rows.stride(0) % 4) or rows.data_ptr() % 16:
         raise KernelError("conv_norm_kvwrite: dense rows that hold q, k and v and start on 16 bytes")
-    _check(weight, "weight", F32, ((H + 2 * KV) * d, taps))
+    _check(weight, "weight", F32, (taps, (H + 2 * KV) * d))
     if not 1 <= taps <= CONVKV_MAX_TAPS or d % 16 or not 0 < d <= 256:
         raise KernelError(f"conv_norm_kvwrite: 1 to {CONVKV_MAX_TAPS} taps and heads in steps of 16 up to 256, got {taps} and {d}")
     if norm_dim is not None and not 0 < norm_dim <= d:

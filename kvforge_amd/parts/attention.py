@@ -315,7 +315,7 @@ class PagedAttention(Mixer):
             self.conv_w = torch.cat([
                 self._padded_heads(tensors[self._conv_name(key)].float(), heads, size)
                 for key, heads, size in (("q", self.H, self.dk), ("k", self.KV, self.dk), ("v", self.KV, self.dv))],
-                dim=0).contiguous()
+                dim=0).t().contiguous()          # [taps, channels]
         if self.distance_bias is not None:
             name, far = self._name(self.distance_bias[0]), self.distance_bias[1]
             self.dist = distance_table(tensors[name], float(far))

@@ -94,7 +94,7 @@ def test_convolved_q_k_and_v_over_runs_steps_and_slots(dtype, taps, H, KV, d, dk
         rows = torch.cat([xs[s][a:e] for s, a, e in parts])
         wide = torch.cat([rows, torch.full((len(rows), 8), 9.0)], dim=1).to(dtype).to(DEV)
         q = torch.full((len(rows), H * d), 7.0, dtype=dtype, device=DEV)
-        ops().conv_norm_kvwrite(wide, w.to(DEV), i32([0] + list(np.cumsum([e - a for _, a, e in parts]))),
+        ops().conv_norm_kvwrite(wide, w.t().contiguous().to(DEV), i32([0] + list(np.cumsum([e - a for _, a, e in parts]))),
                                 i32([p for _, a, e in parts for p in range(a, e)]), i32([slots[s] for s, _, _ in parts]),
                                 state[:, 4:4 + (taps - 1) * C] if taps > 1 else None,
                                 table[[s for s, _, _ in parts]].contiguous().to(DEV), q, k_pages, v_pages, H, KV, d,
@@ -292,6 +292,32 @@ def test_channels_that_are_kept_and_channels_that_are_dropped():
     for t in range(3, n):
         want = torch.zeros(dv) if (t + 1) % 4 == 2 else v[t - 3]
         torch.testing.assert_close(got[t], want, atol=1e-4, rtol=1e-4)
+
+
+@pytest.mark.parametrize("runs", [[400], [20] * 20])
+def test_decays_are_exact_enough_to_hold_over_hundreds_of_tokens(runs):
+    """One channel per head, written once and left to fade: what is left after t tokens is the decay to the power
+    of t, for pre-activations from channels that all but never fade to ones that are gone at once; chunk by chunk and
+    token by token."""
+    H, n = 61, sum(runs)
+    z = torch.linspace(-18.0, 12.0, H)
+    neg_a = -torch.exp(torch.linspace(-3.0, 1.0, H))[torch.randperm(H, generator=torch.Generator().manual_seed(1))]
+    q, k, v = torch.ones(n, H, 1), torch.ones(n, H, 1), torch.ones(n, H, 1)
+    zb = torch.full((n, H), -200.0)
+    zb[0] = 200.0
+    state = torch.zeros(1, H, device=DEV)
+    got, at = [], 0
+    for r in runs:
+        part = slice(at, at + r)
+        got.append(run_memory(q[part].view(r, H), k[part].view(r, H), v[part].view(r, H), z.expand(r, H).contiguous(), zb[part],
+                              neg_a, torch.zeros(H), [r], state, [0], list(range(at, at + r)), H, H, 1, 1))
+        at += r
+    rate = neg_a.double() * plain.softplus(z.double())
+    want = torch.exp(torch.arange(n, dtype=torch.float64)[:, None] * rate[None, :])
+    # a relative error of 3e-7 (and of the exponent's own rounding) a token
+    allowed = 1e-6 + torch.arange(n)[:, None] * (3e-7 + 3e-7 * rate.abs()[None, :]) * want
+    err = (torch.cat(got).double() - want).abs()
+    assert bool((err <= allowed + 1e-30).all()), (float((err / allowed).max()), int((err / allowed).amax(0).argmax()))
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
